@@ -1,175 +1,15 @@
-// engine.hip -- libpgmi host side: weight layout, workspaces, forward orchestration, hipGraph
-// decode, and the extern "C" ABI declared in include/pgmi.h.
+// engine.hip -- the PaliGemma family of libpgmi: weight layout, workspaces, forward orchestration, hipGraph
+// decode, and its extern "C" entry points of include/pgmi.h.
 //
 // Orchestration restates the reference's call stacks:
 //   vision   SiglipVisionTransformer.forward   modeling_siglip.py:236-244
 //   lm       GemmaModel/GemmaForCausalLM        modeling_gemma.py:357-427
 //   decode   one inference.py loop iteration    inference.py:56-78
-#include <algorithm>
-#include <cmath>
-#include <cstdio>
-#include <cstdlib>
-#include <cstring>
-#include <map>
-#include <string>
-#include <tuple>
-#include <unordered_map>
-#include <vector>
-
-#include <dlfcn.h>
-
-#include <rccl/rccl.h>  // types only: librccl is dlopen'ed on first use
-
-#include "../../include/pgmi.h"
-#include "common.h"
-#include "launch.h"
-#include "safetensors_hdr.h"
-
-using namespace pgmi;
-
-static thread_local std::string g_err;
-
-static int fail(int code, const std::string& msg) {
-    g_err = msg;
-    return code;
-}
-
-#define HIPCHK(expr)                                                                       \
-    do {                                                                                   \
-        hipError_t e_ = (expr);                                                            \
-        if (e_ != hipSuccess) return fail(PGMI_E_HIP, std::string(#expr) + ": " + hipGetErrorString(e_)); \
-    } while (0)
-
-#define LAUNCHCHK()                                                                        \
-    do {                                                                                   \
-        hipError_t e_ = hipGetLastError();                                                 \
-        if (e_ != hipSuccess) return fail(PGMI_E_HIP, std::string("kernel launch: ") + hipGetErrorString(e_)); \
-    } while (0)
-
-struct Slot {
-    std::string name;
-    int64_t off;
-    int64_t shape[4];
-    int ndim;
-    int64_t numel;
-};
-
-struct GraphKey {
-    int B;
-    void* kv;
-    int kv_batch, kv_max;
-    float* logits;
-    int64_t* next;
-    const int64_t* ids;  // the ids buffer the graph reads (the context's staging copy, or in place)
-    bool emb;            // the step's input is the staged embedding rows (pgmi_decode_embeds), not ids
-    int masked;          // 0: no mask (a zero word), 1: staged bf16 mask (sum rounded), 2: staged fp32 mask
-    int n_steps;         // decode steps captured back to back (pgmi_decode_steps; 1 otherwise)
-    int64_t* tokens;     // their per-step token record ([n_steps][B], may be null)
-    bool operator<(const GraphKey& o) const {
-        return std::tie(B, kv, kv_batch, kv_max, logits, next, ids, emb, masked, n_steps, tokens) <
-               std::tie(o.B, o.kv, o.kv_batch, o.kv_max, o.logits, o.next, o.ids, o.emb, o.masked, o.n_steps,
-                        o.tokens);
-    }
-};
-
-struct GraphEntry {
-    int seen = 0;
-    hipGraphExec_t exec = nullptr;
-};
-
-struct pgmi_ctx {
-    pgmi_config c;
-    int device;
-    std::vector<Slot> slots;
-    std::unordered_map<std::string, int> index;
-    int64_t slab_bytes = 0;
-    uint8_t* slab = nullptr;
-    std::vector<float> inv_freq;
-    std::vector<uint16_t> host_cos, host_sin;  // optional exact table
-    bool prepared = false;
-    std::vector<void*> allocs;
-    // derived
-    uint16_t* patch_w = nullptr;  // [v_hidden][kpad]
-    int kpad = 0;
-    uint16_t* cosT = nullptr;
-    uint16_t* sinT = nullptr;
-    // text prefill workspace (rows = max_batch*max_seq)
-    uint16_t *Hs, *Tn, *QKV, *Qr, *AO, *ACT, *lastrows;
-    long tn_rows = 0;  // rows of Tn holding the final RMSNorm of the last pgmi_lm_forward (pgmi_lm_final_hidden)
-    int64_t* dpos;
-    int64_t* dids_tmp;
-    // vision workspace (rows = max_batch*N)
-    uint16_t *vX, *vT, *vQKV, *vAO, *vH, *vP;
-    float* ws;
-    size_t ws_bytes;
-    // decode workspace
-    uint16_t *dH, *dQ, *dAO, *dACT;
-    uint16_t* dHn;  // batched decode (B >= 3): the RMSNorm'd rows the unstaged MFMA projections read
-    float* dSS;     // batched decode: o_proj's 16-column partial sums of squares of h, [B][H / 16]
-    // batched decode (max_batch >= 3): fragment-major images of every layer's gate|up, q|k|v (in the GEMV's row
-    // order), o_proj and down weights (mf_swizzle), [layer][gate|up 2 I x H | q|k|v QKVN x H | o_proj | down H x I]
-    uint16_t* mfw = nullptr;
-    size_t mfw_layer = 0;
-    bool mfw_dirty = false;  // the fragment-major images are (re)built by the next batched decode step
-    float *opart, *pmax, *dlogits, *amax_v;
-    int *pidx, *amax_i;
-    int max_chunks;
-    StepState* step;
-    StepState* pstep;  // the generate-loop prefill's last-row attention (flash-decoding over the prompt's keys)
-    int64_t* d_ids;
-    uint16_t* d_emb;             // staged input rows of pgmi_decode_embeds ([max_batch][hidden] bf16)
-    float* d_mask;               // staged additive decode mask ([max_batch][max_kv] fp32, pgmi_decode_embeds_dev)
-    float* d_zero;               // one zero word: the "no mask" mask of the decode attention
-    int64_t* d_next;             // argmax target when the caller passes none
-    unsigned* lm_done;           // lm_head arrival counter (argmax folded into its last workgroup)
-    hipStream_t cap_stream = nullptr;
-    std::map<GraphKey, GraphEntry> graphs;
-    // prefill graphs (vision tower, language-model forward): replayed for repeated calls with
-    // identical pointer/shape arguments (a replay is the eager call: kernels read the same
-    // addresses at run time), captured on the second such call
-    bool prefill_graph = true;
-    int mf_staged = -1;  // batched decode RMSNorm form (mf_staged()); -1 = default (unstaged)
-    // device step state as the last enqueued per-phase decode step leaves it (advanced in-graph)
-    bool step_known = false;
-    int step_kv = 0, step_pos = 0;
-    std::map<std::vector<intptr_t>, GraphEntry> pgraphs;
-    // in-situ timing probe of the prefill MLP GEMMs (pgmi_prefill_probe): events around layer i's gate|up
-    // GEMM (ev[4i], ev[4i+1]) and down GEMM (ev[4i+2], ev[4i+3]) of eager forwards
-    std::vector<hipEvent_t> probe_ev;
-    bool probe_on = false;
-    bool graph_before_probe = true;  // prefill_graph as the caller left it before the probe turned it off
-};
+#include "engine.h"
 
 namespace {
 
-void clear_pgraphs(pgmi_ctx* x) {
-    for (auto& kv : x->pgraphs)
-        if (kv.second.exec) (void)hipGraphExecDestroy(kv.second.exec);
-    x->pgraphs.clear();
-}
-
-// the captured decode steps
-void clear_dgraphs(pgmi_ctx* x) {
-    for (auto& kv : x->graphs)
-        if (kv.second.exec) (void)hipGraphExecDestroy(kv.second.exec);
-    x->graphs.clear();
-}
-
 int n_img(const pgmi_config& c) { return (c.v_image / c.v_patch) * (c.v_image / c.v_patch); }
-
-void add_slot(pgmi_ctx* x, const std::string& name, std::initializer_list<int64_t> shape) {
-    Slot s;
-    s.name = name;
-    s.ndim = (int)shape.size();
-    s.numel = 1;
-    int i = 0;
-    for (int64_t d : shape) { s.shape[i++] = d; s.numel *= d; }
-    for (; i < 4; ++i) s.shape[i] = 1;
-    s.off = x->slab_bytes;
-    x->slab_bytes += (s.numel * 2 + 255) / 256 * 256;
-    x->index[name] = (int)x->slots.size();
-    x->slots.push_back(s);
-}
 
 // Slab layout: the reference state-dict tensors, ordered so that the projections that are
 // fused into one GEMM/GEMV are adjacent (q|k|v weights and biases, gate|up).
@@ -215,67 +55,12 @@ void build_layout(pgmi_ctx* x) {
     }
     add_slot(x, "language_model.model.norm.weight", {H});
 }
-
-inline uint16_t* W(pgmi_ctx* x, const std::string& name) {
-    auto it = x->index.find(name);
-    if (it == x->index.end()) return nullptr;
-    return reinterpret_cast<uint16_t*>(x->slab + x->slots[it->second].off);
-}
-
 inline uint16_t* VL(pgmi_ctx* x, int i, const char* suffix) {
     return W(x, "vision_tower.vision_model.encoder.layers." + std::to_string(i) + "." + suffix);
 }
 inline uint16_t* TL(pgmi_ctx* x, int i, const char* suffix) {
     return W(x, "language_model.model.layers." + std::to_string(i) + "." + suffix);
 }
-
-uint16_t host_f2bf(float f) {
-    uint32_t u;
-    std::memcpy(&u, &f, 4);
-    u += 0x7FFFu + ((u >> 16) & 1u);
-    return (uint16_t)(u >> 16);
-}
-
-float bf16_round_host(float f) {
-    uint32_t u = (uint32_t)host_f2bf(f) << 16;
-    float r;
-    std::memcpy(&r, &u, 4);
-    return r;
-}
-
-uint64_t fnv1a(const char* s) {
-    uint64_t h = 0xCBF29CE484222325ULL;
-    for (const unsigned char* p = (const unsigned char*)s; *p; ++p) { h ^= *p; h *= 0x100000001B3ULL; }
-    return h;
-}
-
-uint64_t splitmix64_h(uint64_t x) {
-    x += 0x9E3779B97F4A7C15ULL;
-    x = (x ^ (x >> 30)) * 0xBF58476D1CE4E5B9ULL;
-    x = (x ^ (x >> 27)) * 0x94D049BB133111EBULL;
-    return x ^ (x >> 31);
-}
-
-__global__ void k_convert(const void* src, int dtype, long n, uint16_t* dst) {
-    for (long i = blockIdx.x * (long)blockDim.x + threadIdx.x; i < n; i += (long)gridDim.x * blockDim.x) {
-        if (dtype == PGMI_DTYPE_F32) dst[i] = f2bf(reinterpret_cast<const float*>(src)[i]);
-        else dst[i] = f2bf((float)reinterpret_cast<const _Float16*>(src)[i]);
-    }
-}
-
-int dalloc(pgmi_ctx* x, void** p, size_t bytes) {
-    if (bytes == 0) bytes = 256;
-    hipError_t e = hipMalloc(p, bytes);
-    if (e != hipSuccess) return fail(PGMI_E_NOMEM, std::string("hipMalloc ") + std::to_string(bytes) + ": " + hipGetErrorString(e));
-    x->allocs.push_back(*p);
-    return 0;
-}
-
-template <typename T>
-int dalloc_t(pgmi_ctx* x, T** p, size_t count) {
-    return dalloc(x, reinterpret_cast<void**>(p), count * sizeof(T));
-}
-
 // RoPE tables: freqs = fp32(pos * inv_freq) (modeling_gemma.py:178), cos/sin in fp32 (:182-183),
 // cast to bf16 (:185).  cos/sin of the fp32 angle are evaluated in double and rounded once.
 void build_rope_host(pgmi_ctx* x, std::vector<uint16_t>& cs, std::vector<uint16_t>& sn) {
@@ -290,54 +75,16 @@ void build_rope_host(pgmi_ctx* x, std::vector<uint16_t>& cs, std::vector<uint16_
         }
 }
 
-int ensure_prepared(pgmi_ctx* x) {
-    if (!x->prepared) return fail(PGMI_E_STATE, "pgmi_prepare() has not been called");
-    if (!x->slab) return fail(PGMI_E_STATE, "weights are not bound (pgmi_bind_weights)");
-    return 0;
+int paligemma_prepare(pgmi_ctx* x);
+
+int64_t paligemma_kv_bytes(const pgmi_ctx* x, int batch, int max_tokens) {
+    return (int64_t)x->c.t_layers * 2 * batch * max_tokens * x->c.t_kv_heads * x->c.t_head_dim * 2;
 }
 
 }  // namespace
 
 // ================================================================ C ABI
-// RCCL is loaded on first use (dlopen), so a single-GPU process -- and the CPU tests that only load
-// the library -- need no librccl; the four entry points it uses are resolved once.
-namespace {
-struct Rccl {
-    void* h = nullptr;
-    std::string why;  // dlerror() of the failed load
-    ncclResult_t (*get_unique_id)(ncclUniqueId*) = nullptr;
-    ncclResult_t (*comm_init_rank)(ncclComm_t*, int, ncclUniqueId, int) = nullptr;
-    ncclResult_t (*comm_destroy)(ncclComm_t) = nullptr;
-    ncclResult_t (*broadcast)(const void*, void*, size_t, ncclDataType_t, int, ncclComm_t, hipStream_t) = nullptr;
-    const char* (*error_string)(ncclResult_t) = nullptr;
-};
-
-// thread-safe one-time load (a function-local static is initialised exactly once)
-Rccl& rccl() {
-    static Rccl r = [] {
-        Rccl t;
-        for (const char* n : {"librccl.so.1", "librccl.so", "/opt/rocm/lib/librccl.so.1"}) {
-            if ((t.h = dlopen(n, RTLD_NOW | RTLD_LOCAL))) break;
-            const char* e = dlerror();
-            if (e) t.why = e;
-        }
-        if (t.h) {
-            t.get_unique_id = reinterpret_cast<decltype(t.get_unique_id)>(dlsym(t.h, "ncclGetUniqueId"));
-            t.comm_init_rank = reinterpret_cast<decltype(t.comm_init_rank)>(dlsym(t.h, "ncclCommInitRank"));
-            t.comm_destroy = reinterpret_cast<decltype(t.comm_destroy)>(dlsym(t.h, "ncclCommDestroy"));
-            t.broadcast = reinterpret_cast<decltype(t.broadcast)>(dlsym(t.h, "ncclBroadcast"));
-            t.error_string = reinterpret_cast<decltype(t.error_string)>(dlsym(t.h, "ncclGetErrorString"));
-        }
-        return t;
-    }();
-    return r;
-}
-}  // namespace
-
 extern "C" {
-
-const char* pgmi_last_error(void) { return g_err.c_str(); }
-const char* pgmi_version(void) { return "pgmi 0.1.0 (gfx950)"; }
 
 int pgmi_create(int device, const pgmi_config* cfg, pgmi_ctx** out) {
     if (!cfg || !out) return fail(PGMI_E_ARG, "null argument");
@@ -354,6 +101,8 @@ int pgmi_create(int device, const pgmi_config* cfg, pgmi_ctx** out) {
     x->c = c;
     if (x->c.max_kv <= 0) x->c.max_kv = c.t_max_pos;
     x->device = device;
+    x->prepare = paligemma_prepare;
+    x->kv_bytes = paligemma_kv_bytes;
     build_layout(x);
     x->inv_freq.resize(c.t_head_dim / 2);
     for (int i = 0; i < c.t_head_dim / 2; ++i) {
@@ -365,194 +114,6 @@ int pgmi_create(int device, const pgmi_config* cfg, pgmi_ctx** out) {
     *out = x;
     return 0;
 }
-
-int pgmi_destroy(pgmi_ctx* x) {
-    if (x)
-        for (auto& e : x->probe_ev) (void)hipEventDestroy(e);
-    if (!x) return 0;
-    clear_dgraphs(x);
-    clear_pgraphs(x);
-    for (void* p : x->allocs) (void)hipFree(p);
-    if (x->cap_stream) (void)hipStreamDestroy(x->cap_stream);
-    delete x;
-    return 0;
-}
-
-int64_t pgmi_weights_bytes(const pgmi_ctx* x) { return x ? x->slab_bytes : -1; }
-int pgmi_weight_count(const pgmi_ctx* x) { return x ? (int)x->slots.size() : -1; }
-
-int pgmi_weight_info(const pgmi_ctx* x, int idx, const char** name, int64_t* off, int64_t* shape4, int* ndim) {
-    if (!x || idx < 0 || idx >= (int)x->slots.size()) return fail(PGMI_E_ARG, "weight index out of range");
-    const Slot& s = x->slots[idx];
-    if (name) *name = s.name.c_str();
-    if (off) *off = s.off;
-    if (shape4) for (int i = 0; i < 4; ++i) shape4[i] = s.shape[i];
-    if (ndim) *ndim = s.ndim;
-    return 0;
-}
-
-int pgmi_bind_weights(pgmi_ctx* x, void* slab) {
-    if (!x || !slab) return fail(PGMI_E_ARG, "null argument");
-    if (reinterpret_cast<uintptr_t>(slab) % 256 != 0) return fail(PGMI_E_ARG, "weight slab must be 256-byte aligned");
-    x->slab = reinterpret_cast<uint8_t*>(slab);
-    clear_dgraphs(x);
-    clear_pgraphs(x);
-    return 0;
-}
-
-int pgmi_load_weight(pgmi_ctx* x, const char* name, const void* src, int dtype, int on_device, void* stream) {
-    if (!x || !name || !src) return fail(PGMI_E_ARG, "null argument");
-    if (!x->slab) return fail(PGMI_E_STATE, "weights are not bound");
-    auto it = x->index.find(name);
-    if (it == x->index.end()) return fail(PGMI_E_ARG, std::string("unknown weight ") + name);
-    const Slot& s = x->slots[it->second];
-    uint16_t* dst = reinterpret_cast<uint16_t*>(x->slab + s.off);
-    hipStream_t st = (hipStream_t)stream;
-    HIPCHK(hipSetDevice(x->device));
-    if (dtype == PGMI_DTYPE_BF16) {
-        HIPCHK(hipMemcpyAsync(dst, src, s.numel * 2, on_device ? hipMemcpyDeviceToDevice : hipMemcpyHostToDevice, st));
-    } else if (dtype == PGMI_DTYPE_F32 || dtype == PGMI_DTYPE_F16) {
-        if (on_device) {
-            hipLaunchKernelGGL(k_convert, dim3(1024), dim3(256), 0, st, src, dtype, (long)s.numel, dst);
-            LAUNCHCHK();
-        } else {
-            std::vector<uint16_t> tmp(s.numel);
-            for (int64_t i = 0; i < s.numel; ++i) {
-                float f = dtype == PGMI_DTYPE_F32 ? reinterpret_cast<const float*>(src)[i]
-                                                 : (float)reinterpret_cast<const _Float16*>(src)[i];
-                tmp[i] = host_f2bf(f);
-            }
-            HIPCHK(hipMemcpyAsync(dst, tmp.data(), s.numel * 2, hipMemcpyHostToDevice, st));
-            HIPCHK(hipStreamSynchronize(st));
-        }
-    } else {
-        return fail(PGMI_E_ARG, "unsupported dtype");
-    }
-    return 0;
-}
-
-int pgmi_safetensors_count(const char* path, int* n) {
-    if (!path || !n) return fail(PGMI_E_ARG, "null argument");
-    StFile f;
-    if (!st_open(path, f)) return fail(PGMI_E_ARG, f.error);
-    *n = (int)f.entries.size();
-    return 0;
-}
-
-int pgmi_safetensors_entry(const char* path, int i, char* name, int name_cap, int* dtype, int64_t* shape4, int* ndim,
-                           int64_t* begin, int64_t* end) {
-    if (!path || !name || name_cap < 1 || !dtype || !shape4 || !ndim || !begin || !end)
-        return fail(PGMI_E_ARG, "null argument");
-    StFile f;
-    if (!st_open(path, f)) return fail(PGMI_E_ARG, f.error);
-    if (i < 0 || i >= (int)f.entries.size()) return fail(PGMI_E_ARG, "entry index out of range");
-    const StEntry& e = f.entries[i];
-    std::snprintf(name, (size_t)name_cap, "%s", e.name.c_str());
-    *dtype = e.dtype == "BF16" ? PGMI_DTYPE_BF16 : e.dtype == "F16" ? PGMI_DTYPE_F16 : e.dtype == "F32" ? PGMI_DTYPE_F32 : -1;
-    *ndim = (int)e.shape.size();
-    for (int d = 0; d < 4; ++d) shape4[d] = d < *ndim ? e.shape[d] : 0;
-    *begin = e.begin;
-    *end = e.end;
-    return 0;
-}
-
-// utils.py:19-44 (safe_open shard loop + load_state_dict(strict=False)) for one shard: tensors
-// named like slab weights are shape-checked, converted to bf16 and written into the slab; BF16
-// bytes go host -> slab directly from the mapped file, F32/F16 through the split-K scratch in
-// chunks and a device-side RNE conversion.  Synchronises the stream before unmapping.
-int pgmi_load_safetensors(pgmi_ctx* x, const char* path, int* n_loaded, int* n_skipped, void* stream) {
-    if (!x || !path) return fail(PGMI_E_ARG, "null argument");
-    if (!x->slab) return fail(PGMI_E_STATE, "weights are not bound");
-    HIPCHK(hipSetDevice(x->device));
-    StFile f;
-    if (!st_open(path, f)) return fail(PGMI_E_ARG, f.error);
-    hipStream_t st = (hipStream_t)stream;
-    // scratch for conversions: the context's workspace if prepared, else a temporary buffer
-    void* tmp = nullptr;
-    size_t tmp_bytes = 0;
-    uint8_t* scratch = reinterpret_cast<uint8_t*>(x->ws);
-    size_t scratch_bytes = x->ws ? x->ws_bytes : 0;
-    int loaded = 0, skipped = 0;
-    int rc = 0;
-    for (const StEntry& e : f.entries) {
-        auto it = x->index.find(e.name);
-        if (it == x->index.end()) {
-            ++skipped;
-            continue;
-        }
-        const Slot& sl = x->slots[it->second];
-        bool same = (int)e.shape.size() == sl.ndim;
-        for (int d = 0; same && d < sl.ndim; ++d) same = e.shape[d] == sl.shape[d];
-        if (!same) {
-            rc = fail(PGMI_E_ARG, "shape mismatch for " + e.name);
-            break;
-        }
-        const int eb = st_elem_bytes(e.dtype);
-        if (eb == 0) {
-            rc = fail(PGMI_E_ARG, "unsupported dtype " + e.dtype + " for " + e.name);
-            break;
-        }
-        if (e.end - e.begin != sl.numel * eb) {
-            rc = fail(PGMI_E_ARG, "byte size mismatch for " + e.name);
-            break;
-        }
-        const uint8_t* src = f.map + f.data0 + e.begin;
-        uint16_t* dst = reinterpret_cast<uint16_t*>(x->slab + sl.off);
-        if (e.dtype == "BF16") {
-            if (hipMemcpyAsync(dst, src, (size_t)sl.numel * 2, hipMemcpyHostToDevice, st) != hipSuccess) {
-                rc = fail(PGMI_E_HIP, "upload of " + e.name);
-                break;
-            }
-        } else {
-            const int dt = e.dtype == "F32" ? PGMI_DTYPE_F32 : PGMI_DTYPE_F16;
-            if (scratch_bytes < ((size_t)8 << 20)) {
-                if (!tmp) {
-                    tmp_bytes = (size_t)64 << 20;
-                    if (hipMalloc(&tmp, tmp_bytes) != hipSuccess) {
-                        rc = fail(PGMI_E_NOMEM, "conversion scratch");
-                        break;
-                    }
-                }
-                scratch = reinterpret_cast<uint8_t*>(tmp);
-                scratch_bytes = tmp_bytes;
-            }
-            const int64_t per = (int64_t)(scratch_bytes / (size_t)eb);
-            for (int64_t i0 = 0; i0 < sl.numel && rc == 0; i0 += per) {
-                const int64_t n = std::min<int64_t>(per, sl.numel - i0);
-                if (hipMemcpyAsync(scratch, src + i0 * eb, (size_t)n * eb, hipMemcpyHostToDevice, st) != hipSuccess) {
-                    rc = fail(PGMI_E_HIP, "upload of " + e.name);
-                    break;
-                }
-                hipLaunchKernelGGL(k_convert, dim3(1024), dim3(256), 0, st, scratch, dt, (long)n, dst + i0);
-            }
-            if (rc) break;
-        }
-        ++loaded;
-    }
-    const hipError_t se = hipStreamSynchronize(st);  // the mapped bytes must outlive the copies
-    if (tmp) (void)hipFree(tmp);
-    if (rc) return rc;
-    if (se != hipSuccess) return fail(PGMI_E_HIP, std::string("safetensors upload: ") + hipGetErrorString(se));
-    x->prepared = false;  // derived tensors (padded patch matrix, ...) are rebuilt by pgmi_prepare
-    if (n_loaded) *n_loaded = loaded;
-    if (n_skipped) *n_skipped = skipped;
-    return 0;
-}
-
-uint64_t pgmi_synthetic_key(const char* name, uint64_t seed) { return splitmix64_h(seed ^ fnv1a(name)); }
-
-int pgmi_fill_synthetic(pgmi_ctx* x, const char* name, uint64_t key, float scale, float offset, void* stream) {
-    if (!x || !name) return fail(PGMI_E_ARG, "null argument");
-    if (!x->slab) return fail(PGMI_E_STATE, "weights are not bound");
-    auto it = x->index.find(name);
-    if (it == x->index.end()) return fail(PGMI_E_ARG, std::string("unknown weight ") + name);
-    const Slot& s = x->slots[it->second];
-    HIPCHK(hipSetDevice(x->device));
-    fill_synthetic((hipStream_t)stream, reinterpret_cast<uint16_t*>(x->slab + s.off), (long)s.numel, key, scale, offset);
-    LAUNCHCHK();
-    return 0;
-}
-
 int pgmi_set_rope_inv_freq(pgmi_ctx* x, const float* inv) {
     if (!x || !inv) return fail(PGMI_E_ARG, "null argument");
     for (int i = 0; i < x->c.t_head_dim / 2; ++i) x->inv_freq[i] = inv[i];
@@ -571,11 +132,11 @@ int pgmi_set_rope_table(pgmi_ctx* x, const uint16_t* cs, const uint16_t* sn, int
     x->prepared = false;
     return 0;
 }
+}  // extern "C"
 
-int pgmi_prepare(pgmi_ctx* x) {
-    if (!x) return fail(PGMI_E_ARG, "null argument");
-    if (!x->slab) return fail(PGMI_E_STATE, "weights are not bound");
-    HIPCHK(hipSetDevice(x->device));
+namespace {
+
+int paligemma_prepare(pgmi_ctx* x) {
     const pgmi_config& c = x->c;
     int rc;
     if (!x->cosT) {
@@ -652,44 +213,9 @@ int pgmi_prepare(pgmi_ctx* x) {
     x->prepared = true;
     return 0;
 }
+}  // namespace
 
-int64_t pgmi_kv_bytes(const pgmi_ctx* x, int batch, int max_tokens) {
-    if (!x) return -1;
-    return (int64_t)x->c.t_layers * 2 * batch * max_tokens * x->c.t_kv_heads * x->c.t_head_dim * 2;
-}
-
-// Run body(stream) eagerly, or replay its captured hipGraph: the first call with a given key
-// runs eagerly (kernel attributes are set on first launch), the second captures, later ones
-// replay.  The key holds every pointer and size the body reads, so a replay is that call.
-extern "C++" {
-template <class F>
-static int run_graphed(pgmi_ctx* x, hipStream_t s, const std::vector<intptr_t>& key, F body) {
-    if (!x->prefill_graph) return body(s);
-    GraphEntry& ge = x->pgraphs[key];
-    if (!ge.exec) {
-        if (ge.seen++ == 0) return body(s);
-        if (x->pgraphs.size() > 64) {  // bound the cache (e.g. fresh buffers every call)
-            clear_pgraphs(x);
-            return body(s);
-        }
-        hipGraph_t g;
-        HIPCHK(hipStreamBeginCapture(x->cap_stream, hipStreamCaptureModeThreadLocal));
-        const int rc = body(x->cap_stream);
-        HIPCHK(hipStreamEndCapture(x->cap_stream, &g));
-        if (rc) {
-            (void)hipGraphDestroy(g);
-            return rc;
-        }
-        GraphEntry& ge2 = x->pgraphs[key];
-        HIPCHK(hipGraphInstantiate(&ge2.exec, g, nullptr, nullptr, 0));
-        (void)hipGraphDestroy(g);
-        HIPCHK(hipGraphLaunch(ge2.exec, s));
-        return 0;
-    }
-    HIPCHK(hipGraphLaunch(ge.exec, s));
-    return 0;
-}
-}  // extern "C++"
+extern "C" {
 
 static int vision_body(pgmi_ctx* x, hipStream_t s, const void* pixels, int dtype, int B, void* feats);
 
@@ -883,11 +409,11 @@ static int lm_body(pgmi_ctx* x, hipStream_t s, const int64_t* ids, const void* i
                                     (size_t)H * 2, B, hipMemcpyDeviceToDevice, s));
             if (kv_start + L <= c.max_kv) {
                 // one query row over the prompt's keys: the decode step's flash-decoding (64-key chunks
-                // in parallel, kv_len from a device step record set by a memset node) and its o_proj
+                // in parallel, kv_len from a device step record that a one-thread kernel sets) and its o_proj
                 // GEMV with the chunk combine in the prologue; a single 16-row prefill workgroup
                 // would walk every key alone
                 a.Lk = 0;
-                HIPCHK(hipMemsetD32Async(reinterpret_cast<hipDeviceptr_t>(&x->pstep->kv_len), kv_start + L - 1, 1, s));
+                set_step(s, x->pstep, kv_start + L - 1, 0);
                 a.mask = x->d_zero; a.mask_b_stride = 0; a.mask_k_stride = 0; a.mask_round = 1;
                 attention_decode(s, a, x->pstep, kv_start + L, x->opart, x->max_chunks);
                 gemv_o_attn(s, B, NH, x->opart, x->max_chunks, x->pstep, TL(x, i, "self_attn.o_proj.weight"), H,
@@ -1260,92 +786,6 @@ int pgmi_lm_final_hidden(pgmi_ctx* x, void* out, int rows, void* stream) {
     HIPCHK(hipMemcpyAsync(out, x->Tn, (size_t)rows * x->c.t_hidden * 2, hipMemcpyDeviceToDevice, (hipStream_t)stream));
     return 0;
 }
-
-// ---------------------------------------------------------------- replicas: load-time broadcast
-#define RCCL_READY()                                                                       \
-    do {                                                                                   \
-        const Rccl& r_ = rccl();                                                           \
-        if (!r_.get_unique_id || !r_.comm_init_rank || !r_.comm_destroy || !r_.broadcast || !r_.error_string) \
-            return fail(PGMI_E_STATE, std::string("librccl could not be loaded (dlopen librccl.so.1): ") + \
-                        (r_.h ? "missing nccl* symbols" : r_.why));                        \
-    } while (0)
-
-#define NCCLCHK(expr)                                                                      \
-    do {                                                                                   \
-        ncclResult_t r_ = (expr);                                                          \
-        if (r_ != ncclSuccess) return fail(PGMI_E_HIP, std::string(#expr) + ": " + rccl().error_string(r_)); \
-    } while (0)
-
-int pgmi_comm_unique_id(void* id_out) {
-    if (!id_out) return fail(PGMI_E_ARG, "null argument");
-    RCCL_READY();
-    static_assert(sizeof(ncclUniqueId) == PGMI_COMM_ID_BYTES, "ncclUniqueId size");
-    ncclUniqueId id;
-    NCCLCHK(rccl().get_unique_id(&id));
-    std::memcpy(id_out, &id, sizeof(id));
-    return 0;
-}
-
-int pgmi_comm_init(int device, int nranks, int rank, const void* id, void** comm_out) {
-    if (!id || !comm_out) return fail(PGMI_E_ARG, "null argument");
-    if (nranks < 1 || rank < 0 || rank >= nranks) return fail(PGMI_E_ARG, "bad rank / world size");
-    RCCL_READY();
-    // the communicator binds to the current device: switch for the init, then give the caller's
-    // thread its own current device back (torch keeps its own notion of it)
-    int prev = 0;
-    HIPCHK(hipGetDevice(&prev));
-    HIPCHK(hipSetDevice(device));
-    ncclUniqueId uid;
-    std::memcpy(&uid, id, sizeof(uid));
-    ncclComm_t comm = nullptr;
-    const ncclResult_t r = rccl().comm_init_rank(&comm, nranks, uid, rank);
-    HIPCHK(hipSetDevice(prev));
-    if (r != ncclSuccess) return fail(PGMI_E_HIP, std::string("ncclCommInitRank: ") + rccl().error_string(r));
-    *comm_out = comm;
-    return 0;
-}
-
-int pgmi_comm_destroy(void* comm) {
-    if (!comm) return 0;
-    RCCL_READY();
-    NCCLCHK(rccl().comm_destroy(reinterpret_cast<ncclComm_t>(comm)));
-    return 0;
-}
-
-int pgmi_broadcast_weights(pgmi_ctx* x, void* comm, int root, void* stream) {
-    if (!x || !comm) return fail(PGMI_E_ARG, "null argument");
-    if (!x->slab) return fail(PGMI_E_STATE, "weights are not bound (pgmi_bind_weights)");
-    RCCL_READY();
-    int prev = 0;
-    HIPCHK(hipGetDevice(&prev));
-    HIPCHK(hipSetDevice(x->device));
-    // the whole slab in one in-place collective: rank `root`'s bytes land in every replica
-    const ncclResult_t r = rccl().broadcast(x->slab, x->slab, (size_t)x->slab_bytes, ncclUint8, root,
-                                            reinterpret_cast<ncclComm_t>(comm), (hipStream_t)stream);
-    HIPCHK(hipSetDevice(prev));
-    if (r != ncclSuccess) return fail(PGMI_E_HIP, std::string("ncclBroadcast: ") + rccl().error_string(r));
-    x->prepared = false;  // derived tensors are rebuilt from the received weights by pgmi_prepare
-    return 0;
-}
-
-int pgmi_argmax(pgmi_ctx* x, const float* logits, int rows, int V, int64_t* out, void* stream) {
-    if (!x || !logits || !out) return fail(PGMI_E_ARG, "null argument");
-    if (rows <= 0 || V <= 0) return fail(PGMI_E_ARG, "argmax: empty logits");
-    if (!x->amax_v) return fail(PGMI_E_STATE, "argmax scratch missing");
-    argmax_rows((hipStream_t)stream, logits, rows, V, x->amax_v, x->amax_i, out);
-    LAUNCHCHK();
-    return 0;
-}
-
-int pgmi_eos_update(pgmi_ctx* x, int64_t* next_ids, int32_t* finished, int B, int64_t eos_id, int64_t pad_id,
-                    int32_t* n_alive, void* stream) {
-    if (!x || !next_ids || !finished) return fail(PGMI_E_ARG, "null argument");
-    if (B <= 0) return fail(PGMI_E_ARG, "eos_update: empty batch");
-    eos_update((hipStream_t)stream, next_ids, finished, B, eos_id, pad_id, n_alive);
-    LAUNCHCHK();
-    return 0;
-}
-
 int pgmi_decode_kernel(pgmi_ctx* x, int which, int layer, int B, void* stream) {
     int rc;
     if ((rc = ensure_prepared(x))) return rc;
@@ -1440,23 +880,6 @@ int pgmi_tune_attention(int variant) {
             return 0;
         }
     return fail(PGMI_E_ARG, "unknown attention variant");
-}
-
-int pgmi_sample_top_p(pgmi_ctx* x, const float* logits, int rows, int V, float temperature, float top_p,
-                      const float* u, int64_t* out, float* kept_mass, void* stream) {
-    if (!x || !logits || !u || !out) return fail(PGMI_E_ARG, "null argument");
-    if (rows <= 0 || V <= 0) return fail(PGMI_E_ARG, "sample_top_p: empty probabilities");
-    if (!(top_p >= 0.f)) return fail(PGMI_E_ARG, "sample_top_p: top_p must be >= 0");
-    if (!x->ws) return fail(PGMI_E_STATE, "workspace not allocated (pgmi_prepare)");
-    const int per = (int)std::min<size_t>((size_t)rows, x->ws_bytes / sample_scratch_bytes(1, V));
-    if (per < 1) return fail(PGMI_E_ARG, "sample_top_p: vocabulary exceeds the scratch");
-    for (int r0 = 0; r0 < rows; r0 += per) {  // row batches that fit the scratch (stream-ordered)
-        const int nr = std::min(per, rows - r0);
-        sample_top_p((hipStream_t)stream, logits + (size_t)r0 * V, nr, V, temperature, top_p, u + r0, x->ws,
-                     out + r0, kept_mass ? kept_mass + r0 : nullptr);
-    }
-    LAUNCHCHK();
-    return 0;
 }
 
 // ---------------------------------------------------------------- single ops (tests)
