@@ -263,6 +263,53 @@ int pgmi_tune_attention(int variant);
 int pgmi_sample_top_p(pgmi_ctx* ctx, const float* x, int rows, int V, float temperature, float top_p,
                       const float* u, int64_t* out, float* kept_mass, void* stream);
 
+/* ---- layered decoders: text models given as a list of layers, each a mixer (selective scan, windowed
+ * attention, minimal gated recurrence) and an optional gated feed-forward, around residual streams
+ * (hyper-connections) with grouped RMS norms.  A pgmi_ctx made by pgmi_decoder_create shares the
+ * weight-slab, loading, prepare, sampling and replica calls above; tensor names are the checkpoint's
+ * ("embed", "l<i>.norm1", "l<i>.mix.in", ..., "final.norm"), all bf16 in the slab.
+ *
+ * State: one caller-owned slab of pgmi_kv_bytes(ctx, n_slots, max_tokens) bytes.  A slot holds one
+ * sequence: per layer its convolution taps and scan state, recurrent state, or key / value rows.  A
+ * sequence starts at position 0, which reads nothing of what its slot held before. */
+#define PGMI_MIXER_MAMBA1 0
+#define PGMI_MIXER_ATTENTION 1
+#define PGMI_MIXER_MINGRU 2
+
+typedef struct pgmi_layer_spec {
+    int mixer;                          /* PGMI_MIXER_* */
+    int conv, dt_rank, inner, state;    /* mamba1: taps, step rank, channels, states per channel */
+    int width;                          /* mingru: channels */
+    int heads, kv_heads, dim, vdim;     /* attention: query / key-value heads, query-key and value head sizes */
+    int window;                         /* attention: position i sees j with 0 <= i - j < window */
+    float scale;                        /* attention: factor of q . k */
+    int ff;                             /* feed-forward size, 0: none */
+} pgmi_layer_spec;
+
+typedef struct pgmi_decoder_config {
+    int vocab, width, streams, norm_groups, n_layers;
+    float norm_eps, embed_scale;
+    int max_batch;  /* sequences per call */
+    int act_dtype;  /* PGMI_DTYPE_BF16, or PGMI_DTYPE_F32: activations, caches and products in fp32 */
+} pgmi_decoder_config;
+
+int pgmi_decoder_create(int device, const pgmi_decoder_config* cfg, const pgmi_layer_spec* layers, pgmi_ctx** out);
+/* The next tokens of n_seq sequences, packed sequence after sequence (device int64 ids, sum of lens): sequence r
+ * continues in slots[r] at position starts[r] with lens[r] >= 1 tokens (slots, starts, lens: host).  The logits of
+ * the rows listed in want (host, n_want indices into the packed rows, may be 0) go to logits (device fp32
+ * [n_want][vocab]).  taps (may be NULL): device fp32 [n_layers][rows][width], the summed streams after every layer.
+ * A slot appears once per call. */
+int pgmi_decoder_forward(pgmi_ctx* ctx, const int64_t* ids, int n_seq, const int32_t* slots, const int32_t* starts,
+                         const int32_t* lens, void* state, int n_slots, int max_tokens, const int32_t* want, int n_want,
+                         float* logits, float* taps, void* stream);
+/* n_steps greedy decode steps for B sequences, one token each per step: ids (device int64 [B]) at positions
+ * positions[b] of slots[b] (host arrays).  next_ids (device int64 [B], may be NULL when n_steps == 1, may be ids
+ * itself) receives the argmax that feeds the following step; tokens (device int64 [n_steps][B], may be NULL) records
+ * every step's.  logits (device fp32 [B][vocab]): the last step's.  use_graph != 0 replays a captured hipGraph. */
+int pgmi_decoder_decode(pgmi_ctx* ctx, const int64_t* ids, int B, const int32_t* slots, const int32_t* positions,
+                        void* state, int n_slots, int max_tokens, int n_steps, float* logits, int64_t* next_ids,
+                        int64_t* tokens, int use_graph, void* stream);
+
 /* ---- single-op entry points (kernel-level parity tests) ---------------------------------- */
 /* out = epilogue(A[M,K] . W[N,K]^T): epi 0 store, 1 +bias, 2 +bias,gelu, 3 +bias,+res, 4 +res,
  * 6 fp32 out (out is float*), 7 GeGLU with up rows at W + N*K */

@@ -61,6 +61,7 @@ __device__ __forceinline__ void epi_store(const EpiArgs& ea, int m, int n, float
             break;
         case EPI_F32: ea.out_f32[(long)m * ea.ldo + n] = rbf(acc); break;
         case EPI_GEGLU: ea.out[(long)m * ea.ldo + n] = f2bf(rbf(gelu_tanh(rbf(acc))) * rbf(acc2)); break;
+        case EPI_SWIGLU: ea.out[(long)m * ea.ldo + n] = f2bf(acc / (1.0f + __expf(-acc)) * acc2); break;
         default: break;  // EPI_ROPE: rope_apply
     }
 }
@@ -152,6 +153,7 @@ __device__ __forceinline__ void epi_apply(const EpiArgs& ea, int M, int N, int m
                 else if constexpr (EPI == EPI_RES) o = rbf(a) + e.xv[i][j][r];
                 else if constexpr (EPI == EPI_BIAS_POS) o = rbf(a + e.bv[j]) + e.xv[i][j][r];
                 else if constexpr (EPI == EPI_GEGLU) o = rbf(gelu_tanh(rbf(a))) * rbf(acc2[i][j][r]);
+                else if constexpr (EPI == EPI_SWIGLU) o = a / (1.0f + __expf(-a)) * acc2[i][j][r];
                 if (m < M && n < N) {
                     if constexpr (EPI == EPI_F32) ea.out_f32[(long)m * ea.ldo + n] = rbf(a);
                     else ea.out[(long)m * ea.ldo + n] = f2bf(o);
@@ -257,7 +259,7 @@ __global__ void __launch_bounds__(64 * WGM * WGN) k_gemm(const uint16_t* __restr
                                                          const uint16_t* __restrict__ W, int ldw, int M, int N, int K,
                                                          int kt_per_split, EpiArgs ea, float* __restrict__ ws,
                                                          long up_off) {
-    constexpr bool DUAL = (EPI == EPI_GEGLU);
+    constexpr bool DUAL = epi_dual(EPI);
     constexpr int NT = 64 * WGM * WGN;
     constexpr int BM = WGM * TM * 16, BN = WGN * TN * 16;
     constexpr int ACH = (BM * 8 + NT - 1) / NT;  // 16-B chunks of the A tile per thread
@@ -407,7 +409,7 @@ __global__ void k_splitk_epi(const float* __restrict__ ws, int S, int M, int N, 
 // lane-linear), and the matching XOR on the ds_read_b128 fragment reads makes them
 // bank-conflict free.  K tails (K % 64, e.g. SigLIP fc2 K = 4304) read a zero block.
 // Waves form a 2 x 2 grid; wave (wm, wn) owns TM x TN (x NB) 16x16 MFMA tiles.
-__device__ __attribute__((aligned(16))) uint4 g_zero_chunk[1] = {{0u, 0u, 0u, 0u}};
+static __device__ __attribute__((aligned(16))) uint4 g_zero_chunk[1] = {{0u, 0u, 0u, 0u}};
 
 // s_waitcnt vmcnt(G * n) for a runtime n in [0, NMAX] (the count must be an immediate)
 template <int G, int NMAX>
@@ -995,7 +997,7 @@ __global__ void __launch_bounds__(512, 1) k_gemm_8p(const uint16_t* __restrict__
                                                     int kt_per_split, EpiArgs ea, float* __restrict__ ws, long up_off,
                                                     int n_mt, int code) {
     static_assert(TM % 2 == 0, "row halves of whole 16-row tiles");
-    constexpr bool DUAL = (EPI == EPI_GEGLU);
+    constexpr bool DUAL = epi_dual(EPI);
     constexpr int H = TM / 2;                 // row tiles per quadrant
     constexpr int BM = 32 * TM;
     constexpr int HAR = 16 * TM;              // rows of an A half image (H tiles of each wave row)
@@ -1206,7 +1208,7 @@ __global__ void __launch_bounds__(512, 1) k_gemm_8p(const uint16_t* __restrict__
     }
 }
 
-// (PGMI_GEMM_KERNELS_ONLY: the kernel templates alone, for single-instantiation ISA / register checks)
+// (PGMI_GEMM_KERNELS_ONLY: the kernel templates alone -- kernels_matmul.hip instantiates its own few)
 #ifndef PGMI_GEMM_KERNELS_ONLY
 // Tile configurations (wave grid, per-wave MFMA tiles).  BM = WGM*TM*16, BN = WGN*TN*16.
 enum Cfg : int {
@@ -1456,7 +1458,7 @@ void gemm_probe_events(hipEvent_t start, hipEvent_t stop) {
 template <int WGM, int WGN, int TM, int TN, int EPI>
 static void launch_t(hipStream_t s, const uint16_t* A, int lda, const uint16_t* W, int ldw, int M, int N, int K,
                      const EpiArgs& ea, float* ws, int split, long up_off) {
-    constexpr int NB = (EPI == EPI_GEGLU) ? 2 : 1;  // EPI < 0: partials only
+    constexpr int NB = epi_dual(EPI) ? 2 : 1;  // EPI < 0: partials only
     constexpr int BM = WGM * TM * 16, BN = WGN * TN * 16, NT = 64 * WGM * WGN;
     const size_t lds = (size_t)(2 * BM * LDSK + 2 * NB * BN * LDSK) * sizeof(uint16_t);
     const int nkt = (K + BK - 1) / BK;
@@ -1495,7 +1497,7 @@ static void launch_t(hipStream_t s, const uint16_t* A, int lda, const uint16_t* 
 template <int NW, int WM, int TM, int TNW, int ST, int EPI>
 static void launch_p(hipStream_t s, const uint16_t* A, int lda, const uint16_t* W, int ldw, int M, int N, int K,
                      const EpiArgs& ea, float* ws, int split, long up_off) {
-    constexpr bool DUAL = (EPI == EPI_GEGLU);
+    constexpr bool DUAL = epi_dual(EPI);
     constexpr int NB = DUAL ? 2 : 1;
     constexpr int TN = DUAL ? (TNW >= 2 ? TNW / 2 : 1) : TNW;  // the dual GEMM keeps the B rows per slot
     constexpr int BM = WM * TM * 16, BN = (NW / WM) * TN * 16;
@@ -1535,7 +1537,7 @@ static void launch_p(hipStream_t s, const uint16_t* A, int lda, const uint16_t* 
 template <int NW, int WM, int TM, int TNW, int ST, int LW, int EPI, bool RL = false>
 static void launch_w(hipStream_t s, const uint16_t* A, int lda, const uint16_t* W, int ldw, int M, int N, int K,
                      const EpiArgs& ea, float* ws, int split, long up_off) {
-    constexpr bool DUAL = (EPI == EPI_GEGLU);
+    constexpr bool DUAL = epi_dual(EPI);
     constexpr int NB = DUAL ? 2 : 1;
     constexpr int TN = DUAL ? (TNW >= 2 ? TNW / 2 : 1) : TNW;
     constexpr int BM = WM * TM * 16, BN = (NW / WM) * TN * 16;
@@ -1575,7 +1577,7 @@ static void launch_w(hipStream_t s, const uint16_t* A, int lda, const uint16_t* 
 template <int TM, int EPI>
 static void launch_8p(hipStream_t s, const uint16_t* A, int lda, const uint16_t* W, int ldw, int M, int N, int K,
                       const EpiArgs& ea, float* ws, int split, long up_off) {
-    constexpr bool DUAL = (EPI == EPI_GEGLU);
+    constexpr bool DUAL = epi_dual(EPI);
     constexpr int BM = 32 * TM, BNO = DUAL ? 128 : 256;
     constexpr size_t lds = (size_t)2 * (2 * 16 * TM * 128 + 2 * 128 * 128);
     static_assert(lds <= 163840, "LDS exceeds 160 KiB");
@@ -1705,7 +1707,8 @@ int gemm(hipStream_t s, const uint16_t* A, int lda, const uint16_t* W, int ldw, 
         case EPI_BIAS_POS: launch_e<EPI_BIAS_POS>(s, A, lda, W, ldw, M, N, K, ea, ws, p, up_off); break;
         case EPI_F32: launch_e<EPI_F32>(s, A, lda, W, ldw, M, N, K, ea, ws, p, up_off); break;
         case EPI_GEGLU: launch_e<EPI_GEGLU>(s, A, lda, W, ldw, M, N, K, ea, ws, p, up_off); break;
-        case EPI_ROPE: return 0;  // gemm_qkv_rope only
+        case EPI_ROPE: return 0;    // gemm_qkv_rope only
+        case EPI_SWIGLU: return 0;  // matmul_rt only
     }
     return 1;
 }

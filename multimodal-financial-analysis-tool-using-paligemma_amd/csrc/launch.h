@@ -17,7 +17,9 @@ enum Epi : int {
     EPI_GEGLU = 7,      // out = bf16(bf16(gelu(bf16(acc_gate))) * bf16(acc_up))  (dual B)
     EPI_ROPE = 8,       // Gemma q|k|v rows: RoPE on q and k, q -> q_out, k / v appended to the KV cache
                         // (modeling_gemma.py:197-198,259); gemm_qkv_rope only
+    EPI_SWIGLU = 9,     // out = bf16(silu(acc_gate) * acc_up)  (dual B); matmul_rt only
 };
+constexpr bool epi_dual(int epi) { return epi == EPI_GEGLU || epi == EPI_SWIGLU; }
 
 struct EpiArgs {
     const uint16_t* bias = nullptr;

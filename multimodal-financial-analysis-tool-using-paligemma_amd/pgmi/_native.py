@@ -14,6 +14,9 @@ import torch  # noqa: F401  (must precede the library load: shared HIP runtime)
 _HERE = os.path.dirname(os.path.abspath(__file__))
 # PGMI_LIB_PATH: an alternative build of the same library, for same-box A/B measurements only
 LIB_PATH = os.environ.get("PGMI_LIB_PATH") or os.path.join(_HERE, "libpgmi.so")
+# the same ABI without the PaliGemma entry points (`make decoder`): used where only it has been built
+DECODER_LIB_PATH = os.path.join(_HERE, "libpgmi_decoder.so")
+CSRC = os.path.join(os.path.dirname(_HERE), "csrc")
 
 PGMI_OK, PGMI_E_ARG, PGMI_E_STATE, PGMI_E_HIP, PGMI_E_NOMEM = 0, -1, -2, -3, -4
 DTYPE_BF16, DTYPE_F16, DTYPE_F32 = 0, 1, 2
@@ -33,6 +36,17 @@ class PgmiConfig(ctypes.Structure):
         ("image_token_index", ctypes.c_int64), ("pad_token_id", ctypes.c_int64),
         ("max_batch", ctypes.c_int), ("max_seq", ctypes.c_int), ("max_kv", ctypes.c_int),
     ]
+
+
+class LayerSpec(ctypes.Structure):
+    _fields_ = [(n, ctypes.c_int) for n in ("mixer", "conv", "dt_rank", "inner", "state", "width", "heads", "kv_heads",
+                                            "dim", "vdim", "window")] + [("scale", ctypes.c_float), ("ff", ctypes.c_int)]
+
+
+class DecoderConfigC(ctypes.Structure):
+    _fields_ = [("vocab", ctypes.c_int), ("width", ctypes.c_int), ("streams", ctypes.c_int), ("norm_groups", ctypes.c_int),
+                ("n_layers", ctypes.c_int), ("norm_eps", ctypes.c_float), ("embed_scale", ctypes.c_float),
+                ("max_batch", ctypes.c_int), ("act_dtype", ctypes.c_int)]
 
 
 vp, i32, i64, f32, u64 = ctypes.c_void_p, ctypes.c_int, ctypes.c_int64, ctypes.c_float, ctypes.c_uint64
@@ -100,6 +114,9 @@ SIGNATURES = {
                                    i64, vp, vp]),
     "pgmi_op_rope": (i32, [vp, vp, vp, vp, i64, i32, i32, vp, vp]),
     "pgmi_op_scale": (i32, [vp, vp, f32, i64, vp, vp]),
+    "pgmi_decoder_create": (i32, [i32, ctypes.POINTER(DecoderConfigC), ctypes.POINTER(LayerSpec), ctypes.POINTER(vp)]),
+    "pgmi_decoder_forward": (i32, [vp, vp, i32, vp, vp, vp, vp, i32, i32, vp, i32, vp, vp, vp]),
+    "pgmi_decoder_decode": (i32, [vp, vp, i32, vp, vp, vp, i32, i32, i32, vp, vp, vp, i32, vp]),
 }
 
 _lib = None
@@ -110,18 +127,37 @@ class NativeError(RuntimeError):
 
 
 def lib():
-    """Load libpgmi.so (once).  Raises if it is missing: there is no CPU fallback."""
+    """Load libpgmi.so (once), or the decoder-only build where that is all there is.  Raises if neither is
+    built: there is no CPU fallback."""
     global _lib
     if _lib is None:
-        if not os.path.exists(LIB_PATH):
-            raise NativeError(f"{LIB_PATH} not built: run `make -C csrc` or __graft_entry__.build()")
-        L = ctypes.CDLL(LIB_PATH)
+        path = LIB_PATH
+        if not os.path.exists(path):
+            if not os.path.exists(DECODER_LIB_PATH):
+                raise NativeError(f"{LIB_PATH} not built: run `make -C csrc` or __graft_entry__.build()")
+            path = DECODER_LIB_PATH
+        L = ctypes.CDLL(path)
         for name, (res, args) in SIGNATURES.items():
+            if path == DECODER_LIB_PATH and not hasattr(L, name):
+                continue  # a PaliGemma entry point: using it raises AttributeError
             fn = getattr(L, name)
             fn.restype = res
             fn.argtypes = args
         _lib = L
     return _lib
+
+
+def ensure_decoder_built() -> None:
+    """Compile the decoder-only library if neither it nor libpgmi.so is there (a fresh checkout's first call)."""
+    if os.path.exists(LIB_PATH) or os.path.exists(DECODER_LIB_PATH):
+        return
+    import fcntl
+    import subprocess
+    with open(os.path.join(_HERE, ".build.lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        if not os.path.exists(DECODER_LIB_PATH):
+            jobs = os.environ.get("MAX_JOBS") or str(min(16, os.cpu_count() or 8))
+            subprocess.run(["make", "-C", CSRC, f"-j{jobs}", "decoder"], check=True, stdout=subprocess.DEVNULL)
 
 
 def check(rc: int, what: str = ""):

@@ -43,29 +43,18 @@ def config_dict(cfg) -> dict:
     }
 
 
-class Engine:
-    # generate(): greedy steps per hipGraph launch (pgmi_decode_steps) for batches of GEN_MIN_BATCH rows or more.
-    # Same box (tools/probes/multistep_probe.py): B = 8 step 1.279 -> 1.271 ms at 8-16 steps per launch, B = 1
-    # 1.056 -> 1.060 ms (slower: B <= 2 keeps one launch per step)
-    GEN_CHUNK = 8
+class EngineBase:
+    """What every model family's engine shares: the context and its bf16 weight slab (named views, loaders,
+    deterministic fills), stream ordering, and token picking (argmax, top-p, stop tokens, the generate loop).
+    A family's constructor creates its context and calls _bind()."""
+
+    vocab = 0       # logits per token
+    GEN_CHUNK = 8   # generate(): greedy steps per hipGraph launch, for batches of GEN_MIN_BATCH rows or more
     GEN_MIN_BATCH = 3
 
-    def __init__(self, cfg, device=None, max_batch: int = 8, max_seq: int = 1472, max_kv: Optional[int] = None):
-        self.lib = N.lib()
-        self.cfgd = config_dict(cfg)
-        self.device = torch.device("cuda", torch.cuda.current_device() if device is None else
-                                   torch.device(device).index or 0)
-        c = N.PgmiConfig()
-        for k, _ in N.PgmiConfig._fields_:
-            if k in ("max_batch", "max_seq", "max_kv"):
-                continue
-            setattr(c, k, self.cfgd[k])
-        c.max_batch, c.max_seq = max_batch, max_seq
-        c.max_kv = max_kv if max_kv else self.cfgd["t_max_pos"]
-        self.max_batch, self.max_seq, self.max_kv = max_batch, max_seq, c.max_kv
-        h = ctypes.c_void_p()
-        N.check(self.lib.pgmi_create(self.device.index, ctypes.byref(c), ctypes.byref(h)), "pgmi_create")
-        self.ctx = h
+    def _bind(self, ctx):
+        """Allocate and bind the weight slab of a freshly created context."""
+        self.ctx = ctx
         nbytes = self.lib.pgmi_weights_bytes(self.ctx)
         self.slab = torch.empty(nbytes, dtype=torch.uint8, device=self.device)
         N.check(self.lib.pgmi_bind_weights(self.ctx, self.slab.data_ptr()), "pgmi_bind_weights")
@@ -142,6 +131,133 @@ class Engine:
             N.check(self.lib.pgmi_fill_synthetic(self.ctx, n.encode(), key, scale, offset, s), n)
         self.prepared = False
 
+    _stream_guard = None  # pgmi/lookahead.py: makes a call wait for a step still running on its side stream
+
+    def _s(self):
+        h = N.stream_handle(self.device)
+        if self._stream_guard is not None:
+            self._stream_guard(h)
+        return h
+
+    def _ready(self):
+        if not self.prepared:
+            self.prepare()
+
+    def argmax(self, logits: torch.Tensor) -> torch.Tensor:
+        l2 = logits.reshape(-1, logits.shape[-1]).contiguous()
+        out = torch.empty(l2.shape[0], dtype=torch.int64, device=self.device)
+        N.check(self.lib.pgmi_argmax(self.ctx, l2.data_ptr(), l2.shape[0], l2.shape[1], out.data_ptr(), self._s()))
+        return out
+
+    def sample_top_p(self, x: torch.Tensor, top_p: float, temperature: Optional[float] = None,
+                     u: Optional[torch.Tensor] = None, generator: Optional[torch.Generator] = None,
+                     return_kept_mass: bool = False):
+        """Nucleus sampling on the device (inference.py:15-24; SURVEY.md sec.8f rank 4).
+        x (..., V) fp32: logits when `temperature` > 0 (softmax(x / T) of inference.py:65 is
+        fused), else probabilities (the reference _sample_top_p's input).  u: uniforms in [0, 1)
+        per row (default: torch.rand on the device with `generator`).  Returns int64 (rows,)."""
+        x2 = x.reshape(-1, x.shape[-1]).to(self.device, torch.float32).contiguous()
+        rows, V = x2.shape
+        if u is None:
+            u = torch.rand(rows, device=self.device, generator=generator)
+        u = u.to(self.device, torch.float32).reshape(-1).contiguous()
+        if u.numel() != rows:
+            raise ValueError(f"need one uniform per row: {u.numel()} != {rows}")
+        out = torch.empty(rows, dtype=torch.int64, device=self.device)
+        kept = torch.empty(rows, dtype=torch.float32, device=self.device) if return_kept_mass else None
+        T = float(temperature) if temperature is not None and temperature > 0 else 0.0
+        N.check(self.lib.pgmi_sample_top_p(self.ctx, x2.data_ptr(), rows, V, T, float(top_p), u.data_ptr(),
+                                           out.data_ptr(), N.ptr(kept), self._s()), "pgmi_sample_top_p")
+        return (out, kept) if return_kept_mass else out
+
+    # ------------------------------------------------------------------ the generate loop
+    def _generate_loop(self, first_logits, n_tokens, decode_one, decode_many, graph, do_sample=False, temperature=0.8,
+                       top_p=0.9, generator=None, eos_token_id=None, pad_token_id=None, sync_every=16,
+                       return_lengths=False):
+        """Tokens 0 .. n_tokens - 1 of every row from the prefill's last logits (B, V): picked on the device, no host
+        sync per token.  decode_one(cur, t, logits, next_ids) runs the step whose input tokens `cur` are token t - 1;
+        decode_many(cur, t, n, logits, record) runs n greedy steps from there in one call."""
+        B = first_logits.shape[0]
+        toks = torch.empty((B, n_tokens), dtype=torch.int64, device=self.device)
+        if do_sample:
+            us = torch.rand((n_tokens, B), device=self.device, generator=generator)
+            toks[:, 0] = self.sample_top_p(first_logits, top_p, temperature, u=us[0])
+        else:
+            toks[:, 0] = self.argmax(first_logits)
+        step_logits = torch.empty((B, self.vocab), dtype=torch.float32, device=self.device)
+        nxt = torch.empty(B, dtype=torch.int64, device=self.device)
+        cur = toks[:, 0].clone()
+        stop = eos_token_id is not None
+        if stop:
+            pad = int(eos_token_id if pad_token_id is None else pad_token_id)
+            finished = torch.zeros(B, dtype=torch.int32, device=self.device)
+            alive = torch.empty(1, dtype=torch.int32, device=self.device)
+            self._eos_update(cur, finished, int(eos_token_id), pad, alive)
+            toks[:, 0] = cur
+        n_done = n_tokens
+        if not do_sample and not stop and graph and n_tokens > 1 and B >= self.GEN_MIN_BATCH:
+            # greedy without a stop token: GEN_CHUNK steps per hipGraph launch (pgmi_decode_steps), the
+            # argmax fed back in place and every step's token kept in a device record
+            rec = torch.empty((self.GEN_CHUNK, B), dtype=torch.int64, device=self.device)
+            t = 1
+            while t < n_tokens:
+                n = min(self.GEN_CHUNK, n_tokens - t)
+                decode_many(cur, t, n, step_logits, rec)
+                toks[:, t:t + n] = rec[:n].t()
+                t += n
+            return (toks, torch.full((B,), n_tokens, dtype=torch.int64, device=self.device)) if return_lengths else toks
+        for t in range(1, n_tokens):
+            if stop and (t - 1) % max(1, sync_every) == 0 and int(alive.item()) == 0:
+                n_done = t
+                break
+            if do_sample:
+                decode_one(cur, t, step_logits, nxt)
+                cur.copy_(self.sample_top_p(step_logits, top_p, temperature, u=us[t]))
+            else:  # greedy: the argmax is fed back in place (pgmi_decode with next_ids == ids)
+                decode_one(cur, t, step_logits, cur)
+            if stop:
+                self._eos_update(cur, finished, int(eos_token_id), pad, alive)
+            toks[:, t] = cur
+        if not stop:
+            return (toks, torch.full((B,), n_tokens, dtype=torch.int64, device=self.device)) if return_lengths else toks
+        toks = toks[:, :n_done]
+        hit = toks == int(eos_token_id)
+        first = torch.where(hit.any(1), hit.int().argmax(1) + 1, torch.full_like(hit[:, 0], n_done, dtype=torch.int64))
+        toks = toks[:, :int(first.max().item())].contiguous()
+        return (toks, first.to(torch.int64)) if return_lengths else toks
+
+    def _eos_update(self, next_ids: torch.Tensor, finished: torch.Tensor, eos: int, pad: int,
+                    n_alive: Optional[torch.Tensor]) -> None:
+        N.check(self.lib.pgmi_eos_update(self.ctx, next_ids.data_ptr(), finished.data_ptr(), next_ids.numel(), eos, pad,
+                                         n_alive.data_ptr() if n_alive is not None else None, self._s()),
+                "pgmi_eos_update")
+
+
+class Engine(EngineBase):
+    # generate(): greedy steps per hipGraph launch (pgmi_decode_steps) for batches of GEN_MIN_BATCH rows or more.
+    # Same box (tools/probes/multistep_probe.py): B = 8 step 1.279 -> 1.271 ms at 8-16 steps per launch, B = 1
+    # 1.056 -> 1.060 ms (slower: B <= 2 keeps one launch per step)
+    GEN_CHUNK = 8
+    GEN_MIN_BATCH = 3
+
+    def __init__(self, cfg, device=None, max_batch: int = 8, max_seq: int = 1472, max_kv: Optional[int] = None):
+        self.lib = N.lib()
+        self.cfgd = config_dict(cfg)
+        self.device = torch.device("cuda", torch.cuda.current_device() if device is None else
+                                   torch.device(device).index or 0)
+        c = N.PgmiConfig()
+        for k, _ in N.PgmiConfig._fields_:
+            if k in ("max_batch", "max_seq", "max_kv"):
+                continue
+            setattr(c, k, self.cfgd[k])
+        c.max_batch, c.max_seq = max_batch, max_seq
+        c.max_kv = max_kv if max_kv else self.cfgd["t_max_pos"]
+        self.max_batch, self.max_seq, self.max_kv = max_batch, max_seq, c.max_kv
+        h = ctypes.c_void_p()
+        N.check(self.lib.pgmi_create(self.device.index, ctypes.byref(c), ctypes.byref(h)), "pgmi_create")
+        self.vocab = self.cfgd["t_vocab"]
+        self._bind(h)
+
     def prepare(self, inv_freq: Optional[torch.Tensor] = None, exact_table: bool = True):
         """RoPE tables from the module's inv_freq buffer (the reference's own values) and the
         padded patch matrix.  With exact_table the cos/sin table is computed by torch on the
@@ -187,18 +303,6 @@ class Engine:
         return buf
 
     # ------------------------------------------------------------------ forward pieces
-    _stream_guard = None  # pgmi/lookahead.py: makes a call wait for a step still running on its side stream
-
-    def _s(self):
-        h = N.stream_handle(self.device)
-        if self._stream_guard is not None:
-            self._stream_guard(h)
-        return h
-
-    def _ready(self):
-        if not self.prepared:
-            self.prepare()
-
     def vision(self, pixel_values: torch.Tensor) -> torch.Tensor:
         self._ready()
         px = pixel_values.to(self.device)
@@ -382,33 +486,6 @@ class Engine:
         """Batched decode RMSNorm form: 0 once per row (default), 1 staged per projection, -1 default."""
         N.check(self.lib.pgmi_set_decode_staged_norm(self.ctx, int(on)), "pgmi_set_decode_staged_norm")
 
-    def argmax(self, logits: torch.Tensor) -> torch.Tensor:
-        l2 = logits.reshape(-1, logits.shape[-1]).contiguous()
-        out = torch.empty(l2.shape[0], dtype=torch.int64, device=self.device)
-        N.check(self.lib.pgmi_argmax(self.ctx, l2.data_ptr(), l2.shape[0], l2.shape[1], out.data_ptr(), self._s()))
-        return out
-
-    def sample_top_p(self, x: torch.Tensor, top_p: float, temperature: Optional[float] = None,
-                     u: Optional[torch.Tensor] = None, generator: Optional[torch.Generator] = None,
-                     return_kept_mass: bool = False):
-        """Nucleus sampling on the device (inference.py:15-24; SURVEY.md sec.8f rank 4).
-        x (..., V) fp32: logits when `temperature` > 0 (softmax(x / T) of inference.py:65 is
-        fused), else probabilities (the reference _sample_top_p's input).  u: uniforms in [0, 1)
-        per row (default: torch.rand on the device with `generator`).  Returns int64 (rows,)."""
-        x2 = x.reshape(-1, x.shape[-1]).to(self.device, torch.float32).contiguous()
-        rows, V = x2.shape
-        if u is None:
-            u = torch.rand(rows, device=self.device, generator=generator)
-        u = u.to(self.device, torch.float32).reshape(-1).contiguous()
-        if u.numel() != rows:
-            raise ValueError(f"need one uniform per row: {u.numel()} != {rows}")
-        out = torch.empty(rows, dtype=torch.int64, device=self.device)
-        kept = torch.empty(rows, dtype=torch.float32, device=self.device) if return_kept_mass else None
-        T = float(temperature) if temperature is not None and temperature > 0 else 0.0
-        N.check(self.lib.pgmi_sample_top_p(self.ctx, x2.data_ptr(), rows, V, T, float(top_p), u.data_ptr(),
-                                           out.data_ptr(), N.ptr(kept), self._s()), "pgmi_sample_top_p")
-        return (out, kept) if return_kept_mass else out
-
     # ------------------------------------------------------------------ batched greedy driver
     @torch.no_grad()
     def generate(self, input_ids: torch.Tensor, pixel_values: torch.Tensor, n_tokens: int, graph: bool = True,
@@ -433,56 +510,12 @@ class Engine:
             kv = self.new_kv(B, L + n_tokens + 1)
         feats = self.project(self.vision(pixel_values))
         logits = self.lm_forward(kv, 0, torch.arange(L).expand(B, L), ids=ids, image_feats=feats, logits_rows=2)
-        toks = torch.empty((B, n_tokens), dtype=torch.int64, device=self.device)
-        if do_sample:
-            us = torch.rand((n_tokens, B), device=self.device, generator=generator)
-            toks[:, 0] = self.sample_top_p(logits[:, 0], top_p, temperature, u=us[0])
-        else:
-            toks[:, 0] = self.argmax(logits[:, 0])
-        step_logits = torch.empty((B, self.cfgd["t_vocab"]), dtype=torch.float32, device=self.device)
-        nxt = torch.empty(B, dtype=torch.int64, device=self.device)
-        cur = toks[:, 0].clone()
-        stop = eos_token_id is not None
-        if stop:
-            pad = int(eos_token_id if pad_token_id is None else pad_token_id)
-            finished = torch.zeros(B, dtype=torch.int32, device=self.device)
-            alive = torch.empty(1, dtype=torch.int32, device=self.device)
-            self._eos_update(cur, finished, int(eos_token_id), pad, alive)
-            toks[:, 0] = cur
-        n_done = n_tokens
-        if not do_sample and not stop and graph and n_tokens > 1 and B >= self.GEN_MIN_BATCH:
-            # greedy without a stop token: GEN_CHUNK steps per hipGraph launch (pgmi_decode_steps), the
-            # argmax fed back in place and every step's token kept in a device record
-            rec = torch.empty((self.GEN_CHUNK, B), dtype=torch.int64, device=self.device)
-            t = 1
-            while t < n_tokens:
-                n = min(self.GEN_CHUNK, n_tokens - t)
-                self.decode_steps(cur, kv, L + t - 1, L + t, n, logits=step_logits, tokens=rec, graph=graph)
-                toks[:, t:t + n] = rec[:n].t()
-                t += n
-            return (toks, torch.full((B,), n_tokens, dtype=torch.int64, device=self.device)) if return_lengths else toks
-        for t in range(1, n_tokens):
-            if stop and (t - 1) % max(1, sync_every) == 0 and int(alive.item()) == 0:
-                n_done = t
-                break
-            if do_sample:
-                self.decode(cur, kv, L + t - 1, L + t, logits=step_logits, next_ids=nxt, graph=graph)
-                cur.copy_(self.sample_top_p(step_logits, top_p, temperature, u=us[t]))
-            else:  # greedy: the argmax is fed back in place (pgmi_decode with next_ids == ids)
-                self.decode(cur, kv, L + t - 1, L + t, logits=step_logits, next_ids=cur, graph=graph)
-            if stop:
-                self._eos_update(cur, finished, int(eos_token_id), pad, alive)
-            toks[:, t] = cur
-        if not stop:
-            return (toks, torch.full((B,), n_tokens, dtype=torch.int64, device=self.device)) if return_lengths else toks
-        toks = toks[:, :n_done]
-        hit = toks == int(eos_token_id)
-        first = torch.where(hit.any(1), hit.int().argmax(1) + 1, torch.full_like(hit[:, 0], n_done, dtype=torch.int64))
-        toks = toks[:, :int(first.max().item())].contiguous()
-        return (toks, first.to(torch.int64)) if return_lengths else toks
 
-    def _eos_update(self, next_ids: torch.Tensor, finished: torch.Tensor, eos: int, pad: int,
-                    n_alive: Optional[torch.Tensor]) -> None:
-        N.check(self.lib.pgmi_eos_update(self.ctx, next_ids.data_ptr(), finished.data_ptr(), next_ids.numel(), eos, pad,
-                                         n_alive.data_ptr() if n_alive is not None else None, self._s()),
-                "pgmi_eos_update")
+        def decode_one(cur, t, step_logits, next_ids):
+            self.decode(cur, kv, L + t - 1, L + t, logits=step_logits, next_ids=next_ids, graph=graph)
+
+        def decode_many(cur, t, n, step_logits, rec):
+            self.decode_steps(cur, kv, L + t - 1, L + t, n, logits=step_logits, tokens=rec, graph=graph)
+
+        return self._generate_loop(logits[:, 0], n_tokens, decode_one, decode_many, graph, do_sample, temperature, top_p,
+                                   generator, eos_token_id, pad_token_id, sync_every, return_lengths)

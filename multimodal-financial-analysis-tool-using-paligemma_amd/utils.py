@@ -9,11 +9,11 @@ tensor raises (the reference's strict=False / ImportError paths silently kept ra
 from __future__ import annotations
 
 import glob
-import json
 import os
 
 import torch
 
+from pgmi import registry
 from modeling_gemma import PaliGemmaConfig, PaliGemmaForConditionalGeneration
 
 
@@ -74,9 +74,12 @@ def load_hf_model(model_path, device="cuda", native: bool = True):
 
 def load_model(model_path, device="cuda", native: bool = True):
     """config.json + *.safetensors -> PaliGemmaForConditionalGeneration (utils.py:6-46 without the
-    tokenizer).  native: libpgmi's reader fills the engine slab; else safe_open per tensor."""
-    with open(f"{model_path}/config.json", "r") as f:
-        config = PaliGemmaConfig(**json.load(f))
+    tokenizer), or a pgmi.DecoderEngine for a layered decoder's checkpoint (pgmi/registry.py).
+    native: libpgmi's reader fills the engine slab; else safe_open per tensor."""
+    cfg = registry.read_config(model_path)
+    if registry.family(cfg) == "decoder":
+        return registry.load_decoder(model_path, device=device)
+    config = PaliGemmaConfig(**cfg)
     model = build_model(config, device=device)
     if native and torch.device(device).type == "cuda":
         model.tie_weights()  # the engine binds the tied tree (lm_head = embed_tokens, utils.py:44)
