@@ -356,6 +356,13 @@ int pgmi_op_rope(pgmi_ctx* ctx, const void* x, const void* cos_rows, const void*
                  int head_dim, void* out, void* stream);
 /* out = bf16(x * a) over n bf16 values (n a multiple of 8): GemmaModel's normalizer (modeling_gemma.py:367-368) */
 int pgmi_op_scale(pgmi_ctx* ctx, const void* x, float a, int64_t n, void* out, void* stream);
+/* the layered decoders' product on its own (any context): A [M][lda] x W [N][ldw]^T (W bf16; K % 8 == 0).  act:
+ * PGMI_DTYPE_BF16 / _F32 activations; mode 0: activation-type out [M][ldo] (+ bias), 1: fp32 out [M][N], 2: as 1 in
+ * *split partial slabs [split][M][N] (out_bytes bounds them), 3: silu(gate) * up with W = N gate rows, then N up
+ * rows (fp32 activations: scratch [M][2N]) */
+int pgmi_op_matmul(pgmi_ctx* ctx, const void* A, int lda, const void* W, int ldw, int M, int N, int K, int act,
+                   int mode, const void* bias, void* out, int ldo, int64_t out_bytes, void* scratch, int* split,
+                   void* stream);
 /* decode GEMV family on one layer's weights (tests): y[b][n] += W x (residual form) */
 int pgmi_op_gemv_res(pgmi_ctx* ctx, const void* x, const void* W, int B, int N, int K, void* h_inout,
                      void* stream);

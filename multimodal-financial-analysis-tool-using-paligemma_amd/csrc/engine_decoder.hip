@@ -842,4 +842,22 @@ int pgmi_decoder_decode(pgmi_ctx* x, const int64_t* ids, int B, const int32_t* s
     return 0;
 }
 
+int pgmi_op_matmul(pgmi_ctx* x, const void* A, int lda, const void* W, int ldw, int M, int N, int K, int act, int mode,
+                   const void* bias, void* out, int ldo, int64_t out_bytes, void* scratch, int* split, void* stream) {
+    if (!x || !A || !W || !out) return fail(PGMI_E_ARG, "null argument");
+    if (M < 1 || N < 1 || K < 8 || K % 8 != 0 || lda < K || ldw < K || lda % 8 != 0 || ldw % 8 != 0)
+        return fail(PGMI_E_ARG, "K, lda, ldw must be multiples of 8 with lda, ldw >= K");
+    if (act != PGMI_DTYPE_BF16 && act != PGMI_DTYPE_F32) return fail(PGMI_E_ARG, "activations are bf16 or fp32");
+    if (mode < 0 || mode > 3) return fail(PGMI_E_ARG, "unknown mode");
+    if ((mode == RT_ACT || mode == RT_SWIGLU) && ldo < N) return fail(PGMI_E_ARG, "ldo < N");
+    if (mode == RT_SWIGLU && act == PGMI_DTYPE_F32 && !scratch) return fail(PGMI_E_ARG, "fp32 gate|up needs scratch");
+    const int sp = matmul_rt((hipStream_t)stream, act == PGMI_DTYPE_F32 ? ACT_F32 : ACT_BF16, A, lda,
+                             reinterpret_cast<const uint16_t*>(W), ldw, M, N, K, (RtOut)mode,
+                             reinterpret_cast<const uint16_t*>(bias), out, ldo, (size_t)std::max<int64_t>(out_bytes, 0),
+                             reinterpret_cast<float*>(scratch));
+    if (split) *split = sp;
+    LAUNCHCHK();
+    return 0;
+}
+
 }  // extern "C"

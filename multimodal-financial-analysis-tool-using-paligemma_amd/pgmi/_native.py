@@ -116,6 +116,7 @@ SIGNATURES = {
     "pgmi_op_scale": (i32, [vp, vp, f32, i64, vp, vp]),
     "pgmi_decoder_create": (i32, [i32, ctypes.POINTER(DecoderConfigC), ctypes.POINTER(LayerSpec), ctypes.POINTER(vp)]),
     "pgmi_decoder_forward": (i32, [vp, vp, i32, vp, vp, vp, vp, i32, i32, vp, i32, vp, vp, vp]),
+    "pgmi_op_matmul": (i32, [vp, vp, i32, vp, i32, i32, i32, i32, i32, i32, vp, vp, i32, i64, vp, ctypes.POINTER(i32), vp]),
     "pgmi_decoder_decode": (i32, [vp, vp, i32, vp, vp, vp, i32, i32, i32, vp, vp, vp, i32, vp]),
 }
 

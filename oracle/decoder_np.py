@@ -276,8 +276,10 @@ def random_weights(cfg, seed):
             w = rng.uniform(-4.0, 0.5, shp)
         elif leaf.endswith(".b"):
             w = 0.3 * r
+        elif leaf in ("mix.o", "mlp.down"):
+            w = r * (0.8 / np.sqrt(shp[-1]))
         else:
-            w = r * (1.3 / np.sqrt(shp[-1]))
+            w = r * (1.1 / np.sqrt(shp[-1]))
         u = np.ascontiguousarray(w, np.float32).view(np.uint32)
         u = (u + np.uint32(0x7FFF) + ((u >> np.uint32(16)) & np.uint32(1))) & np.uint32(0xFFFF0000)
         W[n] = u.view(np.float32).reshape(shp)
