@@ -40,6 +40,34 @@ __device__ __forceinline__ float sigmoidf_(float x) { return 1.0f / (1.0f + __ex
 __device__ __forceinline__ float siluf_(float x) { return x / (1.0f + __expf(-x)); }
 // ln(1 + exp(x)) without overflow or cancellation
 __device__ __forceinline__ float softplusf_(float x) { return fmaxf(x, 0.0f) + log1pf(__expf(-fabsf(x))); }
+// the same from the hardware exponential and logarithm: a short series where 1 + e would round e away
+__device__ __forceinline__ float softplus_fast(float x) {
+    const float e = __expf(-fabsf(x));
+    const float series = e * (1.0f - e * (0.5f - e * (0.33333333f - e * (0.25f - e * 0.2f))));
+    return fmaxf(x, 0.0f) + (e < 0.0625f ? series : __logf(1.0f + e));
+}
+template <typename T>
+__device__ __forceinline__ float softplus_of(float x);
+template <>
+__device__ __forceinline__ float softplus_of<float>(float x) { return softplusf_(x); }
+template <>
+__device__ __forceinline__ float softplus_of<uint16_t>(float x) { return softplus_fast(x); }
+
+__device__ __forceinline__ void ld4(const uint16_t* p, float (&v)[4]) {
+    const ushort4 u = *reinterpret_cast<const ushort4*>(p);
+    v[0] = bf2f(u.x); v[1] = bf2f(u.y); v[2] = bf2f(u.z); v[3] = bf2f(u.w);
+}
+__device__ __forceinline__ void ld4(const float* p, float (&v)[4]) {
+    const float4 u = *reinterpret_cast<const float4*>(p);
+    v[0] = u.x; v[1] = u.y; v[2] = u.z; v[3] = u.w;
+}
+__device__ __forceinline__ void st4(uint16_t* p, const float (&v)[4]) {
+    *reinterpret_cast<ushort4*>(p) = make_ushort4(f2bf(v[0]), f2bf(v[1]), f2bf(v[2]), f2bf(v[3]));
+}
+__device__ __forceinline__ void st4(float* p, const float (&v)[4]) {
+    *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+}
+
 // minGRU's candidate: u + 1/2 for u >= 0, sigmoid(u) below
 __device__ __forceinline__ float gru_candidate(float u) { return u >= 0.0f ? u + 0.5f : sigmoidf_(u); }
 

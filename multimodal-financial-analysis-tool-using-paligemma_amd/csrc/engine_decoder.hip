@@ -47,8 +47,8 @@ struct DecoderState {
     const uint16_t *embed = nullptr, *fnorm = nullptr;
     Lin head;
     std::vector<void*> derived;  // padded weights, joined biases
-    // workspace of `rows` rows and `chunks` scan chunks
-    int rows = 0, chunks = 0;
+    // workspace of `rows` rows, `chunks` scan chunks and `gchunks` chunks of the gated recurrence
+    int rows = 0, chunks = 0, gchunks = 0;
     void* arena = nullptr;
     float *X = nullptr, *slabs = nullptr, *dt = nullptr, *bc = nullptr, *cstate = nullptr, *csum = nullptr;
     uint8_t *h = nullptr, *p0 = nullptr, *p1 = nullptr, *p2 = nullptr, *dtl = nullptr;
@@ -69,8 +69,6 @@ struct DecoderState {
 };
 
 namespace {
-
-constexpr int kGemvParts = 2048;
 
 std::string lname(int i, const char* s) { return "l" + std::to_string(i) + "." + s; }
 
@@ -254,8 +252,8 @@ int decoder_prepare(pgmi_ctx* x) {
         if ((rc = dalloc_t(x, &d.pos, (size_t)B))) return rc;
         if ((rc = dalloc_t(x, &d.d_ids, (size_t)B))) return rc;
         if ((rc = dalloc_t(x, &d.d_next, (size_t)B))) return rc;
-        if ((rc = dalloc_t(x, &d.pmax, (size_t)gemv_rt_max_batch() * kGemvParts))) return rc;
-        if ((rc = dalloc_t(x, &d.pidx, (size_t)gemv_rt_max_batch() * kGemvParts))) return rc;
+        if ((rc = dalloc_t(x, &d.pmax, (size_t)gemv_rt_parts()))) return rc;
+        if ((rc = dalloc_t(x, &d.pidx, (size_t)gemv_rt_parts()))) return rc;
         HIPCHK(hipStreamCreateWithFlags(&x->cap_stream, hipStreamNonBlocking));
     }
     HIPCHK(hipDeviceSynchronize());
@@ -274,17 +272,18 @@ void decoder_release(pgmi_ctx* x) {
     x->dec = nullptr;
 }
 
-// Grow the workspace to `rows` rows and `chunks` scan chunks (captured graphs hold its addresses)
-int ensure_workspace(pgmi_ctx* x, int rows, int chunks) {
+// Grow the workspace to these rows and chunks (captured graphs hold its addresses)
+int ensure_workspace(pgmi_ctx* x, int rows, int chunks, int gchunks) {
     DecoderState& d = *x->dec;
-    if (rows <= d.rows && chunks <= d.chunks) return 0;
+    if (rows <= d.rows && chunks <= d.chunks && gchunks <= d.gchunks) return 0;
     rows = std::max(rows, d.rows);
     chunks = std::max(chunks, d.chunks);
+    gchunks = std::max(gchunks, d.gchunks);
     HIPCHK(hipDeviceSynchronize());
     clear_dgraphs(x);
     if (d.arena) (void)hipFree(d.arena);
     d.arena = nullptr;
-    d.rows = d.chunks = 0;
+    d.rows = d.chunks = d.gchunks = 0;
     const int D = d.c.width;
     int l0 = 8, l1 = 8, l2 = 8, ldd = 8, slab_n = D, inner = 1, bcn = 2, cs = 1, cg = 1;
     for (const pgmi_layer_spec& l : d.L) {
@@ -314,11 +313,10 @@ int ensure_workspace(pgmi_ctx* x, int rows, int chunks) {
     d.ldh = r8(D);
     d.ld0 = l0; d.ld1 = l1; d.ld2 = l2; d.ldd = ldd;
     d.slab_bytes = std::max<size_t>((size_t)rows * slab_n * 4, (size_t)32 << 20);
-    cs = std::max(cs, 2 * cg);
     const size_t sizes[] = {(size_t)rows * d.c.streams * D * 4, (size_t)rows * d.ldh * d.es, (size_t)rows * l0 * d.es,
                             (size_t)rows * l1 * d.es,           (size_t)rows * l2 * d.es,    (size_t)rows * ldd * d.es,
                             d.slab_bytes,                       (size_t)rows * inner * 4,    (size_t)rows * bcn * 4,
-                            (size_t)chunks * cs * 4,            (size_t)chunks * inner * 4};
+                            std::max((size_t)chunks * cs, (size_t)gchunks * 2 * cg) * 4, (size_t)chunks * inner * 4};
     size_t off[11], total = 0;
     for (int i = 0; i < 11; ++i) {
         off[i] = total;
@@ -339,6 +337,7 @@ int ensure_workspace(pgmi_ctx* x, int rows, int chunks) {
     d.csum = reinterpret_cast<float*>(p + off[10]);
     d.rows = rows;
     d.chunks = chunks;
+    d.gchunks = gchunks;
     return 0;
 }
 
@@ -370,9 +369,11 @@ T* at(void* state, int64_t off) { return reinterpret_cast<T*>(reinterpret_cast<u
 struct Meta {
     const SeqInfo* seqs;
     int nseq;
-    const ChunkInfo* chunks;
-    int nchunk;
-    bool multi;
+    struct Chunks {
+        const ChunkInfo* p;
+        int n;
+        bool multi;  // some sequence has more than one
+    } scan, gru;
     const int* row_seq;
     const int* want;
     std::map<int, std::pair<const ChunkInfo*, int>> tiles;  // by query heads per key/value head
@@ -407,7 +408,7 @@ int forward_body(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int rows, const
         if (l.mixer == PGMI_MIXER_MAMBA1) {
             const int C = l.inner, N = l.state, R = l.dt_rank, ldc = r8(C), ldxz = r8(2 * C), ldd = r8(R);
             matmul_rt(s, d.act, d.h, d.ldh, w.in.w, w.in.ldw, rows, 2 * C, w.in.k, RT_ACT, nullptr, d.p0, ldxz, 0, nullptr);
-            conv_silu(s, d.act, d.p0, ldxz, C, l.conv, w.conv, w.conv_b, m.seqs, m.nseq, m.chunks, m.nchunk,
+            conv_silu(s, d.act, d.p0, ldxz, C, l.conv, w.conv, w.conv_b, m.seqs, m.nseq, m.scan.p, m.scan.n,
                       at<float>(state, st[i].a), d.p1, ldc);
             const int sp = matmul_rt(s, d.act, d.p1, ldc, w.x.w, w.x.ldw, rows, R + 2 * N, w.x.k, RT_SLABS, nullptr, d.slabs,
                                      0, d.slab_bytes, nullptr);
@@ -416,8 +417,8 @@ int forward_body(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int rows, const
             ScanArgs a{};
             a.dt = d.dt; a.dtb = w.dt_b; a.x = d.p1; a.ldx = ldc; a.z = d.p0 + (size_t)C * d.es; a.ldz = ldxz; a.bc = d.bc;
             a.A_log = w.A_log; a.Dw = w.D; a.state = at<float>(state, st[i].b); a.cstate = d.cstate; a.csum = d.csum;
-            a.y = d.p2; a.ldy = ldc; a.C = C; a.N = N; a.seqs = m.seqs; a.nseq = m.nseq; a.chunks = m.chunks;
-            a.nchunk = m.nchunk; a.multi = m.multi;
+            a.y = d.p2; a.ldy = ldc; a.C = C; a.N = N; a.seqs = m.seqs; a.nseq = m.nseq; a.chunks = m.scan.p;
+            a.nchunk = m.scan.n; a.multi = m.scan.multi;
             selective_scan(s, d.act, a);
             out_proj(w.o, d.p2, ldc, w.sub[0]);
         } else if (l.mixer == PGMI_MIXER_ATTENTION) {
@@ -438,7 +439,7 @@ int forward_body(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int rows, const
             matmul_rt(s, d.act, d.h, d.ldh, w.in.w, w.in.ldw, rows, 3 * C, w.in.k, RT_ACT, w.bias, d.p0, ldz, 0, nullptr);
             GruArgs a{};
             a.zug = d.p0; a.ld = ldz; a.state = at<float>(state, st[i].a); a.cstate = d.cstate; a.y = d.p2; a.ldy = ldc;
-            a.C = C; a.seqs = m.seqs; a.nseq = m.nseq; a.chunks = m.chunks; a.nchunk = m.nchunk; a.multi = m.multi;
+            a.C = C; a.seqs = m.seqs; a.nseq = m.nseq; a.chunks = m.gru.p; a.nchunk = m.gru.n; a.multi = m.gru.multi;
             mingru_scan(s, d.act, a);
             out_proj(w.o, d.p2, ldc, w.sub[0]);
         }
@@ -484,7 +485,7 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
     Pending pend;
     // the input side of a projection: d.h, or (fused) the streams' read and norm inside the GEMV
     auto base = [&](const Sub& sub, const Lin& w, bool fused) {
-        if (!have_h && (!fused || pend.y)) {
+        if (!have_h && (!fused || pend.y || !gemv_rt_reads_streams(B))) {
             StreamsArgs a = streams_args(d, B);
             fold(a, pend, B);
             a.in = sub.in; a.w = sub.norm;
@@ -596,7 +597,9 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
     if (fl) {
         g.out = logits; g.ldo = V; g.pmax = d.pmax; g.pidx = d.pidx;
         gemv_rt(s, d.act, GR_LOGITS, g);
-        decode_finish(s, B, d.pmax, d.pidx, gemv_rt_blocks(g, GR_LOGITS), next, hist, d.pos);
+        const int parts = gemv_rt_reads_streams(B) ? gemv_rt_blocks(g, GR_LOGITS) : 0;
+        if (!parts) argmax_rows(s, logits, B, V, x->amax_v, x->amax_i, next);
+        decode_finish(s, B, d.pmax, d.pidx, parts, next, hist, d.pos);
     } else {
         matmul_rt(s, d.act, d.h, d.ldh, d.head.w, d.head.ldw, B, V, d.head.k, RT_F32, nullptr, logits, V, 0, nullptr);
         argmax_rows(s, logits, B, V, x->amax_v, x->amax_i, next);
@@ -693,20 +696,21 @@ int pgmi_decoder_forward(pgmi_ctx* x, const int64_t* ids, int n_seq, const int32
     HIPCHK(hipSetDevice(x->device));
     hipStream_t s = (hipStream_t)stream;
     // metadata: sequences, scan chunks, attention tiles per head grouping, row -> sequence, wanted rows
-    const int ct = rows <= 16384 ? 64 : 256;
     std::vector<int>& m = d.host;
     m.clear();
     auto put = [&](std::initializer_list<int> v) { m.insert(m.end(), v); };
-    size_t o_seq = 0;
     for (int r = 0, off = 0; r < n_seq; off += lens[r], ++r) put({off, lens[r], starts[r], slots[r]});
-    const size_t o_chunk = m.size();
-    int nchunk = 0;
-    bool multi = false;
-    for (int r = 0, off = 0; r < n_seq; off += lens[r], ++r) {
-        const int n = (lens[r] + ct - 1) / ct;
-        multi |= n > 1;
-        for (int k = 0; k < n; ++k, ++nchunk) put({r, off + k * ct, std::min(ct, lens[r] - k * ct), k * ct, k, n});
-    }
+    struct Cut { size_t o; int n; bool multi; };
+    auto cut = [&](int ct) {
+        Cut c{m.size(), 0, false};
+        for (int r = 0, off = 0; r < n_seq; off += lens[r], ++r) {
+            const int n = (lens[r] + ct - 1) / ct;
+            c.multi |= n > 1;
+            for (int k = 0; k < n; ++k, ++c.n) put({r, off + k * ct, std::min(ct, lens[r] - k * ct), k * ct, k, n});
+        }
+        return c;
+    };
+    const Cut scan = cut(rows <= 16384 ? 64 : 256), gru = cut(rows <= 16384 ? 32 : 128);
     struct Tiles { int R; size_t o; int n; };
     std::vector<Tiles> tiles;
     for (const pgmi_layer_spec& l : d.L) {
@@ -724,7 +728,7 @@ int pgmi_decoder_forward(pgmi_ctx* x, const int64_t* ids, int n_seq, const int32
     for (int r = 0; r < n_seq; ++r) m.insert(m.end(), lens[r], r);
     const size_t o_want = m.size();
     m.insert(m.end(), want, want + n_want);
-    if ((rc = ensure_workspace(x, std::max(rows, n_want), nchunk))) return rc;
+    if ((rc = ensure_workspace(x, std::max(rows, n_want), scan.n, gru.n))) return rc;
     if (m.size() * 4 > d.meta_bytes) {
         HIPCHK(hipDeviceSynchronize());
         if (d.meta) (void)hipFree(d.meta);
@@ -740,11 +744,10 @@ int pgmi_decoder_forward(pgmi_ctx* x, const int64_t* ids, int n_seq, const int32
     HIPCHK(hipMemcpyAsync(d.meta, m.data(), m.size() * 4, hipMemcpyHostToDevice, s));
     const int* dm = reinterpret_cast<const int*>(d.meta);
     Meta meta{};
-    meta.seqs = reinterpret_cast<const SeqInfo*>(dm + o_seq);
+    meta.seqs = reinterpret_cast<const SeqInfo*>(dm);
     meta.nseq = n_seq;
-    meta.chunks = reinterpret_cast<const ChunkInfo*>(dm + o_chunk);
-    meta.nchunk = nchunk;
-    meta.multi = multi;
+    meta.scan = {reinterpret_cast<const ChunkInfo*>(dm + scan.o), scan.n, scan.multi};
+    meta.gru = {reinterpret_cast<const ChunkInfo*>(dm + gru.o), gru.n, gru.multi};
     meta.row_seq = dm + o_row;
     meta.want = dm + o_want;
     for (const Tiles& t : tiles) meta.tiles[t.R] = {reinterpret_cast<const ChunkInfo*>(dm + t.o), t.n};
@@ -765,7 +768,7 @@ int pgmi_decoder_decode(pgmi_ctx* x, const int64_t* ids, int B, const int32_t* s
         if (positions[b] < 0 || (long)positions[b] + n_steps > max_tokens) return fail(PGMI_E_ARG, "state capacity exceeded");
     HIPCHK(hipSetDevice(x->device));
     hipStream_t s = (hipStream_t)stream;
-    if ((rc = ensure_workspace(x, B, 1))) return rc;
+    if ((rc = ensure_workspace(x, B, 1, 1))) return rc;
     size_t need = 0;
     for (const pgmi_layer_spec& l : d.L)
         if (l.mixer == PGMI_MIXER_ATTENTION)

@@ -1,5 +1,5 @@
-// kernels_step.hip -- one token per sequence: projections as weight-streaming GEMVs of any size with the
-// surrounding steps fused (streams' read + grouped norm in front; convolution step, minGRU step, gated
+// kernels_step.hip -- one token per sequence: projections as weight-streaming GEMVs (1 or 2 rows) or skinny MFMA
+// products (3 .. 16 rows) of any size with the surrounding steps fused (streams' read + grouped norm in front; convolution step, minGRU step, gated
 // activation, streams' update or argmax behind), and the selective-scan step.
 #include <algorithm>
 
@@ -31,35 +31,94 @@ constexpr int unit_rows(int mode) { return mode == GR_GRU ? 3 : 2; }
 // outputs a unit covers (plain modes: two rows; GRU, SwiGLU: one channel)
 constexpr int unit_outs(int mode) { return mode == GR_GRU || mode == GR_SWIGLU ? 1 : 2; }
 
-template <typename T, int NB, int MODE>
+// The step that follows a projection, for output n of row b (v: its sum over K; GR_GRU: v = z, v1 = u, v2 = g;
+// GR_SWIGLU: v = gate, v1 = up).  Every (n, b) is handled by one thread.
+template <typename T, int MODE>
+__device__ __forceinline__ void step_epilogue(const GemvRtArgs& a, int n, int b, float v, float v1, float v2) {
+    if constexpr (MODE == GR_ACT) {
+        if (a.bias) v += bf2f(a.bias[n]);
+        stf(reinterpret_cast<T*>(a.out) + (long)b * a.ldo + n, v);
+    } else if constexpr (MODE == GR_LOGITS || MODE == GR_F32) {
+        reinterpret_cast<float*>(a.out)[(long)b * a.ldo + n] = v;
+    } else if constexpr (MODE == GR_CONV) {
+        if (n < a.C) {
+            const int KT = a.taps_k;
+            float* tp = a.state + (long)a.slot[b] * (KT - 1) * a.C + n;
+            const bool first = a.pos[b] == 0;
+            const uint16_t* cw = a.cw + (long)n * KT;
+            float y = fmaf(bf2f(cw[KT - 1]), v, bf2f(a.cb[n]));
+            for (int j = 0; j < KT - 1; ++j) {
+                const float o = first ? 0.0f : tp[(long)j * a.C];
+                y = fmaf(bf2f(cw[j]), o, y);
+                if (j > 0) tp[(long)(j - 1) * a.C] = o;
+            }
+            if (KT > 1) tp[(long)(KT - 2) * a.C] = v;
+            stf(reinterpret_cast<T*>(a.out) + (long)b * a.ldo + n, siluf_(y));
+        } else {
+            stf(reinterpret_cast<T*>(a.out2) + (long)b * a.ldo2 + n - a.C, v);
+        }
+    } else if constexpr (MODE == GR_GRU) {
+        const float z = sigmoidf_(v + bf2f(a.bias[n]));
+        float* st = a.state + (long)a.slot[b] * a.N + n;
+        const float S = fmaf(1.0f - z, a.pos[b] > 0 ? *st : 0.0f, z * gru_candidate(v1 + bf2f(a.bias[a.N + n])));
+        *st = S;
+        stf(reinterpret_cast<T*>(a.out) + (long)b * a.ldo + n, S * siluf_(v2));
+    } else if constexpr (MODE == GR_SWIGLU) {
+        stf(reinterpret_cast<T*>(a.out) + (long)b * a.ldo + n, siluf_(v) * v1);
+    } else {  // GR_STREAMS: the whole column of streams at once
+        float* Xr = a.X + (long)b * a.S * a.D + n;
+        float x[8];
+#pragma unroll
+        for (int s = 0; s < 8; ++s) x[s] = s < a.S ? Xr[(long)s * a.D] : 0.0f;
+        for (int t = 0; t < a.S; ++t) {
+            float y = bf2f(a.wout[t]) * v;
+#pragma unroll
+            for (int s = 0; s < 8; ++s)
+                if (s < a.S) y = fmaf(bf2f(a.mix[s * a.S + t]), x[s], y);
+            Xr[(long)t * a.D] = y;
+        }
+    }
+}
+
+// the columns that pad an activation row to a multiple of 8 are zero
+template <typename T, int MODE>
+__device__ __forceinline__ void step_pads(const GemvRtArgs& a) {
+    if constexpr (MODE == GR_GRU || MODE == GR_SWIGLU || MODE == GR_CONV) {
+        const int n = MODE == GR_CONV ? a.C : a.N;
+        if (blockIdx.x == 0 && (int)threadIdx.x < a.B)
+            for (int k = n; k < a.ldo; ++k) stf(reinterpret_cast<T*>(a.out) + (long)threadIdx.x * a.ldo + k, 0.0f);
+    }
+}
+
+// WK: waves of the workgroup that share a unit, each a K slice
+template <typename T, int NB, int MODE, int WK>
 __global__ void __launch_bounds__(256) k_gemv_rt(GemvRtArgs a) {
-    constexpr int RW = unit_rows(MODE), UO = unit_outs(MODE);
+    constexpr int RW = unit_rows(MODE), UO = unit_outs(MODE), UPB = 4 / WK;
     extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
     T* xs = reinterpret_cast<T*>(smem);  // [NB][K]
-    __shared__ float red[4];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    __shared__ float red[64];
+    __shared__ float part[WK > 1 ? 4 : 1][RW * NB];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int nunit = (a.N + UO - 1) / UO, K = a.K;
-    int unit = blockIdx.x * 4 + wave;
-    uint4 w[RW][UN];
-    auto wrow = [&](int u, int r) -> long {
-        int n;
-        if constexpr (UO == 1) n = r * a.N + u;
-        else { n = u * 2 + r; n = n < a.N ? n : a.N - 1; }
-        return n;
-    };
-    auto wload = [&](int u, int k0) {
+    const int ustep = gridDim.x * UPB, kw = wave % WK;
+    int unit = blockIdx.x * UPB + wave / WK;
+    uint4 w[2][RW][UN];
+    auto wload = [&](uint4 (&q)[RW][UN], int u, int k0) {
         const int uu = u < nunit ? u : nunit - 1;
 #pragma unroll
         for (int r = 0; r < RW; ++r) {
-            const uint16_t* p = a.W + wrow(uu, r) * a.ldw;
+            int n;
+            if constexpr (UO == 1) n = r * a.N + uu;
+            else { n = uu * 2 + r; n = n < a.N ? n : a.N - 1; }
+            const uint16_t* p = a.W + (long)n * a.ldw;
 #pragma unroll
             for (int i = 0; i < UN; ++i) {
-                const int k = k0 + i * 512 + lane * 8;
-                w[r][i] = ldg16_sel(p + k, k < K, p);
+                const int k = k0 + (i * WK + kw) * 512 + lane * 8;
+                q[r][i] = ldg16_sel(p + k, k < K, p);
             }
         }
     };
-    wload(unit, 0);  // in flight during the prologue
+    wload(w[0], unit, 0);  // in flight during the prologue
     if (a.x) {
         for (int e = tid * 8; e < NB * K; e += 256 * 8) {
             const int b = e / K, k = e % K;
@@ -68,38 +127,72 @@ __global__ void __launch_bounds__(256) k_gemv_rt(GemvRtArgs a) {
             st8(xs + b * K + k, v);
         }
     } else {
-        // the streams' read and grouped norm of each row (fp32 in registers / LDS), as streams_norm
+        // the streams' read and grouped norm of each row, as streams_norm
         float* u_ = reinterpret_cast<float*>(smem + (size_t)NB * K * sizeof(T));  // [D], then [groups]
         float* inv = u_ + a.D;
-        const int P = a.D / a.groups;
+        const int P = a.D / a.groups, D = a.D;
         for (int b = 0; b < NB && b < a.B; ++b) {
-            const float* Xr = a.X + (long)b * a.S * a.D;
-            for (int d = tid; d < a.D; d += 256) {
+            const float* Xr = a.X + (long)b * a.S * D;
+            if (P % 256 == 0 && D <= 8192) {
+                // a wave's 64 x 4 elements lie in one group: one partial per (piece, wave)
+                constexpr int PC = 8;
+                const int np = (D + 1023) / 1024;
+                float4 u[PC];
+                ushort4 nw[PC];
+#pragma unroll
+                for (int i = 0; i < PC; ++i) {
+                    u[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+                    nw[i] = make_ushort4(0, 0, 0, 0);
+                    const int d = i * 1024 + tid * 4;
+                    if (i < np && d < D) {
+                        nw[i] = *reinterpret_cast<const ushort4*>(a.nw + d);
+                        for (int s = 0; s < a.S; ++s) {
+                            const float c = a.in ? bf2f(a.in[s]) : 1.0f;
+                            const float4 q = *reinterpret_cast<const float4*>(Xr + (long)s * D + d);
+                            u[i].x = fmaf(c, q.x, u[i].x); u[i].y = fmaf(c, q.y, u[i].y);
+                            u[i].z = fmaf(c, q.z, u[i].z); u[i].w = fmaf(c, q.w, u[i].w);
+                        }
+                    }
+                }
+#pragma unroll
+                for (int i = 0; i < PC; ++i)
+                    if (i < np) {
+                        const float q = wave_sum(u[i].x * u[i].x + u[i].y * u[i].y + u[i].z * u[i].z + u[i].w * u[i].w);
+                        if (lane == 0) red[i * 4 + wave] = q;
+                    }
+                __syncthreads();
+#pragma unroll
+                for (int i = 0; i < PC; ++i) {
+                    const int d = i * 1024 + tid * 4;
+                    if (i < np && d < D) {
+                        const int p0 = d / P * (P / 256);
+                        float q = 0.0f;
+                        for (int t = 0; t < P / 256; ++t) q += red[p0 + t];
+                        const float f = 1.0f / sqrtf(q / (float)P + a.eps);
+                        T* o = xs + b * K + d;
+                        stf(o, u[i].x * f * bf2f(nw[i].x));
+                        stf(o + 1, u[i].y * f * bf2f(nw[i].y));
+                        stf(o + 2, u[i].z * f * bf2f(nw[i].z));
+                        stf(o + 3, u[i].w * f * bf2f(nw[i].w));
+                    }
+                }
+                __syncthreads();
+                continue;
+            }
+            for (int d = tid; d < D; d += 256) {
                 float u = 0.0f;
-                for (int s = 0; s < a.S; ++s) u = fmaf(a.in ? bf2f(a.in[s]) : 1.0f, Xr[(long)s * a.D + d], u);
+                for (int s = 0; s < a.S; ++s) u = fmaf(a.in ? bf2f(a.in[s]) : 1.0f, Xr[(long)s * D + d], u);
                 u_[d] = u;
             }
             __syncthreads();
-            if (a.groups >= 4) {
-                for (int g = wave; g < a.groups; g += 4) {
-                    float q = 0.0f;
-                    for (int i = lane; i < P; i += 64) q = fmaf(u_[g * P + i], u_[g * P + i], q);
-                    q = wave_sum(q);
-                    if (lane == 0) inv[g] = 1.0f / sqrtf(q / (float)P + a.eps);
-                }
-                __syncthreads();
-            } else {
-                for (int g = 0; g < a.groups; ++g) {
-                    float q = 0.0f;
-                    for (int i = tid; i < P; i += 256) q = fmaf(u_[g * P + i], u_[g * P + i], q);
-                    q = wave_sum(q);
-                    if (lane == 0) red[wave] = q;
-                    __syncthreads();
-                    if (tid == 0) inv[g] = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)P + a.eps);
-                    __syncthreads();
-                }
+            for (int g = wave; g < a.groups; g += 4) {
+                float q = 0.0f;
+                for (int i = lane; i < P; i += 64) q = fmaf(u_[g * P + i], u_[g * P + i], q);
+                q = wave_sum(q);
+                if (lane == 0) inv[g] = 1.0f / sqrtf(q / (float)P + a.eps);
             }
-            for (int d = tid; d < K; d += 256) stf(xs + b * K + d, d < a.D ? u_[d] * inv[d / P] * bf2f(a.nw[d]) : 0.0f);
+            __syncthreads();
+            for (int d = tid; d < K; d += 256) stf(xs + b * K + d, d < D ? u_[d] * inv[d / P] * bf2f(a.nw[d]) : 0.0f);
             __syncthreads();
         }
     }
@@ -108,103 +201,82 @@ __global__ void __launch_bounds__(256) k_gemv_rt(GemvRtArgs a) {
     int bi[NB];
 #pragma unroll
     for (int b = 0; b < NB; ++b) { best[b] = -INFINITY; bi[b] = 0x7fffffff; }
-    for (; unit < nunit; unit += gridDim.x * 4) {
-        float acc[RW][NB];
+    float acc[RW][NB];
+    auto mac = [&](const uint4 (&q)[RW][UN], int k0) {
+#pragma unroll
+        for (int i = 0; i < UN; ++i) {
+            const int k = k0 + (i * WK + kw) * 512 + lane * 8;
+            if (k < K) {
+#pragma unroll
+                for (int b = 0; b < NB; ++b)
+#pragma unroll
+                    for (int r = 0; r < RW; ++r) acc[r][b] = dotx(q[r][i], xs + b * K + k, acc[r][b]);
+            }
+        }
+    };
+    constexpr int KB = UN * WK * 512;  // K elements per block
+    // every wave of a workgroup runs the same number of rounds (WK > 1 meets at a barrier)
+    for (int u0 = blockIdx.x * UPB; u0 < nunit; u0 += ustep, unit += ustep) {
 #pragma unroll
         for (int r = 0; r < RW; ++r)
 #pragma unroll
             for (int b = 0; b < NB; ++b) acc[r][b] = 0.0f;
-        for (int k0 = 0; k0 < K; k0 += UN * 512) {
-#pragma unroll
-            for (int i = 0; i < UN; ++i) {
-                const int k = k0 + i * 512 + lane * 8;
-                if (k < K) {
-#pragma unroll
-                    for (int b = 0; b < NB; ++b)
-#pragma unroll
-                        for (int r = 0; r < RW; ++r) acc[r][b] = dotx(w[r][i], xs + b * K + k, acc[r][b]);
-                }
+        for (int k0 = 0; k0 < K; k0 += 2 * KB) {
+            if (k0 + KB < K) wload(w[1], unit, k0 + KB);
+            mac(w[0], k0);
+            if (k0 + KB < K) {
+                if (k0 + 2 * KB < K) wload(w[0], unit, k0 + 2 * KB);
+                mac(w[1], k0 + KB);
             }
-            if (k0 + UN * 512 < K) wload(unit, k0 + UN * 512);
         }
-        if (unit + (int)gridDim.x * 4 < nunit) wload(unit + gridDim.x * 4, 0);
+        if (u0 + ustep < nunit) wload(w[0], unit + ustep, 0);
 #pragma unroll
         for (int r = 0; r < RW; ++r)
 #pragma unroll
             for (int b = 0; b < NB; ++b) acc[r][b] = wave_sum(acc[r][b]);
-        if constexpr (MODE == GR_GRU || MODE == GR_SWIGLU) {
-            const int c = unit;
+        if constexpr (WK > 1) {
+            __syncthreads();
+            if (lane == 0)
 #pragma unroll
-            for (int b = 0; b < NB; ++b) {
-                if (lane == b && b < a.B) {
-                    float y;
-                    if constexpr (MODE == GR_GRU) {
-                        float zr = acc[0][b] + bf2f(a.bias[c]), ur = acc[1][b] + bf2f(a.bias[a.N + c]);
-                        const float z = sigmoidf_(zr);
-                        float* st = a.state + (long)a.slot[b] * a.N + c;
-                        const float S = fmaf(1.0f - z, a.pos[b] > 0 ? *st : 0.0f, z * gru_candidate(ur));
-                        *st = S;
-                        y = S * siluf_(acc[RW - 1][b]);
-                    } else {
-                        y = siluf_(acc[0][b]) * acc[1][b];
-                    }
-                    stf(reinterpret_cast<T*>(a.out) + (long)b * a.ldo + c, y);
+                for (int r = 0; r < RW; ++r)
+#pragma unroll
+                    for (int b = 0; b < NB; ++b) part[wave][r * NB + b] = acc[r][b];
+            __syncthreads();
+#pragma unroll
+            for (int r = 0; r < RW; ++r)
+#pragma unroll
+                for (int b = 0; b < NB; ++b) {
+                    float t = 0.0f;
+#pragma unroll
+                    for (int q = 0; q < WK; ++q) t += part[(wave / WK) * WK + q][r * NB + b];
+                    acc[r][b] = t;
                 }
-            }
-        } else if constexpr (MODE == GR_STREAMS) {
-            // lane (r, b, t): every lane of the wave has read its streams before any is written
-            const int t = lane & 7, b = (lane >> 3) % NB, r = (lane >> 3) / NB;
-            float y = 0.0f;
-#pragma unroll
-            for (int rr = 0; rr < RW; ++rr)
-#pragma unroll
-                for (int bb = 0; bb < NB; ++bb)
-                    if (r == rr && b == bb) y = acc[rr][bb];
-            const int n = unit * 2 + r;
-            const bool ok = r < RW && b < a.B && t < a.S && n < a.N;
-            float v = 0.0f;
-            if (ok) {
-                const float* Xr = a.X + (long)b * a.S * a.D + n;
-                v = bf2f(a.wout[t]) * y;
-                for (int s = 0; s < a.S; ++s) v = fmaf(bf2f(a.mix[s * a.S + t]), Xr[(long)s * a.D], v);
-            }
-            if (ok) a.X[((long)b * a.S + t) * a.D + n] = v;
-        } else {
+        }
+        if (unit >= nunit) continue;
+        if constexpr (MODE == GR_LOGITS) {
 #pragma unroll
             for (int r = 0; r < RW; ++r)
 #pragma unroll
                 for (int b = 0; b < NB; ++b) {
                     const int n = unit * 2 + r;
-                    if constexpr (MODE == GR_LOGITS) {
-                        if (n < a.N && (acc[r][b] > best[b])) { best[b] = acc[r][b]; bi[b] = n; }
-                    }
-                    if (lane == r * NB + b && b < a.B && n < a.N) {
-                        float v = acc[r][b];
-                        if constexpr (MODE == GR_LOGITS || MODE == GR_F32) {
-                            reinterpret_cast<float*>(a.out)[(long)b * a.ldo + n] = v;
-                        } else if constexpr (MODE == GR_ACT) {
-                            if (a.bias) v += bf2f(a.bias[n]);
-                            stf(reinterpret_cast<T*>(a.out) + (long)b * a.ldo + n, v);
-                        } else if constexpr (MODE == GR_CONV) {
-                            if (n < a.C) {
-                                const int KT = a.taps_k;
-                                float* tp = a.state + (long)a.slot[b] * (KT - 1) * a.C + n;
-                                const bool first = a.pos[b] == 0;
-                                float y = fmaf(bf2f(a.cw[(long)n * KT + KT - 1]), v, bf2f(a.cb[n]));
-                                for (int j = 0; j < KT - 1; ++j) {
-                                    const float o = first ? 0.0f : tp[(long)j * a.C];
-                                    y = fmaf(bf2f(a.cw[(long)n * KT + j]), o, y);
-                                    if (j > 0) tp[(long)(j - 1) * a.C] = o;
-                                }
-                                if (KT > 1) tp[(long)(KT - 2) * a.C] = v;
-                                stf(reinterpret_cast<T*>(a.out) + (long)b * a.ldo + n, siluf_(y));
-                            } else {
-                                stf(reinterpret_cast<T*>(a.out2) + (long)b * a.ldo2 + n - a.C, v);
-                            }
-                        }
-                    }
+                    if (n < a.N && acc[r][b] > best[b]) { best[b] = acc[r][b]; bi[b] = n; }
                 }
         }
+        // lane (r, b) of the unit's first wave finishes output r of row b
+        const int lr = lane / NB, lb = lane % NB;
+        float v = 0.0f, v1 = 0.0f, v2 = 0.0f;
+#pragma unroll
+        for (int b = 0; b < NB; ++b) {
+            if constexpr (UO == 1) {
+                if (lb == b) { v = acc[0][b]; v1 = acc[1][b]; v2 = acc[RW - 1][b]; }
+            } else {
+#pragma unroll
+                for (int r = 0; r < RW; ++r)
+                    if (lr == r && lb == b) v = acc[r][b];
+            }
+        }
+        const int n = unit * UO + lr;
+        if (kw == 0 && lr < UO && lb < a.B && n < a.N) step_epilogue<T, MODE>(a, n, lb, v, v1, v2);
     }
     if constexpr (MODE == GR_LOGITS) {
         __shared__ float sv[4][NB];
@@ -222,21 +294,24 @@ __global__ void __launch_bounds__(256) k_gemv_rt(GemvRtArgs a) {
             a.pidx[(long)tid * gridDim.x + blockIdx.x] = ix;
         }
     }
-    // activation outputs: the columns that pad a row to 8 are zero
-    if constexpr (MODE == GR_GRU || MODE == GR_SWIGLU || MODE == GR_CONV) {
-        const int n = MODE == GR_CONV ? a.C : a.N;
-        if (blockIdx.x == 0 && tid < NB && tid < a.B)
-            for (int k = n; k < a.ldo; ++k) stf(reinterpret_cast<T*>(a.out) + (long)tid * a.ldo + k, 0.0f);
-    }
+    step_pads<T, MODE>(a);
+}
+
+int k_split(const GemvRtArgs& a, int mode) { return mode != GR_LOGITS && a.K >= 4096 ? 4 : 1; }
+
+template <typename T, int NB, int MODE, int WK>
+void run_wk(hipStream_t s, const GemvRtArgs& a) {
+    size_t lds = (size_t)NB * a.K * sizeof(T) + (a.x ? 0 : (size_t)(a.D + a.groups) * sizeof(float));
+    if (lds > 60 * 1024)
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&k_gemv_rt<T, NB, MODE, WK>),
+                                  hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipLaunchKernelGGL((k_gemv_rt<T, NB, MODE, WK>), dim3(gemv_rt_blocks(a, (GemvRtMode)MODE)), dim3(256), lds, s, a);
 }
 
 template <typename T, int NB, int MODE>
 void run(hipStream_t s, const GemvRtArgs& a) {
-    size_t lds = (size_t)NB * a.K * sizeof(T) + (a.x ? 0 : (size_t)(a.D + a.groups) * sizeof(float));
-    if (lds > 64 * 1024)
-        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&k_gemv_rt<T, NB, MODE>),
-                                  hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    hipLaunchKernelGGL((k_gemv_rt<T, NB, MODE>), dim3(gemv_rt_blocks(a, (GemvRtMode)MODE)), dim3(256), lds, s, a);
+    if (MODE != GR_LOGITS && k_split(a, MODE) == 4) run_wk<T, NB, MODE, MODE == GR_LOGITS ? 1 : 4>(s, a);
+    else run_wk<T, NB, MODE, 1>(s, a);
 }
 
 template <typename T, int NB>
@@ -256,6 +331,77 @@ template <typename T>
 void run_t(hipStream_t s, GemvRtMode mode, const GemvRtArgs& a) {
     if (a.B <= 1) run_mode<T, 1>(s, mode, a);
     else run_mode<T, 2>(s, mode, a);
+}
+
+// ---------------------------------------------------------------- 3 .. 16 rows: MFMA
+// A workgroup owns 16 outputs (of each of the unit's matrices) and all rows; its 4 waves split K.  A lane reads 32
+// contiguous bytes of its weight row per 64-deep step (4 lanes: one 128-byte line), so the two MFMAs of a step
+// contract k = 16 lg .. 16 lg + 7 and 16 lg + 8 .. 16 lg + 15 of each lane group -- the activations (straight from
+// L2, B fragments) use the same order.  After the waves' sums meet in LDS, thread (n, b) runs the step's epilogue.
+template <int MODE>
+__global__ void __launch_bounds__(256) k_skinny(GemvRtArgs a) {
+    constexpr int NM = MODE == GR_GRU ? 3 : MODE == GR_SWIGLU ? 2 : 1;
+    constexpr int U = NM == 1 ? 8 : 4;  // 64-deep steps in flight
+    __shared__ float sums[4][NM][16][17];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int li = lane & 15, lg = lane >> 4, n0 = blockIdx.x * 16, K = a.K;
+    const uint16_t* wp[NM];
+#pragma unroll
+    for (int m = 0; m < NM; ++m) {
+        const int n = n0 + li < a.N ? n0 + li : a.N - 1;
+        wp[m] = a.W + ((long)m * a.N + n) * a.ldw;
+    }
+    const uint16_t* xp = reinterpret_cast<const uint16_t*>(a.x) + (long)(li < a.B ? li : a.B - 1) * a.ldx;
+    f32x4 acc[NM];
+#pragma unroll
+    for (int m = 0; m < NM; ++m) acc[m] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int nstep = (K + 63) / 64;
+    for (int s0 = wave; s0 < nstep; s0 += 4 * U) {
+        uint4 w[U][NM][2], x[U][2];
+#pragma unroll
+        for (int i = 0; i < U; ++i) {
+            const int k = (s0 + 4 * i) * 64 + lg * 16;
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                const bool ok = k + 8 * h < K;
+#pragma unroll
+                for (int m = 0; m < NM; ++m) w[i][m][h] = ldg16_sel(wp[m] + k + 8 * h, ok, wp[m]);
+                x[i][h] = ldg16_sel(xp + k + 8 * h, ok, xp);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < U; ++i)
+#pragma unroll
+            for (int h = 0; h < 2; ++h)
+#pragma unroll
+                for (int m = 0; m < NM; ++m)
+                    acc[m] = mfma16(__builtin_bit_cast(short8, w[i][m][h]), __builtin_bit_cast(short8, x[i][h]), acc[m]);
+    }
+#pragma unroll
+    for (int m = 0; m < NM; ++m)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) sums[wave][m][4 * lg + r][li] = acc[m][r];
+    __syncthreads();
+    const int b = tid & 15, n = n0 + (tid >> 4);
+    float v[3] = {0.f, 0.f, 0.f};
+#pragma unroll
+    for (int m = 0; m < NM; ++m)
+#pragma unroll
+        for (int q = 0; q < 4; ++q) v[m] += sums[q][m][tid >> 4][b];
+    if (b < a.B && n < a.N) step_epilogue<uint16_t, MODE>(a, n, b, v[0], v[1], v[2]);
+    step_pads<uint16_t, MODE>(a);
+}
+
+void run_skinny(hipStream_t s, GemvRtMode mode, const GemvRtArgs& a) {
+    const dim3 grid((a.N + 15) / 16), block(256);
+    switch (mode) {
+        case GR_ACT: hipLaunchKernelGGL((k_skinny<GR_ACT>), grid, block, 0, s, a); break;
+        case GR_CONV: hipLaunchKernelGGL((k_skinny<GR_CONV>), grid, block, 0, s, a); break;
+        case GR_GRU: hipLaunchKernelGGL((k_skinny<GR_GRU>), grid, block, 0, s, a); break;
+        case GR_SWIGLU: hipLaunchKernelGGL((k_skinny<GR_SWIGLU>), grid, block, 0, s, a); break;
+        case GR_STREAMS: hipLaunchKernelGGL((k_skinny<GR_STREAMS>), grid, block, 0, s, a); break;
+        default: hipLaunchKernelGGL((k_skinny<GR_F32>), grid, block, 0, s, a); break;
+    }
 }
 
 // ---------------------------------------------------------------- convolution step
@@ -397,19 +543,23 @@ __global__ void __launch_bounds__(256) k_decode_finish(const float* __restrict__
 
 }  // namespace
 
-int gemv_rt_max_batch() { return 2; }
+int gemv_rt_max_batch() { return 16; }
+int gemv_rt_parts() { return 2 * 2048; }
+bool gemv_rt_reads_streams(int B) { return B <= 2; }
 
 bool gemv_rt_fits(int B, int K, Act act) {
-    return B <= gemv_rt_max_batch() && (size_t)gemv_rt_max_batch() * K * (act == ACT_F32 ? 4 : 2) <= 96 * 1024;
+    if (B <= 2) return (size_t)2 * K * (act == ACT_F32 ? 4 : 2) <= 96 * 1024;
+    return act == ACT_BF16 && B <= gemv_rt_max_batch();
 }
 
 int gemv_rt_blocks(const GemvRtArgs& a, GemvRtMode mode) {
-    const int units = (a.N + unit_outs(mode) - 1) / unit_outs(mode);
-    return std::max(1, std::min((units + 3) / 4, 2048));
+    const int units = (a.N + unit_outs(mode) - 1) / unit_outs(mode), upb = 4 / k_split(a, mode);
+    return std::max(1, std::min((units + upb - 1) / upb, 2048));
 }
 
 void gemv_rt(hipStream_t s, Act act, GemvRtMode mode, const GemvRtArgs& a) {
-    if (act == ACT_F32) run_t<float>(s, mode, a);
+    if (a.B > 2) run_skinny(s, mode, a);
+    else if (act == ACT_F32) run_t<float>(s, mode, a);
     else run_t<uint16_t>(s, mode, a);
 }
 

@@ -5,6 +5,7 @@
 //   k_wattn     plain form, any size and both activation types: one workgroup per (row, head), online softmax
 //   k_wattn_m   bf16 MFMA form: 64 (position, head) pairs per workgroup against 64-key tiles of one key/value head
 //   k_wattn_d   one new token per sequence: keys split over workgroups, partials merged by k_wattn_dc
+//   k_wattn_dm  the same on bf16 MFMA
 #include <algorithm>
 
 #include "act.h"
@@ -28,41 +29,66 @@ __device__ __forceinline__ float biased_exact(float dot, float c1, float r1, flo
 }
 
 // ---------------------------------------------------------------- append
-// a wave per head of a row
-template <typename T>
+// LPH lanes per head of a row (8 elements each when V == 8: head sizes that are multiples of 8)
+template <typename T, int LPH, int V>
 __global__ void __launch_bounds__(256) k_append(WAttnArgs a) {
-    const int row = blockIdx.x, lane = threadIdx.x & 63;
-    const int head = blockIdx.y * 4 + (threadIdx.x >> 6);
-    if (head >= a.H + 2 * a.G) return;
+    const int row = blockIdx.x, sub = threadIdx.x % LPH;
+    const int head = blockIdx.y * (256 / LPH) + threadIdx.x / LPH, NH = a.H + 2 * a.G;
     const SeqInfo q = a.seqs[a.row_seq[row]];
     const long pos = q.start + (row - q.off);
     const T* src = reinterpret_cast<const T*>(a.qkv) + (long)row * a.ldqkv;
+    const int hd = head < NH ? head : NH - 1;
     T* dst;
     int n, np;
-    bool norm = true;
-    if (head < a.H) {
-        src += head * a.d; n = a.d; np = a.dp;
-        dst = reinterpret_cast<T*>(a.q) + ((long)row * a.H + head) * a.dp;
-    } else if (head < a.H + a.G) {
-        const int g = head - a.H;
+    const bool norm = hd < a.H + a.G;
+    if (hd < a.H) {
+        src += hd * a.d; n = a.d; np = a.dp;
+        dst = reinterpret_cast<T*>(a.q) + ((long)row * a.H + hd) * a.dp;
+    } else if (hd < a.H + a.G) {
+        const int g = hd - a.H;
         src += a.H * a.d + g * a.d; n = a.d; np = a.dp;
         dst = reinterpret_cast<T*>(a.kc) + (((long)q.slot * a.G + g) * a.max_tokens + pos) * a.dp;
     } else {
-        const int g = head - a.H - a.G;
+        const int g = hd - a.H - a.G;
         src += (a.H + a.G) * a.d + g * a.e; n = a.e; np = a.ep;
         dst = reinterpret_cast<T*>(a.vc) + (((long)q.slot * a.G + g) * a.max_tokens + pos) * a.ep;
-        norm = false;
     }
-    float inv = 1.0f;
-    if (norm) {
-        float ss = 0.0f;
-        for (int i = lane; i < n; i += 64) {
+    float ss = 0.0f;
+    for (int i = sub * V; i < n; i += LPH * V) {
+        if constexpr (V == 8) {
+            float v[8];
+            ld8(src + i, v);
+#pragma unroll
+            for (int t = 0; t < 8; ++t) ss = fmaf(v[t], v[t], ss);
+        } else {
             const float v = ldf(src + i);
             ss = fmaf(v, v, ss);
         }
-        inv = 1.0f / sqrtf(wave_sum(ss) / (float)n + a.eps);
     }
-    for (int i = lane; i < np; i += 64) stf(dst + i, i < n ? ldf(src + i) * inv : 0.0f);
+#pragma unroll
+    for (int o = 1; o < LPH; o <<= 1) ss += __shfl_xor(ss, o, 64);
+    const float inv = norm ? 1.0f / sqrtf(ss / (float)n + a.eps) : 1.0f;
+    if (head >= NH) return;
+    for (int i = sub * V; i < np; i += LPH * V) {
+        if constexpr (V == 8) {
+            float v[8];
+            ld8(src + i, v);
+#pragma unroll
+            for (int t = 0; t < 8; ++t) v[t] *= inv;
+            st8(dst + i, v);
+        } else {
+            stf(dst + i, i < n ? ldf(src + i) * inv : 0.0f);
+        }
+    }
+}
+
+template <typename T>
+void append_t(hipStream_t s, const WAttnArgs& a) {
+    const int NH = a.H + 2 * a.G;
+    if (a.d % 8 == 0 && a.e % 8 == 0)
+        hipLaunchKernelGGL((k_append<T, 16, 8>), dim3(a.rows, (NH + 15) / 16), dim3(256), 0, s, a);
+    else
+        hipLaunchKernelGGL((k_append<T, 64, 1>), dim3(a.rows, (NH + 3) / 4), dim3(256), 0, s, a);
 }
 
 // ---------------------------------------------------------------- plain form
@@ -447,22 +473,188 @@ __global__ void __launch_bounds__(256) k_wattn_d(WAttnDecodeArgs a) {
     }
 }
 
-// merge a head's partials: grid (H, B)
+// bf16 MFMA form, 16 query heads of a group per workgroup (grid (split, G * head blocks, B)).  A wave takes 32-key
+// tiles: S^T = K Q^T with the key fragments straight from the cache, then O^T += V^T P^T as k_wattn_m, the values
+// through the wave's own LDS rows; the four waves' running sums meet in LDS.
+template <int DQ, int DV>
+__global__ void __launch_bounds__(256) k_wattn_dm(WAttnDecodeArgs a) {
+    constexpr int VS = DV + 8;
+    __shared__ __attribute__((aligned(16))) uint16_t Vs[4][32 * VS];
+    __shared__ float sml[4][16][2];
+    const int R = a.H / a.G, hb = blockIdx.y / a.G, g = blockIdx.y % a.G, b = blockIdx.z, sp = blockIdx.x;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lg = lane >> 4;
+    const int slot = a.slot[b], i = a.pos[b];
+    const int lo = max(0, i - a.window + 1), span = i - lo + 1;
+    const int per = ((span + a.nsplit - 1) / a.nsplit + 127) / 128 * 128;
+    const int k0 = lo + sp * per, k1 = min(i + 1, k0 + per);
+    const uint16_t* qkv = reinterpret_cast<const uint16_t*>(a.qkv) + (long)b * a.ldqkv;
+    const int r0 = hb * 16, nr = min(16, R - r0), rs = a.ep + 2;
+    float* part = a.part + (((long)b * a.H + g * R + r0) * a.nsplit + sp) * rs;
+    if (k0 >= k1) {
+        if (tid < nr) {
+            part[(long)tid * a.nsplit * rs + a.ep] = kNone;
+            part[(long)tid * a.nsplit * rs + a.ep + 1] = 0.0f;
+        }
+        return;
+    }
+    uint16_t* kc = reinterpret_cast<uint16_t*>(a.kc) + ((long)slot * a.G + g) * a.max_tokens * a.dp;
+    uint16_t* vc = reinterpret_cast<uint16_t*>(a.vc) + ((long)slot * a.G + g) * a.max_tokens * a.ep;
+    if (k1 == i + 1) {  // the new token's cache rows (every head block of the group writes the same)
+        if (wave == 0) {
+            const uint16_t* src = qkv + a.H * a.d + g * a.d;
+            float ss = 0.0f;
+            for (int k = lane; k < a.d; k += 64) ss = fmaf(bf2f(src[k]), bf2f(src[k]), ss);
+            const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)a.d + a.eps);
+            for (int k = lane; k < a.dp; k += 64) kc[(long)i * a.dp + k] = k < a.d ? f2bf(bf2f(src[k]) * inv) : 0;
+        } else if (wave == 1) {
+            const uint16_t* src = qkv + (a.H + a.G) * a.d + g * a.e;
+            for (int k = lane; k < a.ep; k += 64) vc[(long)i * a.ep + k] = k < a.e ? src[k] : 0;
+        }
+    }
+    // this lane's query head: dims 8 lg .. 8 lg + 7 of every 32
+    const int h = g * R + r0 + (li < nr ? li : 0);
+    short8 qf[DQ / 32];
+    {
+        const uint16_t* src = qkv + h * a.d;
+        float q[DQ / 32][8], ss = 0.0f;
+#pragma unroll
+        for (int c = 0; c < DQ / 32; ++c)
+#pragma unroll
+            for (int v = 0; v < 8; ++v) {
+                const int k = c * 32 + 8 * lg + v;
+                q[c][v] = k < a.d ? bf2f(src[k]) : 0.0f;
+                ss = fmaf(q[c][v], q[c][v], ss);
+            }
+        ss += __shfl_xor(ss, 16, 64);
+        ss += __shfl_xor(ss, 32, 64);
+        const float inv = 1.0f / sqrtf(ss / (float)a.d + a.eps);
+#pragma unroll
+        for (int c = 0; c < DQ / 32; ++c)
+#pragma unroll
+            for (int v = 0; v < 8; ++v) qf[c][v] = (short)f2bf(q[c][v] * inv);
+    }
+    const float r1 = bf2f(a.r1[h]), r2 = bf2f(a.r2[h]), c1 = a.scale * kLog2e;
+    if (k1 == i + 1) {
+        __threadfence_block();
+        __syncthreads();
+    }
+    f32x4 o[DV / 16];
+#pragma unroll
+    for (int c = 0; c < DV / 16; ++c) o[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float m = kNone, l = 0.0f;
+    for (int j0 = k0 + wave * 32; j0 < k1; j0 += 128) {
+        uint4 vr[DV / 16];
+#pragma unroll
+        for (int x = 0; x < DV / 16; ++x) {
+            const int e = lane + 64 * x, r = e / (DV / 8), k = (e % (DV / 8)) * 8;
+            vr[x] = ldg16_sel(vc + (long)min(j0 + r, i) * a.ep + k, k < a.ep, vc);
+        }
+        f32x4 st[2];
+#pragma unroll
+        for (int t = 0; t < 2; ++t) {
+            st[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+            const uint16_t* kr = kc + (long)min(j0 + t * 16 + li, i) * a.dp;
+#pragma unroll
+            for (int c = 0; c < DQ / 32; ++c) {
+                const int k = c * 32 + 8 * lg;
+                st[t] = mfma16(__builtin_bit_cast(short8, ldg16_sel(kr + k, k < a.dp, kr)), qf[c], st[t]);
+            }
+        }
+        float mt = m;
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int j = j0 + t * 16 + 4 * lg + r;
+                st[t][r] = j < k1 ? biased(st[t][r], c1, r1, r2, (float)(i - j)) : -INFINITY;
+                mt = fmaxf(mt, st[t][r]);
+            }
+        mt = fmaxf(mt, __shfl_xor(mt, 16, 64));
+        mt = fmaxf(mt, __shfl_xor(mt, 32, 64));
+        const float alpha = __builtin_amdgcn_exp2f(m - mt);
+        m = mt;
+        l *= alpha;
+        short8 pf;
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const float p = __builtin_amdgcn_exp2f(st[t][r] - m);
+                l += p;
+                pf[4 * t + r] = (short)f2bf(p);
+            }
+#pragma unroll
+        for (int x = 0; x < DV / 16; ++x) {
+            const int e = lane + 64 * x, r = e / (DV / 8), k = (e % (DV / 8)) * 8;
+            *reinterpret_cast<uint4*>(&Vs[wave][r * VS + k]) = vr[x];
+        }
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // this wave's own rows: no barrier
+#pragma unroll
+        for (int c = 0; c < DV / 16; ++c) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) o[c][r] *= alpha;
+            uint16_t* vp = &Vs[wave][(4 * lg + (li >> 2)) * VS + c * 16 + 4 * (li & 3)];
+            const s4v lo4 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4v*)(vp));
+            const s4v hi4 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4v*)(vp + 16 * VS));
+            const short8 vf = {lo4[0], lo4[1], lo4[2], lo4[3], hi4[0], hi4[1], hi4[2], hi4[3]};
+            o[c] = mfma16(vf, pf, o[c]);
+        }
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    }
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    if (lg == 0) { sml[wave][li][0] = m; sml[wave][li][1] = l; }
+    __syncthreads();
+    float M = kNone;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) M = fmaxf(M, sml[w][li][0]);
+    const float f = __builtin_amdgcn_exp2f(m - M);
+    float* os = reinterpret_cast<float*>(&Vs[0][0]);  // [wave][head][DV], in place of the value rows
+#pragma unroll
+    for (int c = 0; c < DV / 16; ++c)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) os[(wave * 16 + li) * DV + c * 16 + 4 * lg + r] = o[c][r] * f;
+    __syncthreads();
+    for (int e = tid; e < nr * a.ep; e += 256) {
+        const int r = e / a.ep, c = e % a.ep;
+        float t = 0.0f;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) t += os[(w * 16 + r) * DV + c];
+        part[(long)r * a.nsplit * rs + c] = t;
+    }
+    if (tid < nr) {
+        float mm = kNone, ll = 0.0f;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) mm = fmaxf(mm, sml[w][tid][0]);
+#pragma unroll
+        for (int w = 0; w < 4; ++w) ll += sml[w][tid][1] * __builtin_amdgcn_exp2f(sml[w][tid][0] - mm);
+        part[(long)tid * a.nsplit * rs + a.ep] = mm;
+        part[(long)tid * a.nsplit * rs + a.ep + 1] = ll;
+    }
+}
+
+// merge a head's partials: grid (H, B), nsplit <= 64
 template <typename T>
 __global__ void __launch_bounds__(256) k_wattn_dc(WAttnDecodeArgs a) {
-    const int h = blockIdx.x, b = blockIdx.y, rs = a.ep + 2;
-    const float* p = a.part + ((long)b * a.H + h) * a.nsplit * rs;
-    float m = kNone;
-    for (int s = 0; s < a.nsplit; ++s) m = fmaxf(m, p[(long)s * rs + a.ep]);
-    float l = 0.0f;
-    for (int s = 0; s < a.nsplit; ++s) l += p[(long)s * rs + a.ep + 1] * exp2f(p[(long)s * rs + a.ep] - m);
+    __shared__ float wt[64];
+    const int h = blockIdx.x, b = blockIdx.y, rs = a.ep + 2, n = a.nsplit, lane = threadIdx.x & 63;
+    const float* p = a.part + ((long)b * a.H + h) * n * rs;
+    {
+        const float m = lane < n ? p[(long)lane * rs + a.ep] : kNone, l = lane < n ? p[(long)lane * rs + a.ep + 1] : 0.0f;
+        const float M = wave_max(l > 0.0f ? m : kNone);
+        const float w = l > 0.0f ? exp2f(m - M) : 0.0f;
+        const float L = wave_sum(l * w);
+        if (threadIdx.x < 64) wt[lane] = w / L;
+    }
+    __syncthreads();
     T* o = reinterpret_cast<T*>(a.o) + (long)b * a.ldo;
     for (int c = threadIdx.x; c < a.e; c += 256) {
         float t = 0.0f;
-        for (int s = 0; s < a.nsplit; ++s) {
-            if (p[(long)s * rs + a.ep + 1] > 0.0f) t = fmaf(p[(long)s * rs + c], exp2f(p[(long)s * rs + a.ep] - m), t);
-        }
-        stf(o + h * a.e + c, t / l);
+        // an empty split's values were never written: weight 0, not read
+#pragma unroll 8
+        for (int s = 0; s < n; ++s)
+            if (wt[s] > 0.0f) t = fmaf(p[(long)s * rs + c], wt[s], t);
+        stf(o + h * a.e + c, t);
     }
     if (h == a.H - 1)
         for (int k = a.H * a.e + threadIdx.x; k < a.ldo; k += 256) stf(o + k, 0.0f);
@@ -477,6 +669,18 @@ void run_d(hipStream_t s, const WAttnDecodeArgs& a) {
                                   hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     hipLaunchKernelGGL((k_wattn_d<T, RB>), dim3(a.nsplit, a.G, a.B), dim3(256), lds, s, a);
     hipLaunchKernelGGL((k_wattn_dc<T>), dim3(a.H, a.B), dim3(256), 0, s, a);
+}
+
+template <int DQ, int DV>
+void run_dm(hipStream_t s, const WAttnDecodeArgs& a) {
+    hipLaunchKernelGGL((k_wattn_dm<DQ, DV>), dim3(a.nsplit, a.G * ((a.H / a.G + 15) / 16), a.B), dim3(256), 0, s, a);
+    hipLaunchKernelGGL((k_wattn_dc<uint16_t>), dim3(a.H, a.B), dim3(256), 0, s, a);
+}
+template <int DQ>
+void run_dmv(hipStream_t s, const WAttnDecodeArgs& a) {
+    if (a.ep <= 64) run_dm<DQ, 64>(s, a);
+    else if (a.ep <= 128) run_dm<DQ, 128>(s, a);
+    else run_dm<DQ, 256>(s, a);
 }
 
 template <typename T>
@@ -497,9 +701,8 @@ void plain_t(hipStream_t s, const WAttnArgs& a) {
 }  // namespace
 
 void wattn_append(hipStream_t s, Act act, const WAttnArgs& a) {
-    const dim3 grid(a.rows, (a.H + 2 * a.G + 3) / 4);
-    if (act == ACT_F32) hipLaunchKernelGGL((k_append<float>), grid, dim3(256), 0, s, a);
-    else hipLaunchKernelGGL((k_append<uint16_t>), grid, dim3(256), 0, s, a);
+    if (act == ACT_F32) append_t<float>(s, a);
+    else append_t<uint16_t>(s, a);
 }
 
 void wattn_prefill(hipStream_t s, Act act, const WAttnArgs& a) {
@@ -520,8 +723,8 @@ void wattn_prefill(hipStream_t s, Act act, const WAttnArgs& a) {
 
 int wattn_decode_splits(int B, int G, int window, int max_tokens) {
     const int span = std::max(1, std::min(window, max_tokens));
-    const int tiles = (span + DK - 1) / DK;
-    int n = (512 + B * G - 1) / (B * G);
+    const int tiles = (span + 127) / 128;
+    int n = (1024 + B * G - 1) / (B * G);
     return std::max(1, std::min(std::min(n, tiles), 64));
 }
 
@@ -529,7 +732,10 @@ size_t wattn_decode_floats(int B, int H, int ep, int nsplit) { return (size_t)B 
 
 void wattn_decode(hipStream_t s, Act act, const WAttnDecodeArgs& a) {
     if (act == ACT_F32) decode_t<float>(s, a);
-    else decode_t<uint16_t>(s, a);
+    else if (a.dp > 256 || a.ep > 256) decode_t<uint16_t>(s, a);
+    else if (a.dp <= 64) run_dmv<64>(s, a);
+    else if (a.dp <= 128) run_dmv<128>(s, a);
+    else run_dmv<256>(s, a);
 }
 
 }  // namespace pgmi

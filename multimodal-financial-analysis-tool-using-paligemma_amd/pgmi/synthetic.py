@@ -66,3 +66,42 @@ def prompt_ids(image_token_index: int, n_image_tokens: int, vocab: int, n_text: 
     txt = rng.integers(3, hi, size=n_text)
     newline = 108 if hi > 108 else 5
     return np.array([[image_token_index] * n_image_tokens + [2] + txt.tolist() + [newline]], dtype=np.int64)
+
+
+def decoder_policy(name: str, shape: tuple) -> "tuple[float, float]":
+    """init_policy's counterpart for layered decoders (pgmi/decoder.py tensor names): values that keep the streams,
+    decays and gates in an ordinary range, for benchmarks."""
+    leaf = name.split(".", 1)[1] if name.startswith("l") else name
+    if leaf == "embed":
+        return 0.02, 0.0
+    if "norm" in leaf:
+        return 0.1, 1.0
+    if leaf.startswith("hc"):
+        if leaf.endswith(".out"):
+            return 0.1, 1.0
+        return 0.02, 1.0 / shape[0]
+    if leaf == "mix.A_log":
+        return 1.0, 0.5
+    if leaf == "mix.dt.b":
+        return 1.0, -4.0
+    if leaf == "mix.D":
+        return 0.1, 1.0
+    if leaf in ("mix.r1", "mix.r2"):
+        return 0.2, 0.4
+    if leaf.endswith(".b"):
+        return 0.02, 0.0
+    return _f32(1.7 / math.sqrt(math.prod(shape[1:]))), 0.0
+
+
+def decoder_bench_config(size: str) -> dict:
+    """Tuvodra configurations with the layer sizes of real models, random weights ("2b": PaliGemma's text width,
+    feed-forward, attention width and vocabulary)."""
+    w = {"1b": 1024, "2b": 2048, "7b": 4096}[size]
+    heads, kv, ff, vocab, blocks = {"1b": (8, 2, 4096, 32768, 4), "2b": (16, 2, 16384, 257216, 4),
+                                    "7b": (32, 8, 14336, 65536, 2)}[size]
+    mamba = {"type": "mamba1", "mixer": {"inner": 2 * w, "state": 16, "dt_rank": w // 16, "conv": 4}, "mlp": None}
+    gru = {"type": "mingru", "mixer": {"width": w}, "mlp": None}
+    attn = {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                                           "mask": {"size": 1024}}, "mlp": {"kind": "dense", "ff": ff}}
+    return {"architecture": "Tuvodra", "vocab": vocab, "width": w, "streams": 2, "norm": {"groups": 4, "eps": 1e-5},
+            "embedding": {"scale": 32.0}, "layers": [mamba, gru, mamba, attn] * blocks}
