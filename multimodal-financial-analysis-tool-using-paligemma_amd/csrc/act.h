@@ -35,9 +35,9 @@ __device__ __forceinline__ void st8(float* p, const float (&v)[8]) {
     *reinterpret_cast<float4*>(p + 4) = make_float4(v[4], v[5], v[6], v[7]);
 }
 
-// 1 / (1 + exp(-x)); exp overflowing to +inf gives 0
-__device__ __forceinline__ float sigmoidf_(float x) { return 1.0f / (1.0f + __expf(-x)); }
-__device__ __forceinline__ float siluf_(float x) { return x / (1.0f + __expf(-x)); }
+// 1 / (1 + exp(-x)) with the hardware reciprocal (1 ulp); exp overflowing to +inf gives 0
+__device__ __forceinline__ float sigmoidf_(float x) { return __builtin_amdgcn_rcpf(1.0f + __expf(-x)); }
+__device__ __forceinline__ float siluf_(float x) { return x * sigmoidf_(x); }
 // ln(1 + exp(x)) without overflow or cancellation
 __device__ __forceinline__ float softplusf_(float x) { return fmaxf(x, 0.0f) + log1pf(__expf(-fabsf(x))); }
 // the same from the hardware exponential and logarithm: a short series where 1 + e would round e away

@@ -174,7 +174,7 @@ enum GemvRtMode : int {
     GR_SWIGLU = 3,   // N channels, rows n, N + n: silu(gate) * up -> out
     GR_STREAMS = 4,  // X'[t] = sum_s mix[s][t] X[s] + wout[t] acc, in place
     GR_LOGITS = 5,   // fp32 out + (B <= 2) per-workgroup argmax partials
-    GR_F32 = 6,      // fp32 out
+    GR_F32 = 6,      // fp32 out; B > 2: `split` partial slabs [split][B][ldo]
 };
 struct GemvRtArgs {
     int B, N, K;  // N: outputs (rows of W, or channels); K: padded to 8
@@ -203,6 +203,7 @@ struct GemvRtArgs {
     // GR_STREAMS
     const uint16_t* mix;
     const uint16_t* wout;
+    int split;  // GR_F32
     // GR_LOGITS
     float* pmax;
     int* pidx;
@@ -210,6 +211,7 @@ struct GemvRtArgs {
 int gemv_rt_max_batch();
 int gemv_rt_parts();  // words of pmax / pidx
 bool gemv_rt_reads_streams(int B);
+int gemv_rt_split(int B, int N, int K);  // slabs of a GR_F32 product
 bool gemv_rt_fits(int B, int K, Act act);
 int gemv_rt_blocks(const GemvRtArgs& a, GemvRtMode mode);
 void gemv_rt(hipStream_t s, Act act, GemvRtMode mode, const GemvRtArgs& a);

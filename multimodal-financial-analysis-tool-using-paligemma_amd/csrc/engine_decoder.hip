@@ -463,8 +463,15 @@ int forward_body(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int rows, const
         fold(a, pend, rows);
         a.in = nullptr; a.w = d.fnorm; a.rows_idx = m.want;
         streams_norm(s, d.act, a);
-        matmul_rt(s, d.act, d.h, d.ldh, d.head.w, d.head.ldw, n_want, d.c.vocab, d.head.k, RT_F32, nullptr, logits,
-                  d.c.vocab, 0, nullptr);
+        if (gemv_rt_fits(n_want, d.head.k, d.act)) {
+            GemvRtArgs g{};
+            g.B = n_want; g.N = d.c.vocab; g.K = d.head.k; g.W = d.head.w; g.ldw = d.head.ldw; g.x = d.h; g.ldx = d.ldh;
+            g.out = logits; g.ldo = d.c.vocab;
+            gemv_rt(s, d.act, GR_F32, g);
+        } else {
+            matmul_rt(s, d.act, d.h, d.ldh, d.head.w, d.head.ldw, n_want, d.c.vocab, d.head.k, RT_F32, nullptr, logits,
+                      d.c.vocab, 0, nullptr);
+        }
     }
     LAUNCHCHK();
     return 0;
@@ -506,7 +513,13 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
         return g;
     };
     auto out_proj = [&](const Lin& o, const void* in, int ldin, const Sub& sub) {
-        if (gemv_rt_fits(B, o.k, d.act) && d.c.streams <= 8) {
+        const bool fits = gemv_rt_fits(B, o.k, d.act);
+        if (fits && !gemv_rt_reads_streams(B)) {  // the next streams pass sums the slabs
+            GemvRtArgs g = row_in(o, in, ldin);
+            g.out = d.slabs; g.ldo = D; g.split = gemv_rt_split(B, D, o.k);
+            gemv_rt(s, d.act, GR_F32, g);
+            pend = {d.slabs, g.split, &sub};
+        } else if (fits) {
             GemvRtArgs g = row_in(o, in, ldin);
             g.X = d.X; g.S = d.c.streams; g.D = D; g.mix = sub.mix; g.wout = sub.out;
             gemv_rt(s, d.act, GR_STREAMS, g);
@@ -539,8 +552,9 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
             a.split = 1;
             if (gemv_rt_fits(B, w.x.k, d.act)) {
                 g = row_in(w.x, d.p1, ldc);
-                g.out = d.slabs; g.ldo = w.x.n;
+                g.out = d.slabs; g.ldo = w.x.n; g.split = gemv_rt_split(B, w.x.n, w.x.k);
                 gemv_rt(s, d.act, GR_F32, g);
+                a.split = g.split;
             } else {
                 a.split = matmul_rt(s, d.act, d.p1, ldc, w.x.w, w.x.ldw, B, w.x.n, w.x.k, RT_SLABS, nullptr, d.slabs, 0,
                                     d.slab_bytes, nullptr);

@@ -139,7 +139,7 @@ void run_plan(const Job& j) {
     const int bn2 = epi_dual(EPI) ? 2 : 1;
     if (j.K % 64 == 0 && j.K >= 1024 && j.M >= 1024 && tiles(j.M, j.N, 256, 256 / bn2) * j.split >= 160)
         run_e256<EPI, SPLIT>(j);
-    else if (tiles(j.M, j.N, 128, 128 / bn2) * j.split >= 128)
+    else if (j.N > 192 && tiles(j.M, j.N, 128, 128 / bn2) * j.split >= 128)
         run_w128<EPI, SPLIT>(j);
     else
         run_p64<EPI, SPLIT>(j);

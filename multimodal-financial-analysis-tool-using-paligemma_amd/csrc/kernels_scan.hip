@@ -295,13 +295,7 @@ void scan_t(hipStream_t s, const ScanArgs& a) {
 }
 
 // ---------------------------------------------------------------- minGRU
-// V channels per lane (4 where rows allow it, else 1)
-template <typename T, int V>
-__device__ __forceinline__ void ldv(const T* p, float (&v)[V]) {
-    if constexpr (V == 4) ld4(p, v);
-    else v[0] = ldf(p);
-}
-
+// V channels per lane (2 where rows allow it, else 1)
 template <typename T, int PHASE, int V>
 __global__ void __launch_bounds__(64) k_gru(GruArgs a) {
     const ChunkInfo ck = a.chunks[blockIdx.y];
@@ -327,15 +321,29 @@ __global__ void __launch_bounds__(64) k_gru(GruArgs a) {
             else if (q.start > 0) S[v] = a.state[(long)q.slot * a.C + c + v];
         }
     }
-    for (int t0 = 0; t0 < ck.len; t0 += kPre) {
-        float z[kPre][V], u[kPre][V], g[kPre][V];
+    struct alignas(sizeof(T) * V) Raw { T v[V]; };
+    Raw rz[kPre], ru[kPre], rg[PHASE ? kPre : 1];
+    auto fetch = [&](int t0) {  // rows past the chunk repeat its last one (never used)
 #pragma unroll
         for (int t = 0; t < kPre; ++t) {
             const T* r = zp + (long)min(t0 + t, ck.len - 1) * a.ld;
-            ldv<T, V>(r, z[t]);
-            ldv<T, V>(r + a.C, u[t]);
-            if constexpr (PHASE == 1) ldv<T, V>(r + 2 * a.C, g[t]);
+            rz[t] = *reinterpret_cast<const Raw*>(r);
+            ru[t] = *reinterpret_cast<const Raw*>(r + a.C);
+            if constexpr (PHASE == 1) rg[t] = *reinterpret_cast<const Raw*>(r + 2 * a.C);
         }
+    };
+    fetch(0);
+    for (int t0 = 0; t0 < ck.len; t0 += kPre) {
+        float z[kPre][V], u[kPre][V], g[kPre][V];
+#pragma unroll
+        for (int t = 0; t < kPre; ++t)
+#pragma unroll
+            for (int v = 0; v < V; ++v) {
+                z[t][v] = ldf(&rz[t].v[v]);
+                u[t][v] = ldf(&ru[t].v[v]);
+                if constexpr (PHASE == 1) g[t][v] = ldf(&rg[t].v[v]);
+            }
+        if (t0 + kPre < ck.len) fetch(t0 + kPre);
 #pragma unroll
         for (int t = 0; t < kPre; ++t) {
             if (t0 + t >= ck.len) break;
@@ -348,8 +356,10 @@ __global__ void __launch_bounds__(64) k_gru(GruArgs a) {
                 else y[v] = S[v] * siluf_(g[t][v]);
             }
             if constexpr (PHASE == 1) {
-                if constexpr (V == 4) st4(yp + (long)(t0 + t) * a.ldy, y);
-                else stf(yp + (long)(t0 + t) * a.ldy, y[0]);
+                Raw o;
+#pragma unroll
+                for (int v = 0; v < V; ++v) stf(&o.v[v], y[v]);
+                *reinterpret_cast<Raw*>(yp + (long)(t0 + t) * a.ldy) = o;
             }
         }
     }
@@ -403,7 +413,7 @@ void gru_v(hipStream_t s, const GruArgs& a) {
 
 template <typename T>
 void gru_t(hipStream_t s, const GruArgs& a) {
-    if (a.C % 8 == 0 && a.ld % 8 == 0) gru_v<T, 4>(s, a);
+    if (a.C % 8 == 0 && a.ld % 8 == 0) gru_v<T, 2>(s, a);
     else gru_v<T, 1>(s, a);
 }
 

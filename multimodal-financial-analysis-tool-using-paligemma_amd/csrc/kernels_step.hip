@@ -12,13 +12,20 @@ namespace {
 
 constexpr int UN = 4;  // K steps (512 elements each) whose weight loads are in flight together
 
-__device__ __forceinline__ float dotx(const uint4 w, const uint16_t* x, float acc) {
-    return dot8(w, *reinterpret_cast<const uint4*>(x), acc);
+// eight activations as loaded
+struct X8b { uint4 q; };
+struct X8f { float4 a, b; };
+template <typename T> struct X8 { typedef X8b type; };
+template <> struct X8<float> { typedef X8f type; };
+__device__ __forceinline__ void ldx(const uint16_t* p, X8b& x) { x.q = *reinterpret_cast<const uint4*>(p); }
+__device__ __forceinline__ void ldx(const float* p, X8f& x) {
+    x.a = *reinterpret_cast<const float4*>(p);
+    x.b = *reinterpret_cast<const float4*>(p + 4);
 }
-__device__ __forceinline__ float dotx(const uint4 w, const float* x, float acc) {
+__device__ __forceinline__ float dotx(const uint4 w, const X8b& x, float acc) { return dot8(w, x.q, acc); }
+__device__ __forceinline__ float dotx(const uint4 w, const X8f& x, float acc) {
     const uint32_t q[4] = {w.x, w.y, w.z, w.w};
-    float v[8];
-    ld8(x, v);
+    const float v[8] = {x.a.x, x.a.y, x.a.z, x.a.w, x.b.x, x.b.y, x.b.z, x.b.w};
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         acc = fmaf(__uint_as_float(q[i] << 16), v[2 * i], acc);
@@ -90,8 +97,9 @@ __device__ __forceinline__ void step_pads(const GemvRtArgs& a) {
     }
 }
 
-// WK: waves of the workgroup that share a unit, each a K slice
-template <typename T, int NB, int MODE, int WK>
+// WK: waves of the workgroup that share a unit, each a K slice.  XG: the input is rows of activations, loaded with the
+// weights; else the streams' read and norm, staged in LDS by the prologue.
+template <typename T, int NB, int MODE, int WK, bool XG>
 __global__ void __launch_bounds__(256) k_gemv_rt(GemvRtArgs a) {
     constexpr int RW = unit_rows(MODE), UO = unit_outs(MODE), UPB = 4 / WK;
     extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
@@ -103,6 +111,20 @@ __global__ void __launch_bounds__(256) k_gemv_rt(GemvRtArgs a) {
     const int ustep = gridDim.x * UPB, kw = wave % WK;
     int unit = blockIdx.x * UPB + wave / WK;
     uint4 w[2][RW][UN];
+    typename X8<T>::type xr[2][XG ? NB : 1][XG ? UN : 1];
+    auto xload = [&](int buf, int k0) {
+        if constexpr (XG) {
+#pragma unroll
+            for (int b = 0; b < NB; ++b) {
+                const T* p = reinterpret_cast<const T*>(a.x) + (long)(b < a.B ? b : 0) * a.ldx;
+#pragma unroll
+                for (int i = 0; i < UN; ++i) {
+                    const int k = k0 + (i * WK + kw) * 512 + lane * 8;
+                    ldx(p + (k < K ? k : 0), xr[buf][b][i]);
+                }
+            }
+        }
+    };
     auto wload = [&](uint4 (&q)[RW][UN], int u, int k0) {
         const int uu = u < nunit ? u : nunit - 1;
 #pragma unroll
@@ -119,13 +141,8 @@ __global__ void __launch_bounds__(256) k_gemv_rt(GemvRtArgs a) {
         }
     };
     wload(w[0], unit, 0);  // in flight during the prologue
-    if (a.x) {
-        for (int e = tid * 8; e < NB * K; e += 256 * 8) {
-            const int b = e / K, k = e % K;
-            float v[8];
-            ld8(reinterpret_cast<const T*>(a.x) + (long)(b < a.B ? b : 0) * a.ldx + k, v);
-            st8(xs + b * K + k, v);
-        }
+    if constexpr (XG) {
+        xload(0, 0);
     } else {
         // the streams' read and grouped norm of each row, as streams_norm
         float* u_ = reinterpret_cast<float*>(smem + (size_t)NB * K * sizeof(T));  // [D], then [groups]
@@ -196,21 +213,24 @@ __global__ void __launch_bounds__(256) k_gemv_rt(GemvRtArgs a) {
             __syncthreads();
         }
     }
-    __syncthreads();
     float best[NB];
     int bi[NB];
 #pragma unroll
     for (int b = 0; b < NB; ++b) { best[b] = -INFINITY; bi[b] = 0x7fffffff; }
     float acc[RW][NB];
-    auto mac = [&](const uint4 (&q)[RW][UN], int k0) {
+    auto mac = [&](int buf, int k0) {
 #pragma unroll
         for (int i = 0; i < UN; ++i) {
             const int k = k0 + (i * WK + kw) * 512 + lane * 8;
             if (k < K) {
 #pragma unroll
-                for (int b = 0; b < NB; ++b)
+                for (int b = 0; b < NB; ++b) {
+                    typename X8<T>::type x;
+                    if constexpr (XG) x = xr[buf][b][i];
+                    else ldx(xs + b * K + k, x);
 #pragma unroll
-                    for (int r = 0; r < RW; ++r) acc[r][b] = dotx(q[r][i], xs + b * K + k, acc[r][b]);
+                    for (int r = 0; r < RW; ++r) acc[r][b] = dotx(w[buf][r][i], x, acc[r][b]);
+                }
             }
         }
     };
@@ -222,14 +242,23 @@ __global__ void __launch_bounds__(256) k_gemv_rt(GemvRtArgs a) {
 #pragma unroll
             for (int b = 0; b < NB; ++b) acc[r][b] = 0.0f;
         for (int k0 = 0; k0 < K; k0 += 2 * KB) {
-            if (k0 + KB < K) wload(w[1], unit, k0 + KB);
-            mac(w[0], k0);
             if (k0 + KB < K) {
-                if (k0 + 2 * KB < K) wload(w[0], unit, k0 + 2 * KB);
-                mac(w[1], k0 + KB);
+                wload(w[1], unit, k0 + KB);
+                xload(1, k0 + KB);
+            }
+            mac(0, k0);
+            if (k0 + KB < K) {
+                if (k0 + 2 * KB < K) {
+                    wload(w[0], unit, k0 + 2 * KB);
+                    xload(0, k0 + 2 * KB);
+                }
+                mac(1, k0 + KB);
             }
         }
-        if (u0 + ustep < nunit) wload(w[0], unit + ustep, 0);
+        if (u0 + ustep < nunit) {
+            wload(w[0], unit + ustep, 0);
+            xload(0, 0);
+        }
 #pragma unroll
         for (int r = 0; r < RW; ++r)
 #pragma unroll
@@ -301,11 +330,16 @@ int k_split(const GemvRtArgs& a, int mode) { return mode != GR_LOGITS && a.K >= 
 
 template <typename T, int NB, int MODE, int WK>
 void run_wk(hipStream_t s, const GemvRtArgs& a) {
-    size_t lds = (size_t)NB * a.K * sizeof(T) + (a.x ? 0 : (size_t)(a.D + a.groups) * sizeof(float));
+    const dim3 grid(gemv_rt_blocks(a, (GemvRtMode)MODE));
+    if (a.x) {
+        hipLaunchKernelGGL((k_gemv_rt<T, NB, MODE, WK, true>), grid, dim3(256), 0, s, a);
+        return;
+    }
+    const size_t lds = (size_t)NB * a.K * sizeof(T) + (size_t)(a.D + a.groups) * sizeof(float);
     if (lds > 60 * 1024)
-        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&k_gemv_rt<T, NB, MODE, WK>),
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&k_gemv_rt<T, NB, MODE, WK, false>),
                                   hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    hipLaunchKernelGGL((k_gemv_rt<T, NB, MODE, WK>), dim3(gemv_rt_blocks(a, (GemvRtMode)MODE)), dim3(256), lds, s, a);
+    hipLaunchKernelGGL((k_gemv_rt<T, NB, MODE, WK, false>), grid, dim3(256), lds, s, a);
 }
 
 template <typename T, int NB, int MODE>
@@ -338,6 +372,7 @@ void run_t(hipStream_t s, GemvRtMode mode, const GemvRtArgs& a) {
 // contiguous bytes of its weight row per 64-deep step (4 lanes: one 128-byte line), so the two MFMAs of a step
 // contract k = 16 lg .. 16 lg + 7 and 16 lg + 8 .. 16 lg + 15 of each lane group -- the activations (straight from
 // L2, B fragments) use the same order.  After the waves' sums meet in LDS, thread (n, b) runs the step's epilogue.
+// GR_F32 with gridDim.y > 1: K is cut over the y workgroups too, out holds their partial slabs [y][B][N].
 template <int MODE>
 __global__ void __launch_bounds__(256) k_skinny(GemvRtArgs a) {
     constexpr int NM = MODE == GR_GRU ? 3 : MODE == GR_SWIGLU ? 2 : 1;
@@ -356,14 +391,15 @@ __global__ void __launch_bounds__(256) k_skinny(GemvRtArgs a) {
 #pragma unroll
     for (int m = 0; m < NM; ++m) acc[m] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int nstep = (K + 63) / 64;
-    for (int s0 = wave; s0 < nstep; s0 += 4 * U) {
+    const int per = (nstep + gridDim.y - 1) / gridDim.y, s_end = min(nstep, (int)(blockIdx.y + 1) * per);
+    for (int s0 = blockIdx.y * per + wave; s0 < s_end; s0 += 4 * U) {
         uint4 w[U][NM][2], x[U][2];
 #pragma unroll
         for (int i = 0; i < U; ++i) {
             const int k = (s0 + 4 * i) * 64 + lg * 16;
 #pragma unroll
             for (int h = 0; h < 2; ++h) {
-                const bool ok = k + 8 * h < K;
+                const bool ok = s0 + 4 * i < s_end && k + 8 * h < K;
 #pragma unroll
                 for (int m = 0; m < NM; ++m) w[i][m][h] = ldg16_sel(wp[m] + k + 8 * h, ok, wp[m]);
                 x[i][h] = ldg16_sel(xp + k + 8 * h, ok, xp);
@@ -388,6 +424,11 @@ __global__ void __launch_bounds__(256) k_skinny(GemvRtArgs a) {
     for (int m = 0; m < NM; ++m)
 #pragma unroll
         for (int q = 0; q < 4; ++q) v[m] += sums[q][m][tid >> 4][b];
+    if constexpr (MODE == GR_F32) {
+        if (b < a.B && n < a.N)
+            reinterpret_cast<float*>(a.out)[((long)blockIdx.y * a.B + b) * a.ldo + n] = v[0];
+        return;
+    }
     if (b < a.B && n < a.N) step_epilogue<uint16_t, MODE>(a, n, b, v[0], v[1], v[2]);
     step_pads<uint16_t, MODE>(a);
 }
@@ -400,7 +441,7 @@ void run_skinny(hipStream_t s, GemvRtMode mode, const GemvRtArgs& a) {
         case GR_GRU: hipLaunchKernelGGL((k_skinny<GR_GRU>), grid, block, 0, s, a); break;
         case GR_SWIGLU: hipLaunchKernelGGL((k_skinny<GR_SWIGLU>), grid, block, 0, s, a); break;
         case GR_STREAMS: hipLaunchKernelGGL((k_skinny<GR_STREAMS>), grid, block, 0, s, a); break;
-        default: hipLaunchKernelGGL((k_skinny<GR_F32>), grid, block, 0, s, a); break;
+        default: hipLaunchKernelGGL((k_skinny<GR_F32>), dim3(grid.x, a.split < 1 ? 1 : a.split), block, 0, s, a); break;
     }
 }
 
@@ -544,7 +585,7 @@ __global__ void __launch_bounds__(256) k_decode_finish(const float* __restrict__
 }  // namespace
 
 int gemv_rt_max_batch() { return 16; }
-int gemv_rt_parts() { return 2 * 2048; }
+int gemv_rt_parts() { return 2 * 1024; }
 bool gemv_rt_reads_streams(int B) { return B <= 2; }
 
 bool gemv_rt_fits(int B, int K, Act act) {
@@ -552,9 +593,18 @@ bool gemv_rt_fits(int B, int K, Act act) {
     return act == ACT_BF16 && B <= gemv_rt_max_batch();
 }
 
+int gemv_rt_split(int B, int N, int K) {
+    if (B <= 2) return 1;
+    const int tiles = (N + 15) / 16, nstep = (K + 63) / 64;
+    int split = 1;
+    while (split < 8 && tiles * split < 512 && nstep / (split * 2) >= 4) split *= 2;
+    const int per = (nstep + split - 1) / split;  // no empty slice
+    return (nstep + per - 1) / per;
+}
+
 int gemv_rt_blocks(const GemvRtArgs& a, GemvRtMode mode) {
     const int units = (a.N + unit_outs(mode) - 1) / unit_outs(mode), upb = 4 / k_split(a, mode);
-    return std::max(1, std::min((units + upb - 1) / upb, 2048));
+    return std::max(1, std::min((units + upb - 1) / upb, 1024));
 }
 
 void gemv_rt(hipStream_t s, Act act, GemvRtMode mode, const GemvRtArgs& a) {

@@ -499,66 +499,111 @@ __global__ void __launch_bounds__(256) k_wattn_dm(WAttnDecodeArgs a) {
     }
     uint16_t* kc = reinterpret_cast<uint16_t*>(a.kc) + ((long)slot * a.G + g) * a.max_tokens * a.dp;
     uint16_t* vc = reinterpret_cast<uint16_t*>(a.vc) + ((long)slot * a.G + g) * a.max_tokens * a.ep;
-    if (k1 == i + 1) {  // the new token's cache rows (every head block of the group writes the same)
-        if (wave == 0) {
-            const uint16_t* src = qkv + a.H * a.d + g * a.d;
-            float ss = 0.0f;
-            for (int k = lane; k < a.d; k += 64) ss = fmaf(bf2f(src[k]), bf2f(src[k]), ss);
-            const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)a.d + a.eps);
-            for (int k = lane; k < a.dp; k += 64) kc[(long)i * a.dp + k] = k < a.d ? f2bf(bf2f(src[k]) * inv) : 0;
-        } else if (wave == 1) {
-            const uint16_t* src = qkv + (a.H + a.G) * a.d + g * a.e;
-            for (int k = lane; k < a.ep; k += 64) vc[(long)i * a.ep + k] = k < a.e ? src[k] : 0;
-        }
-    }
-    // this lane's query head: dims 8 lg .. 8 lg + 7 of every 32
+    // The new token (position i) never passes through the cache here: its score and value come from its qkv row, in
+    // wave 0 of the last split, which also writes its cache rows.  Cached keys end at kend.
+    const bool own = k1 == i + 1;
+    const int kend = own ? i : k1;
     const int h = g * R + r0 + (li < nr ? li : 0);
-    short8 qf[DQ / 32];
-    {
-        const uint16_t* src = qkv + h * a.d;
+    const uint16_t* kn = qkv + a.H * a.d + g * a.d;
+    const uint16_t* vn = qkv + (a.H + a.G) * a.d + g * a.e;
+    // first tile's loads, then the query's: all in flight together
+    uint4 vr[DV / 16], kr[2][DQ / 32];
+    auto gload = [&](int j0) {
+        const int jm = max(kend - 1, 0);
+#pragma unroll
+        for (int t = 0; t < 2; ++t) {
+            const uint16_t* p = kc + (long)min(j0 + t * 16 + li, jm) * a.dp;
+#pragma unroll
+            for (int c = 0; c < DQ / 32; ++c) kr[t][c] = ldg16_sel(p + c * 32 + 8 * lg, c * 32 + 8 * lg < a.dp, p);
+        }
+#pragma unroll
+        for (int x = 0; x < DV / 16; ++x) {
+            const int e = lane + 64 * x, r = e / (DV / 8), k = (e % (DV / 8)) * 8;
+            vr[x] = ldg16_sel(vc + (long)min(j0 + r, jm) * a.ep + k, k < a.ep, vc);
+        }
+    };
+    if (k0 + wave * 32 < kend) gload(k0 + wave * 32);
+    // a head row's dims 8 lg .. 8 lg + 7 of every 32, over its root mean square, as bf16
+    auto unit_row = [&](const uint16_t* src, short8 (&f)[DQ / 32]) {
         float q[DQ / 32][8], ss = 0.0f;
+        if (a.d % 8 == 0) {
+#pragma unroll
+            for (int c = 0; c < DQ / 32; ++c) {
+                const int k = c * 32 + 8 * lg;
+                ld8(src + (k < a.d ? k : 0), q[c]);
+#pragma unroll
+                for (int v = 0; v < 8; ++v) q[c][v] = k < a.d ? q[c][v] : 0.0f;
+            }
+        } else {
+#pragma unroll
+            for (int c = 0; c < DQ / 32; ++c)
+#pragma unroll
+                for (int v = 0; v < 8; ++v) {
+                    const int k = c * 32 + 8 * lg + v;
+                    q[c][v] = k < a.d ? bf2f(src[k]) : 0.0f;
+                }
+        }
 #pragma unroll
         for (int c = 0; c < DQ / 32; ++c)
 #pragma unroll
-            for (int v = 0; v < 8; ++v) {
-                const int k = c * 32 + 8 * lg + v;
-                q[c][v] = k < a.d ? bf2f(src[k]) : 0.0f;
-                ss = fmaf(q[c][v], q[c][v], ss);
-            }
+            for (int v = 0; v < 8; ++v) ss = fmaf(q[c][v], q[c][v], ss);
         ss += __shfl_xor(ss, 16, 64);
         ss += __shfl_xor(ss, 32, 64);
         const float inv = 1.0f / sqrtf(ss / (float)a.d + a.eps);
 #pragma unroll
         for (int c = 0; c < DQ / 32; ++c)
 #pragma unroll
-            for (int v = 0; v < 8; ++v) qf[c][v] = (short)f2bf(q[c][v] * inv);
-    }
+            for (int v = 0; v < 8; ++v) f[c][v] = (short)f2bf(q[c][v] * inv);
+    };
+    short8 qf[DQ / 32];
+    unit_row(qkv + h * a.d, qf);
     const float r1 = bf2f(a.r1[h]), r2 = bf2f(a.r2[h]), c1 = a.scale * kLog2e;
-    if (k1 == i + 1) {
-        __threadfence_block();
-        __syncthreads();
-    }
     f32x4 o[DV / 16];
 #pragma unroll
     for (int c = 0; c < DV / 16; ++c) o[c] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m = kNone, l = 0.0f;
-    for (int j0 = k0 + wave * 32; j0 < k1; j0 += 128) {
-        uint4 vr[DV / 16];
+    if (own && wave == 0) {
+        short8 kf[DQ / 32];
+        unit_row(kn, kf);
+        float dot = 0.0f;
 #pragma unroll
-        for (int x = 0; x < DV / 16; ++x) {
-            const int e = lane + 64 * x, r = e / (DV / 8), k = (e % (DV / 8)) * 8;
-            vr[x] = ldg16_sel(vc + (long)min(j0 + r, i) * a.ep + k, k < a.ep, vc);
+        for (int c = 0; c < DQ / 32; ++c)
+#pragma unroll
+            for (int v = 0; v < 8; ++v) dot = fmaf(bf2f((uint16_t)qf[c][v]), bf2f((uint16_t)kf[c][v]), dot);
+        dot += __shfl_xor(dot, 16, 64);
+        dot += __shfl_xor(dot, 32, 64);
+        m = dot * c1;  // distance 0: no bias; weight exp2(m - m) = 1
+        l = lg == 0 ? 1.0f : 0.0f;  // summed over the lane groups below
+        const bool vec = a.d % 8 == 0 && a.e % 8 == 0;
+#pragma unroll
+        for (int c = 0; c < DV / 16; ++c) {
+            const int k = c * 16 + 4 * lg;
+            float v[4];
+            if (vec) {
+                ld4(vn + (k < a.e ? k : 0), v);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) v[r] = k < a.e ? v[r] : 0.0f;
+            } else {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) v[r] = k + r < a.e ? bf2f(vn[k + r]) : 0.0f;
+            }
+#pragma unroll
+            for (int r = 0; r < 4; ++r) o[c][r] = v[r];
         }
+        if (li == 0) {
+#pragma unroll
+            for (int c = 0; c < DQ / 32; ++c)
+                if (c * 32 + 8 * lg < a.dp) *reinterpret_cast<short8*>(kc + (long)i * a.dp + c * 32 + 8 * lg) = kf[c];
+        }
+        for (int k = lane; k < a.ep; k += 64) vc[(long)i * a.ep + k] = k < a.e ? vn[k] : 0;
+    }
+    for (int j0 = k0 + wave * 32; j0 < kend; j0 += 128) {
         f32x4 st[2];
 #pragma unroll
         for (int t = 0; t < 2; ++t) {
             st[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-            const uint16_t* kr = kc + (long)min(j0 + t * 16 + li, i) * a.dp;
 #pragma unroll
-            for (int c = 0; c < DQ / 32; ++c) {
-                const int k = c * 32 + 8 * lg;
-                st[t] = mfma16(__builtin_bit_cast(short8, ldg16_sel(kr + k, k < a.dp, kr)), qf[c], st[t]);
-            }
+            for (int c = 0; c < DQ / 32; ++c) st[t] = mfma16(__builtin_bit_cast(short8, kr[t][c]), qf[c], st[t]);
         }
         float mt = m;
 #pragma unroll
@@ -566,7 +611,7 @@ __global__ void __launch_bounds__(256) k_wattn_dm(WAttnDecodeArgs a) {
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int j = j0 + t * 16 + 4 * lg + r;
-                st[t][r] = j < k1 ? biased(st[t][r], c1, r1, r2, (float)(i - j)) : -INFINITY;
+                st[t][r] = j < kend ? biased(st[t][r], c1, r1, r2, (float)(i - j)) : -INFINITY;
                 mt = fmaxf(mt, st[t][r]);
             }
         mt = fmaxf(mt, __shfl_xor(mt, 16, 64));
@@ -589,6 +634,7 @@ __global__ void __launch_bounds__(256) k_wattn_dm(WAttnDecodeArgs a) {
             *reinterpret_cast<uint4*>(&Vs[wave][r * VS + k]) = vr[x];
         }
         asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // this wave's own rows: no barrier
+        if (j0 + 128 < kend) gload(j0 + 128);
 #pragma unroll
         for (int c = 0; c < DV / 16; ++c) {
 #pragma unroll
@@ -609,17 +655,19 @@ __global__ void __launch_bounds__(256) k_wattn_dm(WAttnDecodeArgs a) {
 #pragma unroll
     for (int w = 0; w < 4; ++w) M = fmaxf(M, sml[w][li][0]);
     const float f = __builtin_amdgcn_exp2f(m - M);
-    float* os = reinterpret_cast<float*>(&Vs[0][0]);  // [wave][head][DV], in place of the value rows
+    float* os = reinterpret_cast<float*>(&Vs[0][0]);  // [wave][head][DV + 4], in place of the value rows
+    constexpr int OS = DV + 4;
+    static_assert(4 * 16 * OS * 4 <= 4 * 32 * VS * 2, "the sums fit the value rows");
 #pragma unroll
     for (int c = 0; c < DV / 16; ++c)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) os[(wave * 16 + li) * DV + c * 16 + 4 * lg + r] = o[c][r] * f;
+        *reinterpret_cast<float4*>(os + (wave * 16 + li) * OS + c * 16 + 4 * lg) =
+            make_float4(o[c][0] * f, o[c][1] * f, o[c][2] * f, o[c][3] * f);
     __syncthreads();
     for (int e = tid; e < nr * a.ep; e += 256) {
         const int r = e / a.ep, c = e % a.ep;
         float t = 0.0f;
 #pragma unroll
-        for (int w = 0; w < 4; ++w) t += os[(w * 16 + r) * DV + c];
+        for (int w = 0; w < 4; ++w) t += os[(w * 16 + r) * OS + c];
         part[(long)r * a.nsplit * rs + c] = t;
     }
     if (tid < nr) {
