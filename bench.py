@@ -65,6 +65,9 @@ def parse():
     ap.add_argument("--no-api", action="store_true",
                     help="skip the drop-in module API leg (inference.py's loop through PaliGemmaForConditionalGeneration)")
     ap.add_argument("--api-tokens", type=int, default=32)
+    ap.add_argument("--decoder", default=None, metavar="SIZES",
+                    help="measure the layered decoders instead (1b, 2b, 7b, with commas between; bench_decoder.py): one "
+                         "JSON line per size, one GPU")
     ap.add_argument("--dry-run", action="store_true",
                     help="rank logic only (world / batch / image shards / max-over-ranks timing / token gather) "
                          "over gloo with no GPU call: the CPU test of the N > 1 flow")
@@ -647,6 +650,10 @@ def run_dry(a, world, rank):
 
 def main():
     a = parse()
+    if a.decoder:
+        import bench_decoder
+        bench_decoder.run(a)
+        return
     if a.gpus > 1 and "WORLD_SIZE" not in os.environ:
         sys.exit(relaunch_multi(a))
     import torch

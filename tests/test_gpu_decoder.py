@@ -69,8 +69,8 @@ def test_matmul_any_shape(M, N, K, act):
     import ctypes
 
     from pgmi import _native as N_
-    if act == 2 and M * N * K > 1 << 30:
-        pytest.skip("the fp32 form has one tile shape")
+    if act == 2:  # the fp32 form has one tile shape: smaller sizes say as much
+        M, N = min(M, 200), min(N, 600)
     eng, _ = build(C.MECHANISMS["gru"], "float32")
     g = torch.Generator(device="cuda").manual_seed(M + N + K)
     A = torch.randn((M, K + 8), generator=g, device="cuda")
@@ -390,9 +390,8 @@ def test_generation_stop_tokens_and_sampling():
 
 # ---------------------------------------------------------------- loading, refusals, the runner
 def save(cfg, W, path):
-    from safetensors.numpy import save_file  # noqa: F401  (bf16 needs torch's)
-    from safetensors.torch import save_file as save_torch
-    save_torch({k: torch.from_numpy(v).bfloat16() for k, v in W.items()}, os.path.join(path, "model.safetensors"))
+    from safetensors.torch import save_file
+    save_file({k: torch.from_numpy(v).bfloat16() for k, v in W.items()}, os.path.join(path, "model.safetensors"))
     with open(os.path.join(path, "config.json"), "w") as f:
         json.dump(cfg, f)
 
@@ -439,6 +438,21 @@ def test_load_model_and_trace_runner(tmp_path):
             assert f.exists() == bool(w)
             if w:
                 close(np.fromfile(f, "<f4").reshape(len(w), -1).astype(np.float64), np.stack(w), dtype)
+
+
+def test_command_line(tmp_path):
+    from pgmi import registry
+    cfg = C.MIXED["a"]
+    save(cfg, O.random_weights(cfg, 11), tmp_path)
+    prompts = [tokens(cfg, 6, 95), tokens(cfg, 14, 96)]
+    want = registry.load_decoder(str(tmp_path)).generate(prompts, 7).cpu().tolist()
+    cmd = [sys.executable, "-m", "pgmi", "--model", str(tmp_path), "--max-new-tokens", "7"]
+    for p in prompts:
+        cmd += ["--prompt", ",".join(map(str, p))]
+    out = subprocess.run(cmd, capture_output=True, text=True, timeout=100,
+                         cwd=os.path.join(REPO, "multimodal-financial-analysis-tool-using-paligemma_amd"))
+    assert out.returncode == 0, out.stderr[-2000:]
+    assert [[int(t) for t in x.split(",")] for x in out.stdout.split()] == want
 
 
 def test_refusals():
