@@ -164,19 +164,23 @@ size_t wattn_decode_floats(int B, int H, int ep, int nsplit);
 void wattn_decode(hipStream_t s, Act act, const WAttnDecodeArgs& a);
 
 // ---------------------------------------------------------------- one token per sequence: fused projections
-// y = W x for B <= gemv_rt_max_batch() rows, one launch per projection: the input is rows of activations or
-// (gemv_rt_reads_streams) the streams' next read and norm (as streams_norm), the epilogue is the step that follows
-// the projection.
+// y = W x for a few rows, one launch per projection, the epilogue being the step that follows the projection.
+enum GemvRtForm : int {
+    GF_NONE = 0,    // too many rows: matmul_rt and the step kernels below
+    GF_STREAM = 1,  // weight-streaming GEMV; the input may be the streams' next read and norm (as streams_norm)
+    GF_SKINNY = 2,  // MFMA, up to gemv_rt_max_batch() rows of bf16 activations
+};
 enum GemvRtMode : int {
     GR_ACT = 0,      // out (activation type) = acc + bias
     GR_CONV = 1,     // rows < C: convolution step with the taps in place, silu -> out; rows >= C -> out2
     GR_GRU = 2,      // N channels, rows c, N + c, 2N + c (z, u, g): one minGRU step, state in place -> out
     GR_SWIGLU = 3,   // N channels, rows n, N + n: silu(gate) * up -> out
     GR_STREAMS = 4,  // X'[t] = sum_s mix[s][t] X[s] + wout[t] acc, in place
-    GR_LOGITS = 5,   // fp32 out + (B <= 2) per-workgroup argmax partials
-    GR_F32 = 6,      // fp32 out; B > 2: `split` partial slabs [split][B][ldo]
+    GR_LOGITS = 5,   // fp32 out + (GF_STREAM) per-workgroup argmax partials
+    GR_F32 = 6,      // fp32 out; GF_SKINNY: `split` partial slabs [split][B][ldo]
 };
 struct GemvRtArgs {
+    GemvRtForm form;
     int B, N, K;  // N: outputs (rows of W, or channels); K: padded to 8
     const uint16_t* W;
     int ldw;
@@ -210,9 +214,9 @@ struct GemvRtArgs {
 };
 int gemv_rt_max_batch();
 int gemv_rt_parts();  // words of pmax / pidx
-bool gemv_rt_reads_streams(int B);
-int gemv_rt_split(int B, int N, int K);  // slabs of a GR_F32 product
-bool gemv_rt_fits(int B, int K, Act act);
+GemvRtForm gemv_rt_form(int B, Act act, int streams, int width);
+bool gemv_rt_fits(GemvRtForm form, int K, Act act);
+int gemv_rt_split(GemvRtForm form, int N, int K);  // slabs of a GR_F32 product
 int gemv_rt_blocks(const GemvRtArgs& a, GemvRtMode mode);
 void gemv_rt(hipStream_t s, Act act, GemvRtMode mode, const GemvRtArgs& a);
 

@@ -463,9 +463,10 @@ int forward_body(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int rows, const
         fold(a, pend, rows);
         a.in = nullptr; a.w = d.fnorm; a.rows_idx = m.want;
         streams_norm(s, d.act, a);
-        if (gemv_rt_fits(n_want, d.head.k, d.act)) {
+        const GemvRtForm form = gemv_rt_form(n_want, d.act, 1, 1);
+        if (gemv_rt_fits(form, d.head.k, d.act)) {
             GemvRtArgs g{};
-            g.B = n_want; g.N = d.c.vocab; g.K = d.head.k; g.W = d.head.w; g.ldw = d.head.ldw; g.x = d.h; g.ldx = d.ldh;
+            g.form = form; g.B = n_want; g.N = d.c.vocab; g.K = d.head.k; g.W = d.head.w; g.ldw = d.head.ldw; g.x = d.h; g.ldx = d.ldh;
             g.out = logits; g.ldo = d.c.vocab;
             gemv_rt(s, d.act, GR_F32, g);
         } else {
@@ -488,11 +489,12 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
         a.ids = ids; a.in = d.W[0].sub[0].in; a.w = d.W[0].sub[0].norm;
         streams_norm(s, d.act, a);
     }
+    const GemvRtForm form = gemv_rt_form(B, d.act, d.c.streams, D);
     bool have_h = true;  // d.h holds the coming sublayer's input
     Pending pend;
     // the input side of a projection: d.h, or (fused) the streams' read and norm inside the GEMV
     auto base = [&](const Sub& sub, const Lin& w, bool fused) {
-        if (!have_h && (!fused || pend.y || !gemv_rt_reads_streams(B))) {
+        if (!have_h && (!fused || pend.y || form != GF_STREAM)) {
             StreamsArgs a = streams_args(d, B);
             fold(a, pend, B);
             a.in = sub.in; a.w = sub.norm;
@@ -501,7 +503,7 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
             have_h = true;
         }
         GemvRtArgs g{};
-        g.B = B; g.N = w.n; g.K = w.k; g.W = w.w; g.ldw = w.ldw; g.S = d.c.streams; g.D = D; g.groups = d.c.norm_groups;
+        g.form = form; g.B = B; g.N = w.n; g.K = w.k; g.W = w.w; g.ldw = w.ldw; g.S = d.c.streams; g.D = D; g.groups = d.c.norm_groups;
         g.eps = d.c.norm_eps; g.X = d.X; g.in = sub.in; g.nw = sub.norm; g.slot = d.slot; g.pos = d.pos;
         if (have_h) { g.x = d.h; g.ldx = d.ldh; }
         have_h = false;
@@ -509,14 +511,14 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
     };
     auto row_in = [&](const Lin& w, const void* in, int ldin) {
         GemvRtArgs g{};
-        g.B = B; g.N = w.n; g.K = w.k; g.W = w.w; g.ldw = w.ldw; g.x = in; g.ldx = ldin; g.slot = d.slot; g.pos = d.pos;
+        g.form = form; g.B = B; g.N = w.n; g.K = w.k; g.W = w.w; g.ldw = w.ldw; g.x = in; g.ldx = ldin; g.slot = d.slot; g.pos = d.pos;
         return g;
     };
     auto out_proj = [&](const Lin& o, const void* in, int ldin, const Sub& sub) {
-        const bool fits = gemv_rt_fits(B, o.k, d.act);
-        if (fits && !gemv_rt_reads_streams(B)) {  // the next streams pass sums the slabs
+        const bool fits = gemv_rt_fits(form, o.k, d.act);
+        if (fits && form != GF_STREAM) {  // the next streams pass sums the slabs
             GemvRtArgs g = row_in(o, in, ldin);
-            g.out = d.slabs; g.ldo = D; g.split = gemv_rt_split(B, D, o.k);
+            g.out = d.slabs; g.ldo = D; g.split = gemv_rt_split(form, D, o.k);
             gemv_rt(s, d.act, GR_F32, g);
             pend = {d.slabs, g.split, &sub};
         } else if (fits) {
@@ -532,7 +534,7 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
     for (int i = 0; i < d.c.n_layers; ++i) {
         const pgmi_layer_spec& l = d.L[i];
         const LayerW& w = d.W[i];
-        const bool fin = gemv_rt_fits(B, w.in.k, d.act);
+        const bool fin = gemv_rt_fits(form, w.in.k, d.act);
         if (l.mixer == PGMI_MIXER_MAMBA1) {
             const int C = l.inner, N = l.state, R = l.dt_rank, ldc = r8(C);
             float* taps = at<float>(state, st[i].a);
@@ -550,9 +552,9 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
                 a.z = d.p0 + (size_t)C * d.es; a.ldz = ldxz;
             }
             a.split = 1;
-            if (gemv_rt_fits(B, w.x.k, d.act)) {
+            if (gemv_rt_fits(form, w.x.k, d.act)) {
                 g = row_in(w.x, d.p1, ldc);
-                g.out = d.slabs; g.ldo = w.x.n; g.split = gemv_rt_split(B, w.x.n, w.x.k);
+                g.out = d.slabs; g.ldo = w.x.n; g.split = gemv_rt_split(form, w.x.n, w.x.k);
                 gemv_rt(s, d.act, GR_F32, g);
                 a.split = g.split;
             } else {
@@ -593,7 +595,7 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
             out_proj(w.o, d.p2, ldc, w.sub[0]);
         }
         if (l.ff) {
-            const bool fgu = gemv_rt_fits(B, w.gu.k, d.act);
+            const bool fgu = gemv_rt_fits(form, w.gu.k, d.act);
             GemvRtArgs g = base(w.sub[1], w.gu, fgu);
             if (fgu) {
                 g.N = l.ff; g.out = d.p2; g.ldo = r8(l.ff);
@@ -606,12 +608,12 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
         }
     }
     const Sub fin{nullptr, nullptr, nullptr, d.fnorm};
-    const bool fl = gemv_rt_fits(B, d.head.k, d.act);
+    const bool fl = gemv_rt_fits(form, d.head.k, d.act);
     GemvRtArgs g = base(fin, d.head, fl);
     if (fl) {
         g.out = logits; g.ldo = V; g.pmax = d.pmax; g.pidx = d.pidx;
         gemv_rt(s, d.act, GR_LOGITS, g);
-        const int parts = gemv_rt_reads_streams(B) ? gemv_rt_blocks(g, GR_LOGITS) : 0;
+        const int parts = form == GF_STREAM ? gemv_rt_blocks(g, GR_LOGITS) : 0;
         if (!parts) argmax_rows(s, logits, B, V, x->amax_v, x->amax_i, next);
         decode_finish(s, B, d.pmax, d.pidx, parts, next, hist, d.pos);
     } else {

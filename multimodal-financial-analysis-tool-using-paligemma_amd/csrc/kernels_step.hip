@@ -1,5 +1,5 @@
-// kernels_step.hip -- one token per sequence: projections as weight-streaming GEMVs (1 or 2 rows) or skinny MFMA
-// products (3 .. 16 rows) of any size with the surrounding steps fused (streams' read + grouped norm in front; convolution step, minGRU step, gated
+// kernels_step.hip -- one token per sequence: projections as weight-streaming GEMVs or skinny MFMA products
+// (up to 16 rows) of any size with the surrounding steps fused (streams' read + grouped norm in front; convolution step, minGRU step, gated
 // activation, streams' update or argmax behind), and the selective-scan step.
 #include <algorithm>
 
@@ -361,13 +361,7 @@ void run_mode(hipStream_t s, GemvRtMode mode, const GemvRtArgs& a) {
     }
 }
 
-template <typename T>
-void run_t(hipStream_t s, GemvRtMode mode, const GemvRtArgs& a) {
-    if (a.B <= 1) run_mode<T, 1>(s, mode, a);
-    else run_mode<T, 2>(s, mode, a);
-}
-
-// ---------------------------------------------------------------- 3 .. 16 rows: MFMA
+// ---------------------------------------------------------------- up to 16 rows: MFMA
 // A workgroup owns 16 outputs (of each of the unit's matrices) and all rows; its 4 waves split K.  A lane reads 32
 // contiguous bytes of its weight row per 64-deep step (4 lanes: one 128-byte line), so the two MFMAs of a step
 // contract k = 16 lg .. 16 lg + 7 and 16 lg + 8 .. 16 lg + 15 of each lane group -- the activations (straight from
@@ -586,15 +580,21 @@ __global__ void __launch_bounds__(256) k_decode_finish(const float* __restrict__
 
 int gemv_rt_max_batch() { return 16; }
 int gemv_rt_parts() { return 2 * 1024; }
-bool gemv_rt_reads_streams(int B) { return B <= 2; }
-
-bool gemv_rt_fits(int B, int K, Act act) {
-    if (B <= 2) return (size_t)2 * K * (act == ACT_F32 ? 4 : 2) <= 96 * 1024;
-    return act == ACT_BF16 && B <= gemv_rt_max_batch();
+GemvRtForm gemv_rt_form(int B, Act act, int streams, int width) {
+    // fp32 activations: no MFMA form.  bf16: one row, while every workgroup's own read of the streams stays small;
+    // measured, batch 1, 2 streams: width 1024 0.379 against 0.432 ms per step, 2048 0.802 / 0.818, 4096 0.828 / 0.661
+    if (act == ACT_F32) return B <= 2 ? GF_STREAM : GF_NONE;
+    if (B == 1 && streams * width <= 4096) return GF_STREAM;
+    return B <= gemv_rt_max_batch() ? GF_SKINNY : GF_NONE;
 }
 
-int gemv_rt_split(int B, int N, int K) {
-    if (B <= 2) return 1;
+bool gemv_rt_fits(GemvRtForm form, int K, Act act) {
+    if (form == GF_STREAM) return (size_t)2 * K * (act == ACT_F32 ? 4 : 2) <= 96 * 1024;
+    return form == GF_SKINNY;
+}
+
+int gemv_rt_split(GemvRtForm form, int N, int K) {
+    if (form != GF_SKINNY) return 1;
     const int tiles = (N + 15) / 16, nstep = (K + 63) / 64;
     int split = 1;
     while (split < 8 && tiles * split < 512 && nstep / (split * 2) >= 4) split *= 2;
@@ -608,9 +608,10 @@ int gemv_rt_blocks(const GemvRtArgs& a, GemvRtMode mode) {
 }
 
 void gemv_rt(hipStream_t s, Act act, GemvRtMode mode, const GemvRtArgs& a) {
-    if (a.B > 2) run_skinny(s, mode, a);
-    else if (act == ACT_F32) run_t<float>(s, mode, a);
-    else run_t<uint16_t>(s, mode, a);
+    if (a.form == GF_SKINNY) run_skinny(s, mode, a);
+    else if (act == ACT_BF16) run_mode<uint16_t, 1>(s, mode, a);
+    else if (a.B <= 1) run_mode<float, 1>(s, mode, a);
+    else run_mode<float, 2>(s, mode, a);
 }
 
 void conv_step(hipStream_t s, Act act, const void* xz, int ldxz, int B, int C, int K, const uint16_t* w,

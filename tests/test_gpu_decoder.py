@@ -151,16 +151,16 @@ def test_portions(name, sizes, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("lens", [[1, 70], [5, 1, 130], [64, 65, 63, 2, 129]])
+@pytest.mark.parametrize("lens", [[1, 70], [5, 1, 130], [64, 65, 63, 2, 129], [2 + r for r in range(17)]])
 def test_unequal_batch_then_decoding(lens, dtype):
     """Prompts of unequal lengths in one step, then single tokens together; sequences leave one by one, so every
-    batch size down to one is decoded (the fused GEMV form at 1 and 2, the batched form above)."""
+    batch size down to one is decoded (every form of the decode projections: one row, up to 16, more)."""
     cfg = C.MIXED["a"]
     eng, W = build(cfg, dtype)
     extra = 12
     seqs = [tokens(cfg, n + extra, 10 + n) for n in lens]
     want = [O.run(cfg, W, s) for s in seqs]
-    cache = eng.new_cache(8, 160)
+    cache = eng.new_cache(17, 160)
     slots = [cache.alloc() for _ in lens]
     lg = eng.step(cache, slots, [s[:n] for s, n in zip(seqs, lens)], want=list(range(sum(lens))))
     close(lg, np.concatenate([w[:n] for w, n in zip(want, lens)]), dtype)
