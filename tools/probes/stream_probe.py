@@ -37,12 +37,9 @@ def main():
     import ctypes
     hip = ctypes.CDLL("libamdhip64.so")
 
-    def hip_stream(flags, prio=None):
+    def hip_stream(flags):
         h = ctypes.c_void_p()
-        if prio is None:
-            assert hip.hipStreamCreateWithFlags(ctypes.byref(h), ctypes.c_uint(flags)) == 0
-        else:
-            assert hip.hipStreamCreateWithPriority(ctypes.byref(h), ctypes.c_uint(flags), ctypes.c_int(prio)) == 0
+        assert hip.hipStreamCreateWithFlags(ctypes.byref(h), ctypes.c_uint(flags)) == 0
         return torch.cuda.ExternalStream(h.value)
 
     def run(label, side, rotate, extra, graph=True, waits=False, nowait=False):
@@ -97,10 +94,8 @@ def main():
     return
     run("E main, eager (no graph)", False, False, False, graph=False)
     run("F side, eager (no graph)", True, False, False, graph=False)
-    run("G torch stream priority -1", torch.cuda.Stream(priority=-1), False, False)
     run("H hipStreamNonBlocking", hip_stream(1), False, False)
     run("I hipStreamDefault flags", hip_stream(0), False, False)
-    run("J hip priority stream -1", hip_stream(0, -1), False, False)
     s2 = torch.cuda.Stream()
     with torch.cuda.stream(s2):
         run("K a torch stream made current (as main)", False, False, False)
