@@ -169,7 +169,7 @@ __global__ void __launch_bounds__(256) k_wattn_m(WAttnArgs a) {
     const ChunkInfo tl = a.tiles[blockIdx.x];
     const SeqInfo sq = a.seqs[tl.seq];
     const int g = blockIdx.y, R = a.H / a.G;
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int li = lane & 15, lg = lane >> 4;
     const int nrow = sq.len * R;
     // this lane's query row
@@ -190,6 +190,9 @@ __global__ void __launch_bounds__(256) k_wattn_m(WAttnArgs a) {
     // keys the tile's rows see: [lo, hi]
     const int last = min(tl.rel + kWAttnRows, nrow) - 1;
     const int lo = max(0, sq.start + tl.rel / R - a.window + 1), hi = sq.start + last / R;
+    // positions of this wave's first and last rows
+    const int wfirst = sq.start + min(tl.rel + wave * 16, nrow - 1) / R;
+    const int wlast = sq.start + min(tl.rel + wave * 16 + 15, nrow - 1) / R;
     const uint16_t* kc = reinterpret_cast<const uint16_t*>(a.kc) + ((long)sq.slot * a.G + g) * a.max_tokens * a.dp;
     const uint16_t* vc = reinterpret_cast<const uint16_t*>(a.vc) + ((long)sq.slot * a.G + g) * a.max_tokens * a.ep;
     f32x4 o[DV / 16];
@@ -226,6 +229,7 @@ __global__ void __launch_bounds__(256) k_wattn_m(WAttnArgs a) {
         }
         __syncthreads();
         if (j0 + KT <= hi) gload(j0 + KT);
+        if (j0 > wlast || j0 + KT <= wfirst - a.window + 1) continue;  // no row of this wave sees the tile
         f32x4 st[4];
 #pragma unroll
         for (int t = 0; t < 4; ++t) {
@@ -237,16 +241,29 @@ __global__ void __launch_bounds__(256) k_wattn_m(WAttnArgs a) {
             }
         }
         float mt = m;
+        // 1 + r2 (i - j) for key j0 + 4 lg, less r2 per key after it
+        const float x0 = fmaf(r2, (float)(i - j0 - 4 * lg), 1.0f);
+        if (j0 + KT - 1 <= wfirst && wlast - j0 < a.window) {  // every row sees every key
 #pragma unroll
-        for (int t = 0; t < 4; ++t)
+            for (int t = 0; t < 4; ++t)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int j = j0 + t * 16 + 4 * lg + r;
-                const int dist = i - j;
-                const float s = biased(st[t][r], c1, r1, r2, (float)max(dist, 0));
-                st[t][r] = (unsigned)dist < (unsigned)a.window ? s : -INFINITY;
-                mt = fmaxf(mt, st[t][r]);
-            }
+                for (int r = 0; r < 4; ++r) {
+                    const float x = fmaf(-r2, (float)(t * 16 + r), x0);
+                    st[t][r] = fmaf(-r1, __builtin_amdgcn_logf(x), st[t][r] * c1);
+                    mt = fmaxf(mt, st[t][r]);
+                }
+        } else {
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int dist = i - (j0 + t * 16 + 4 * lg + r);
+                    const float x = fmaf(-r2, (float)(t * 16 + r), x0);
+                    const float s = fmaf(-r1, __builtin_amdgcn_logf(x), st[t][r] * c1);
+                    st[t][r] = (unsigned)dist < (unsigned)a.window ? s : -INFINITY;
+                    mt = fmaxf(mt, st[t][r]);
+                }
+        }
         mt = fmaxf(mt, __shfl_xor(mt, 16, 64));
         mt = fmaxf(mt, __shfl_xor(mt, 32, 64));
         const float alpha = __builtin_amdgcn_exp2f(m - mt);
@@ -260,10 +277,12 @@ __global__ void __launch_bounds__(256) k_wattn_m(WAttnArgs a) {
                 ls += st[t][r];
             }
         l = l * alpha + ls;  // this lane's keys; summed over the lane groups at the end
+        if (__any(alpha != 1.0f)) {
 #pragma unroll
-        for (int c = 0; c < DV / 16; ++c)
+            for (int c = 0; c < DV / 16; ++c)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) o[c][r] *= alpha;
+                for (int r = 0; r < 4; ++r) o[c][r] *= alpha;
+        }
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
             short8 pf;
