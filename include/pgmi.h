@@ -264,13 +264,14 @@ int pgmi_sample_top_p(pgmi_ctx* ctx, const float* x, int rows, int V, float temp
                       const float* u, int64_t* out, float* kept_mass, void* stream);
 
 /* ---- layered decoders: text models given as a list of layers, each a mixer (selective scan, windowed
- * attention, minimal gated recurrence) and an optional gated feed-forward, around residual streams
- * (hyper-connections) with grouped RMS norms.  A pgmi_ctx made by pgmi_decoder_create shares the
+ * attention, minimal gated recurrence) and an optional feed-forward (gated, or a mixture of experts), around
+ * residual streams (hyper-connections) with grouped RMS norms, or around one plain residual stream.  A pgmi_ctx made by pgmi_decoder_create shares the
  * weight-slab, loading, prepare, sampling and replica calls above; tensor names are the checkpoint's
  * ("embed", "l<i>.norm1", "l<i>.mix.in", ..., "final.norm"), all bf16 in the slab.
  *
  * State: one caller-owned slab of pgmi_kv_bytes(ctx, n_slots, max_tokens) bytes.  A slot holds one
- * sequence: per layer its convolution taps and scan state, recurrent state, or key / value rows.  A
+ * sequence: per layer its convolution taps and scan state, recurrent state, or key / value rows and the last
+ * inputs of its input convolution; and the sequence's token ids where the embedding reads pairs.  A
  * sequence starts at position 0, which reads nothing of what its slot held before. */
 #define PGMI_MIXER_MAMBA1 0
 #define PGMI_MIXER_ATTENTION 1
@@ -283,7 +284,21 @@ typedef struct pgmi_layer_spec {
     int heads, kv_heads, dim, vdim;     /* attention: query / key-value heads, query-key and value head sizes */
     int window;                         /* attention: position i sees j with 0 <= i - j < window */
     float scale;                        /* attention: factor of q . k */
-    int ff;                             /* feed-forward size, 0: none */
+    int ff;                             /* gated feed-forward size, 0: none */
+    /* attention, continued */
+    int qk_norm, v_norm;                /* heads over their root mean square: queries and keys; values */
+    int proj_bias, distance_bias;       /* q, k, v have biases; r1 ln(1 + r2 distance) is taken off the scores */
+    int keep_first;                     /* position i also sees every j <= i with j < keep_first */
+    int kv_from;                        /* >= 0: the earlier attention layer whose keys and values are read; -1: own */
+    float softcap;                      /* > 0: score = softcap tanh(score / softcap) */
+    int rot_dims;                       /* leading dims of a q / k head rotated in pairs (2i, 2i + 1), 0: none */
+    double rot_base;                    /* pair i turns by position * base^(-2i / rot_dims), scaled by wavelength: */
+    double rot_factor, rot_low, rot_high, rot_original; /* longer than original / low: / factor; shorter than
+                                                          * original / high: kept; blended between.  original 0: none */
+    /* feed-forward as a mixture of experts (experts > 0; then ff is 0) */
+    int experts, identity;              /* gated experts, and experts that return their input */
+    int top, groups, groups_keep;       /* experts per token, from the groups_keep best of `groups` equal groups */
+    int expert_ff, shared_ff;           /* sizes; shared_ff 0: no shared expert */
 } pgmi_layer_spec;
 
 typedef struct pgmi_decoder_config {
@@ -291,6 +306,13 @@ typedef struct pgmi_decoder_config {
     float norm_eps, embed_scale;
     int max_batch;  /* sequences per call */
     int act_dtype;  /* PGMI_DTYPE_BF16, or PGMI_DTYPE_F32: activations, caches and products in fp32 */
+    int plain_residual;    /* one residual stream without hyper-connections: x + residual_mult * sublayer */
+    float residual_mult;
+    int norm_scalar;       /* RMS norms weigh every coordinate with one number (plain_residual only) */
+    int canon_taps;        /* > 0: a mixer reads h + conv(h), a causal convolution of this many taps (plain_residual) */
+    int bigram_buckets;    /* > 0: a row of "bigram" [buckets + 1][width] is added to the token's (plain_residual) */
+    int64_t bigram_mul_prev, bigram_mul_cur; /* row (previous * mul_prev + current * mul_cur) mod buckets; first: last */
+    int untied_head;       /* logits from "head" instead of "embed" */
 } pgmi_decoder_config;
 
 int pgmi_decoder_create(int device, const pgmi_decoder_config* cfg, const pgmi_layer_spec* layers, pgmi_ctx** out);

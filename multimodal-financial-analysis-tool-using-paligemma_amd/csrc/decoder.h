@@ -49,6 +49,137 @@ struct StreamsArgs {
 };
 void streams_norm(hipStream_t s, Act act, const StreamsArgs& a);
 
+// ---------------------------------------------------------------- one residual stream
+// The outputs of a mixture of experts, folded into the residual row by row: sum_k w[k] (expert sel[k]'s output), where a
+// chosen expert >= experts is an identity: its output is the mixture's input h.
+struct ExpertMix {
+    const void* y;  // [rows * top][ldy] activation type: entry row * top + k
+    int ldy;
+    const int* sel;  // [rows][top]
+    const float* w;  // [rows][top]
+    int top, experts;
+    const void* h;  // [rows][ldh]
+    int ldh;
+    const float* gate;  // [rows]: factor of ResidualArgs.y (the shared expert's output), null: 1
+};
+// X [rows][D] fp32.  First X is made (ids: embed[token] * escale, plus a row of a table indexed by token pairs) or
+// updated in place, X += mult (y + mix) with y in `ysplit` fp32 slabs; then h = X over its root mean square times w.
+// rows_idx: only these rows (h compact), X left alone.
+struct ResidualArgs {
+    float* X;
+    int rows, D;
+    const int64_t* ids;
+    const uint16_t* E;
+    float escale;
+    int vocab;
+    // pairs: row (previous * mul_prev + current * mul_cur) mod buckets of `pairs`, row `buckets` at position 0;
+    // history [slot][max_tokens] holds every sequence's tokens by position (null: no pairs)
+    const uint16_t* pairs;
+    int64_t mul_prev, mul_cur;
+    int buckets;
+    int* history;
+    int max_tokens;
+    const float* y;  // null: nothing to add from here
+    int ysplit;
+    long ystride;
+    ExpertMix mix;  // mix.y null: none
+    float mult;
+    const uint16_t* w;  // norm weights [D], or one number
+    int w_scalar;
+    float eps;
+    void* h;  // null: no norm
+    int ldh;  // columns D .. ldh-1 are written as zeros
+    float* inv;  // optional [rows]: 1 / root mean square (with h null: instead of it)
+    const int* rows_idx;
+    float* tap;  // optional [rows][D]: X after the update
+    int* zero;   // optional: nzero words cleared
+    int nzero;
+    // where a row stands: packed sequences, or (seqs null) one row per sequence
+    const SeqInfo* seqs;
+    const int* row_seq;
+    const int* slot;
+    const int* pos;
+    // one row per sequence: h also takes the input convolution's step (taps > 0), see CanonArgs
+    const uint16_t* cw;
+    int taps;
+    float* ring;
+};
+void residual_norm(hipStream_t s, Act act, const ResidualArgs& a);
+
+// Input convolution over packed rows: n = X * inv * w is what the norm gives, h = n + conv(n),
+// conv(n)_t = sum_j cw[:, j] n_(t - taps + 1 + j), zeros before the sequence.  ring [slot][taps][D] fp32 keeps the norm of
+// position p in row p % taps; the last taps - 1 of every sequence are written once h is complete.
+struct CanonArgs {
+    const float* X;
+    const float* inv;
+    const uint16_t* w;
+    int w_scalar;
+    int rows, D, taps;
+    const uint16_t* cw;  // [D][taps]
+    float* ring;
+    void* h;
+    int ldh;
+    const SeqInfo* seqs;
+    int nseq;
+    const ChunkInfo* chunks;
+    int nchunk;
+};
+void canon(hipStream_t s, Act act, const CanonArgs& a);
+
+// ---------------------------------------------------------------- mixture of experts
+// z: fp32 slabs [split][rows][ldz], summed: columns 0 .. n-1 the router's logits, column n the shared expert's gate (gate
+// != null).  Scores are their softmax; choice = score + correction picks the groups (largest choice of a group, `keep` of
+// `groups` equal ones) and the top experts inside them; weights are the scores.  Lists: list[e * cap ..] the entries
+// (row * top + k) of expert e < experts, cnt[e] how many.
+struct RouteArgs {
+    const float* z;
+    int split;
+    long zstride;
+    int ldz, rows, n, experts, top, groups, keep;
+    const uint16_t* correction;
+    int* sel;
+    float* w;
+    float* gate;
+    int* cnt;  // zeroed before the launch, unless active is given
+    int* list;
+    int cap;
+    int* active;  // up to kRouteRows rows: cnt is set, active[0] experts are used, active[1 ..] which
+};
+constexpr int kRouteRows = 16;
+constexpr int kMaxExperts = 512;  // identity experts included: a workgroup's choice scores fit LDS
+void route(hipStream_t s, const RouteArgs& a);
+
+// One product of every expert over the rows that chose it: entry -> row entry / gather of A (gather: `top` where A is
+// the mixture's input, 1 where it is per entry), W + e * wstride, out row = entry.
+enum ExpertMode : int {
+    EX_SWIGLU = 0,  // silu(A . W_gate^T) * (A . W_up^T), W = N gate rows, then N up rows
+    EX_STORE = 1,
+};
+struct ExpertArgs {
+    const void* A;
+    int lda, gather;
+    const uint16_t* W;
+    int ldw;
+    long wstride;
+    int N, K;
+    void* out;
+    int ldo;  // columns N .. ldo-1 are written as zeros
+    const int* cnt;
+    const int* list;
+    int cap, experts, entries;  // entries: rows * top
+    // few rows (RouteArgs.active given): the shared expert rides along, its rows 0 .. B-1 (Wsh null: none)
+    const int* active;
+    const uint16_t* Wsh;
+    int ldwsh, Nsh, Ksh;
+    const void* Ash;
+    int ldash, B;
+    void* outsh;
+    int ldosh;
+};
+void experts_rt(hipStream_t s, Act act, ExpertMode mode, const ExpertArgs& a);
+// the same for up to kRouteRows rows of bf16 activations, the shared expert included (EX_STORE: its output is fp32)
+void experts_skinny(hipStream_t s, ExpertMode mode, const ExpertArgs& a);
+
 // ---------------------------------------------------------------- matrix products, any M, N, K (K a multiple of 8)
 // C = A [M][lda] . W [N][ldw]^T
 enum RtOut : int {
@@ -111,24 +242,39 @@ struct GruArgs {
 };
 void mingru_scan(hipStream_t s, Act act, const GruArgs& a);
 
-// ---------------------------------------------------------------- windowed attention with a distance bias
-// qkv rows [q: H d | k: G d | v: G e]; q and k are divided by their root mean square per head; the cache holds
-// the normalised k: K [slot][G][max_tokens][dp], V [slot][G][max_tokens][ep], activation type, dp / ep = d / e
-// rounded up to 8 with zero pads
+// ---------------------------------------------------------------- windowed attention
+// qkv rows [q: H d | k: G d | v: G e] (no k and v when own_kv is false: the cache is another layer's).  What the cache
+// holds: K [slot][G][max_tokens][dp] after head norm and rotation, V [slot][G][max_tokens][ep] after head norm,
+// activation type, dp / ep = d / e rounded up to 8 with zero pads.
+struct WAttnHeads {
+    int H, G, d, e, dp, ep;
+    bool own_kv;
+    bool qk_norm, v_norm;  // heads over their root mean square
+    float eps;
+    const double* turns;   // [rot / 2] turns per position of the pairs (2i, 2i + 1) of q and k
+    int rot;               // rotated leading dims, 0: none
+};
+// Which keys a query sees, and what becomes of its score q . k scale:
+//   position i sees j <= i with i - j < window or j < keep
+//   cap > 0: cap tanh(score / cap);  r1: r1[h] ln(1 + r2[h] (i - j)) is taken off (one of the two at most)
+struct WAttnScore {
+    int window, keep;
+    float scale, cap;
+    const uint16_t* r1;  // [H], null: no distance bias
+    const uint16_t* r2;
+};
 struct WAttnArgs {
+    WAttnHeads hd;
+    WAttnScore sc;
     const void* qkv;
     int ldqkv;
-    void* q;  // normalised q [rows][H][dp]
+    void* q;  // queries after norm and rotation [rows][H][dp]
     void* kc;
     void* vc;
     int max_tokens;
     void* o;  // [rows][ldo], head-major H * e
     int ldo;
-    int rows, H, G, d, e, dp, ep;
-    int window;  // position i sees j with 0 <= i - j < window
-    float scale, eps;
-    const uint16_t* r1;  // [H]: r1 ln(1 + r2 (i - j)) is taken off the score
-    const uint16_t* r2;
+    int rows;
     const SeqInfo* seqs;
     int nseq;
     const int* row_seq;  // [rows]
@@ -142,6 +288,8 @@ void wattn_prefill(hipStream_t s, Act act, const WAttnArgs& a);
 // one new token per sequence: row b of qkv (activation type [B][ldqkv], biases added) is position pos[b] of slot[b]; appends
 // its k and v, attends, and leaves the heads' outputs in o [B][ldo].  part: fp32 scratch of wattn_decode_floats().
 struct WAttnDecodeArgs {
+    WAttnHeads hd;
+    WAttnScore sc;
     const void* qkv;
     int ldqkv;
     void* kc;
@@ -149,17 +297,13 @@ struct WAttnDecodeArgs {
     int max_tokens;
     void* o;
     int ldo;
-    int B, H, G, d, e, dp, ep;
-    int window;
-    float scale, eps;
-    const uint16_t* r1;
-    const uint16_t* r2;
+    int B;
     const int* slot;
     const int* pos;
     float* part;
     int nsplit;
 };
-int wattn_decode_splits(int B, int G, int window, int max_tokens);
+int wattn_decode_splits(int B, int G, const WAttnScore& sc, int max_tokens);
 size_t wattn_decode_floats(int B, int H, int ep, int nsplit);
 void wattn_decode(hipStream_t s, Act act, const WAttnDecodeArgs& a);
 
@@ -204,9 +348,10 @@ struct GemvRtArgs {
     float* state;
     const int* slot;
     const int* pos;
-    // GR_STREAMS
+    // GR_STREAMS; mix null: one stream, X += mult acc
     const uint16_t* mix;
     const uint16_t* wout;
+    float mult;
     int split;  // GR_F32
     // GR_LOGITS
     float* pmax;

@@ -1,5 +1,5 @@
 // engine_decoder.hip -- the layered-decoder family of libpgmi: a text model described as a list of layers, each a
-// mixer and an optional feed-forward, around residual streams.  Weight layout, derived tensors, the per-sequence
+// mixer and an optional feed-forward, around residual streams or one plain residual.  Weight layout, derived tensors, the per-sequence
 // state slab, the ragged forward (prompts and portions of prompts) and the decode step (hipGraph-replayed), over
 // the mechanisms of decoder.h.  A design is its layer list and constants; nothing here names one.
 #include <set>
@@ -17,7 +17,7 @@ struct Lin {
     int n = 0, k = 0, ldw = 0;
 };
 
-struct Sub {  // one residual sublayer's stream weights and norm
+struct Sub {  // one residual sublayer's stream weights (null: plain residual) and norm
     const uint16_t *in, *out, *mix, *norm;
 };
 
@@ -26,7 +26,11 @@ struct LayerW {
     Lin in;    // mamba1: in; attention: q|k|v; mingru: z|x|g
     Lin x, dt;  // mamba1
     Lin o;
-    Lin gu, down;  // feed-forward
+    Lin gu, down;  // feed-forward, or the shared expert
+    Lin router;    // with the shared expert's gate as its last row
+    Lin egu, ed;   // every expert's gate|up and down, expert after expert
+    const uint16_t *correction = nullptr, *canon = nullptr;
+    const double* turns = nullptr;  // rotary: turns per position of every pair
     const uint16_t* bias = nullptr;  // of `in`
     const uint16_t *conv = nullptr, *conv_b = nullptr, *dt_b = nullptr, *A_log = nullptr, *D = nullptr, *r1 = nullptr,
                    *r2 = nullptr;
@@ -34,6 +38,12 @@ struct LayerW {
 
 struct StateAt {  // byte offsets of a layer's regions in the state slab
     int64_t a = 0, b = 0;  // mamba1: taps, scan state; attention: keys, values; mingru: state
+    int64_t ring = 0;      // last inputs of the input convolution
+};
+struct StateMap {
+    std::vector<StateAt> at;
+    int64_t history = 0;  // tokens by position, where the embedding reads pairs
+    int64_t bytes = 0;
 };
 
 }  // namespace
@@ -44,7 +54,7 @@ struct DecoderState {
     std::vector<LayerW> W;
     Act act;
     int es;  // bytes per activation element
-    const uint16_t *embed = nullptr, *fnorm = nullptr;
+    const uint16_t *embed = nullptr, *fnorm = nullptr, *pairs = nullptr;
     Lin head;
     std::vector<void*> derived;  // padded weights, joined biases
     // workspace of `rows` rows, `chunks` scan chunks and `gchunks` chunks of the gated recurrence
@@ -52,6 +62,10 @@ struct DecoderState {
     void* arena = nullptr;
     float *X = nullptr, *slabs = nullptr, *dt = nullptr, *bc = nullptr, *cstate = nullptr, *csum = nullptr;
     uint8_t *h = nullptr, *p0 = nullptr, *p1 = nullptr, *p2 = nullptr, *dtl = nullptr;
+    // mixture of experts: activations and outputs per entry, choices, weights, gates, lists, counters, used experts
+    uint8_t *ea = nullptr, *ey = nullptr;
+    float *inv = nullptr, *ew = nullptr, *egate = nullptr;
+    int *esel = nullptr, *elist = nullptr, *ecnt = nullptr, *eactive = nullptr;
     size_t slab_bytes = 0;
     int ldh = 0, ld0 = 0, ld1 = 0, ld2 = 0, ldd = 0;
     // step metadata
@@ -91,19 +105,30 @@ void add_joined(pgmi_ctx* x, const std::vector<std::pair<std::string, std::vecto
     x->slab_bytes = (x->slab_bytes + 255) / 256 * 256;
 }
 
+int qkv_rows(const pgmi_layer_spec& l) { return l.heads * l.dim + (l.kv_from < 0 ? l.kv_heads * (l.dim + l.vdim) : 0); }
+bool has_ff(const pgmi_layer_spec& l) { return l.ff > 0 || l.experts > 0; }
+
 void build_decoder_layout(pgmi_ctx* x) {
     const DecoderState& d = *x->dec;
     const int64_t D = d.c.width, S = d.c.streams;
+    auto add_norm = [&](const std::string& name) {
+        if (d.c.norm_scalar) add_slot(x, name, {});
+        else add_slot(x, name, {D});
+    };
     add_slot(x, "embed", {d.c.vocab, D});
+    if (d.c.untied_head) add_slot(x, "head", {d.c.vocab, D});
+    if (d.c.bigram_buckets) add_slot(x, "bigram", {(int64_t)d.c.bigram_buckets + 1, D});
     for (int i = 0; i < d.c.n_layers; ++i) {
         const pgmi_layer_spec& l = d.L[i];
-        for (int q = 1; q <= (l.ff ? 2 : 1); ++q) {
+        for (int q = 1; q <= (has_ff(l) ? 2 : 1); ++q) {
             const std::string n = std::to_string(q);
-            add_slot(x, lname(i, "norm") + n, {D});
+            add_norm(lname(i, "norm") + n);
+            if (d.c.plain_residual) continue;
             add_slot(x, lname(i, "hc") + n + ".in", {S});
             add_slot(x, lname(i, "hc") + n + ".out", {S});
             add_slot(x, lname(i, "hc") + n + ".mix", {S, S});
         }
+        if (d.c.canon_taps) add_slot(x, lname(i, "canon1"), {D, d.c.canon_taps});
         if (l.mixer == PGMI_MIXER_MAMBA1) {
             const int64_t C = l.inner, N = l.state, R = l.dt_rank;
             add_slot(x, lname(i, "mix.in"), {2 * C, D});
@@ -117,10 +142,18 @@ void build_decoder_layout(pgmi_ctx* x) {
             add_slot(x, lname(i, "mix.o"), {D, C});
         } else if (l.mixer == PGMI_MIXER_ATTENTION) {
             const int64_t q = (int64_t)l.heads * l.dim, k = (int64_t)l.kv_heads * l.dim, v = (int64_t)l.kv_heads * l.vdim;
-            add_joined(x, {{lname(i, "mix.q"), {q, D}}, {lname(i, "mix.k"), {k, D}}, {lname(i, "mix.v"), {v, D}}});
-            add_joined(x, {{lname(i, "mix.q.b"), {q}}, {lname(i, "mix.k.b"), {k}}, {lname(i, "mix.v.b"), {v}}});
-            add_slot(x, lname(i, "mix.r1"), {l.heads});
-            add_slot(x, lname(i, "mix.r2"), {l.heads});
+            if (l.kv_from < 0) {
+                add_joined(x, {{lname(i, "mix.q"), {q, D}}, {lname(i, "mix.k"), {k, D}}, {lname(i, "mix.v"), {v, D}}});
+                if (l.proj_bias)
+                    add_joined(x, {{lname(i, "mix.q.b"), {q}}, {lname(i, "mix.k.b"), {k}}, {lname(i, "mix.v.b"), {v}}});
+            } else {
+                add_slot(x, lname(i, "mix.q"), {q, D});
+                if (l.proj_bias) add_slot(x, lname(i, "mix.q.b"), {q});
+            }
+            if (l.distance_bias) {
+                add_slot(x, lname(i, "mix.r1"), {l.heads});
+                add_slot(x, lname(i, "mix.r2"), {l.heads});
+            }
             add_slot(x, lname(i, "mix.o"), {D, (int64_t)l.heads * l.vdim});
         } else {
             const int64_t C = l.width;
@@ -132,38 +165,62 @@ void build_decoder_layout(pgmi_ctx* x) {
             add_joined(x, {{lname(i, "mlp.gate"), {l.ff, D}}, {lname(i, "mlp.up"), {l.ff, D}}});
             add_slot(x, lname(i, "mlp.down"), {D, l.ff});
         }
+        if (l.experts) {
+            const int64_t n = l.experts + l.identity;
+            std::vector<std::pair<std::string, std::vector<int64_t>>> gu, down, router = {{lname(i, "mlp.router"), {n, D}}};
+            for (int e = 0; e < l.experts; ++e) {
+                const std::string at = lname(i, "mlp.e") + std::to_string(e);
+                gu.push_back({at + ".gate", {l.expert_ff, D}});
+                gu.push_back({at + ".up", {l.expert_ff, D}});
+                down.push_back({at + ".down", {D, l.expert_ff}});
+            }
+            add_joined(x, gu);
+            add_joined(x, down);
+            if (l.shared_ff) router.push_back({lname(i, "mlp.shared.sg"), {1, D}});
+            add_joined(x, router);
+            add_slot(x, lname(i, "mlp.correction"), {n});
+            if (l.shared_ff) {
+                add_joined(x, {{lname(i, "mlp.shared.gate"), {l.shared_ff, D}}, {lname(i, "mlp.shared.up"), {l.shared_ff, D}}});
+                add_slot(x, lname(i, "mlp.shared.down"), {D, l.shared_ff});
+            }
+        }
     }
-    add_slot(x, "final.norm", {D});
+    if (d.c.norm_scalar) add_slot(x, "final.norm", {});
+    else add_slot(x, "final.norm", {D});
 }
 
-// the state slab's regions for n_slots sequences of up to max_tokens; returns the total
-int64_t state_layout(const DecoderState& d, int n_slots, int max_tokens, std::vector<StateAt>* at) {
-    int64_t off = 0;
+// the state slab's regions for n_slots sequences of up to max_tokens
+StateMap state_layout(const DecoderState& d, int n_slots, int max_tokens) {
+    StateMap m;
     auto take = [&](int64_t bytes) {
-        const int64_t o = off;
-        off += (bytes + 255) / 256 * 256;
+        const int64_t o = m.bytes;
+        m.bytes += (bytes + 255) / 256 * 256;
         return o;
     };
-    if (at) at->assign(d.c.n_layers, {});
+    m.at.assign(d.c.n_layers, {});
     for (int i = 0; i < d.c.n_layers; ++i) {
         const pgmi_layer_spec& l = d.L[i];
-        StateAt s;
+        StateAt& s = m.at[i];
         if (l.mixer == PGMI_MIXER_MAMBA1) {
             s.a = take((int64_t)n_slots * (l.conv - 1) * l.inner * 4);
             s.b = take((int64_t)n_slots * l.inner * l.state * 4);
-        } else if (l.mixer == PGMI_MIXER_ATTENTION) {
+        } else if (l.mixer == PGMI_MIXER_ATTENTION && l.kv_from < 0) {
             s.a = take((int64_t)n_slots * l.kv_heads * max_tokens * r8(l.dim) * d.es);
             s.b = take((int64_t)n_slots * l.kv_heads * max_tokens * r8(l.vdim) * d.es);
+        } else if (l.mixer == PGMI_MIXER_ATTENTION) {
+            s.a = m.at[l.kv_from].a;
+            s.b = m.at[l.kv_from].b;
         } else {
             s.a = take((int64_t)n_slots * l.width * 4);
         }
-        if (at) (*at)[i] = s;
+        if (d.c.canon_taps > 1) s.ring = take((int64_t)n_slots * d.c.canon_taps * d.c.width * 4);
     }
-    return off;
+    if (d.c.bigram_buckets) m.history = take((int64_t)n_slots * max_tokens * 4);
+    return m;
 }
 
 int64_t decoder_state_bytes(const pgmi_ctx* x, int batch, int max_tokens) {
-    return state_layout(*x->dec, batch, max_tokens, nullptr);
+    return state_layout(*x->dec, batch, max_tokens).bytes;
 }
 
 int derived_alloc(DecoderState& d, uint16_t** p, size_t elems) {
@@ -187,6 +244,32 @@ int make_lin(DecoderState& d, const uint16_t* w, int n, int k, Lin* out) {
     return 0;
 }
 
+// turns per position of the rotated pairs: base^(-2i / dims) over a full turn, scaled by wavelength
+int make_turns(DecoderState& d, const pgmi_layer_spec& l, const double** out) {
+    if (!l.rot_dims) return 0;
+    constexpr double kTurn = 6.283185307179586476925286766559;
+    std::vector<double> t;
+    for (int i = 0; i < l.rot_dims / 2; ++i) {
+        double f = std::pow(l.rot_base, -2.0 * i / l.rot_dims);
+        if (l.rot_original > 0) {
+            const double wave = kTurn / f;
+            if (wave > l.rot_original / l.rot_low) {
+                f /= l.rot_factor;
+            } else if (!(wave < l.rot_original / l.rot_high)) {
+                const double s = (l.rot_original / wave - l.rot_low) / (l.rot_high - l.rot_low);
+                f = (1.0 - s) * f / l.rot_factor + s * f;
+            }
+        }
+        t.push_back(f / kTurn);
+    }
+    uint16_t* p;
+    int rc;
+    if ((rc = derived_alloc(d, &p, t.size() * 4))) return rc;
+    HIPCHK(hipMemcpy(p, t.data(), t.size() * sizeof(double), hipMemcpyHostToDevice));
+    *out = reinterpret_cast<const double*>(p);
+    return 0;
+}
+
 void drop_derived(DecoderState& d) {
     for (void* p : d.derived) (void)hipFree(p);
     d.derived.clear();
@@ -201,16 +284,18 @@ int decoder_prepare(pgmi_ctx* x) {
     const int D = d.c.width, B = d.c.max_batch;
     d.embed = W(x, "embed");
     d.fnorm = W(x, "final.norm");
-    if ((rc = make_lin(d, d.embed, d.c.vocab, D, &d.head))) return rc;
+    d.pairs = W(x, "bigram");
+    if ((rc = make_lin(d, d.c.untied_head ? W(x, "head") : d.embed, d.c.vocab, D, &d.head))) return rc;
     d.W.assign(d.c.n_layers, {});
     for (int i = 0; i < d.c.n_layers; ++i) {
         const pgmi_layer_spec& l = d.L[i];
         LayerW& w = d.W[i];
-        for (int q = 0; q < (l.ff ? 2 : 1); ++q) {
+        for (int q = 0; q < (has_ff(l) ? 2 : 1); ++q) {
             const std::string n = std::to_string(q + 1);
             w.sub[q] = {W(x, lname(i, "hc") + n + ".in"), W(x, lname(i, "hc") + n + ".out"), W(x, lname(i, "hc") + n + ".mix"),
                         W(x, lname(i, "norm") + n)};
         }
+        w.canon = W(x, lname(i, "canon1"));
         auto lin = [&](const char* name, int n, int k, Lin* o) { return make_lin(d, W(x, lname(i, name)), n, k, o); };
         if (l.mixer == PGMI_MIXER_MAMBA1) {
             if ((rc = lin("mix.in", 2 * l.inner, D, &w.in))) return rc;
@@ -223,7 +308,8 @@ int decoder_prepare(pgmi_ctx* x) {
             w.A_log = W(x, lname(i, "mix.A_log"));
             w.D = W(x, lname(i, "mix.D"));
         } else if (l.mixer == PGMI_MIXER_ATTENTION) {
-            if ((rc = lin("mix.q", l.heads * l.dim + l.kv_heads * (l.dim + l.vdim), D, &w.in))) return rc;
+            if ((rc = lin("mix.q", qkv_rows(l), D, &w.in))) return rc;
+            if ((rc = make_turns(d, l, &w.turns))) return rc;
             if ((rc = lin("mix.o", D, l.heads * l.vdim, &w.o))) return rc;
             w.bias = W(x, lname(i, "mix.q.b"));
             w.r1 = W(x, lname(i, "mix.r1"));
@@ -240,6 +326,16 @@ int decoder_prepare(pgmi_ctx* x) {
         if (l.ff) {
             if ((rc = lin("mlp.gate", 2 * l.ff, D, &w.gu))) return rc;
             if ((rc = lin("mlp.down", D, l.ff, &w.down))) return rc;
+        }
+        if (l.experts) {
+            if ((rc = lin("mlp.e0.gate", l.experts * 2 * l.expert_ff, D, &w.egu))) return rc;
+            if ((rc = lin("mlp.e0.down", l.experts * D, l.expert_ff, &w.ed))) return rc;
+            if ((rc = lin("mlp.router", l.experts + l.identity + (l.shared_ff > 0), D, &w.router))) return rc;
+            w.correction = W(x, lname(i, "mlp.correction"));
+            if (l.shared_ff) {
+                if ((rc = lin("mlp.shared.gate", 2 * l.shared_ff, D, &w.gu))) return rc;
+                if ((rc = lin("mlp.shared.down", D, l.shared_ff, &w.down))) return rc;
+            }
         }
     }
     LAUNCHCHK();
@@ -285,7 +381,8 @@ int ensure_workspace(pgmi_ctx* x, int rows, int chunks, int gchunks) {
     d.arena = nullptr;
     d.rows = d.chunks = d.gchunks = 0;
     const int D = d.c.width;
-    int l0 = 8, l1 = 8, l2 = 8, ldd = 8, slab_n = D, inner = 1, bcn = 2, cs = 1, cg = 1;
+    int l0 = r8(D), l1 = 8, l2 = 8, ldd = 8, slab_n = D, inner = 1, bcn = 2, cs = 1, cg = 1;
+    int lea = 8, top = 0, ne = 0;  // mixtures: expert activations, choices per row, experts
     for (const pgmi_layer_spec& l : d.L) {
         if (l.mixer == PGMI_MIXER_MAMBA1) {
             l0 = std::max(l0, 2 * r8(l.inner));
@@ -297,7 +394,7 @@ int ensure_workspace(pgmi_ctx* x, int rows, int chunks, int gchunks) {
             bcn = std::max(bcn, 2 * l.state);
             cs = std::max(cs, l.inner * l.state);
         } else if (l.mixer == PGMI_MIXER_ATTENTION) {
-            l0 = std::max(l0, r8(l.heads * l.dim + l.kv_heads * (l.dim + l.vdim)));
+            l0 = std::max(l0, r8(qkv_rows(l)));
             l1 = std::max(l1, l.heads * r8(l.dim));
             l2 = std::max(l2, r8(l.heads * l.vdim));
         } else {
@@ -305,20 +402,30 @@ int ensure_workspace(pgmi_ctx* x, int rows, int chunks, int gchunks) {
             l2 = std::max(l2, r8(l.width));
             cg = std::max(cg, l.width);
         }
-        if (l.ff) {
-            l2 = std::max(l2, r8(l.ff));
-            if (d.act == ACT_F32) l0 = std::max(l0, 2 * l.ff);  // unfused gate|up
+        if (const int ff = l.experts ? l.shared_ff : l.ff) {
+            l2 = std::max(l2, r8(ff));
+            if (d.act == ACT_F32) l0 = std::max(l0, 2 * ff);  // unfused gate|up
+        }
+        if (l.experts) {
+            lea = std::max(lea, r8(l.expert_ff));
+            top = std::max(top, l.top);
+            ne = std::max(ne, l.experts);
+            slab_n = std::max(slab_n, l.experts + l.identity + 1);
         }
     }
+    const size_t ent = (size_t)rows * top;
     d.ldh = r8(D);
     d.ld0 = l0; d.ld1 = l1; d.ld2 = l2; d.ldd = ldd;
     d.slab_bytes = std::max<size_t>((size_t)rows * slab_n * 4, (size_t)32 << 20);
     const size_t sizes[] = {(size_t)rows * d.c.streams * D * 4, (size_t)rows * d.ldh * d.es, (size_t)rows * l0 * d.es,
                             (size_t)rows * l1 * d.es,           (size_t)rows * l2 * d.es,    (size_t)rows * ldd * d.es,
                             d.slab_bytes,                       (size_t)rows * inner * 4,    (size_t)rows * bcn * 4,
-                            std::max((size_t)chunks * cs, (size_t)gchunks * 2 * cg) * 4, (size_t)chunks * inner * 4};
-    size_t off[11], total = 0;
-    for (int i = 0; i < 11; ++i) {
+                            std::max((size_t)chunks * cs, (size_t)gchunks * 2 * cg) * 4, (size_t)chunks * inner * 4,
+                            ent * lea * d.es, ent * d.ldh * d.es, ent * 4, ent * 4, (size_t)rows * 4, (size_t)rows * 4,
+                            (size_t)rows * ne * 4, (size_t)(2 * ne + 2) * 4};
+    constexpr int NB = sizeof(sizes) / sizeof(sizes[0]);
+    size_t off[NB], total = 0;
+    for (int i = 0; i < NB; ++i) {
         off[i] = total;
         total += (sizes[i] + 511) / 256 * 256;
     }
@@ -335,6 +442,14 @@ int ensure_workspace(pgmi_ctx* x, int rows, int chunks, int gchunks) {
     d.bc = reinterpret_cast<float*>(p + off[8]);
     d.cstate = reinterpret_cast<float*>(p + off[9]);
     d.csum = reinterpret_cast<float*>(p + off[10]);
+    d.ea = p + off[11]; d.ey = p + off[12];
+    d.esel = reinterpret_cast<int*>(p + off[13]);
+    d.ew = reinterpret_cast<float*>(p + off[14]);
+    d.egate = reinterpret_cast<float*>(p + off[15]);
+    d.inv = reinterpret_cast<float*>(p + off[16]);
+    d.elist = reinterpret_cast<int*>(p + off[17]);
+    d.ecnt = reinterpret_cast<int*>(p + off[18]);
+    d.eactive = d.ecnt + ne;
     d.rows = rows;
     d.chunks = chunks;
     d.gchunks = gchunks;
@@ -346,6 +461,7 @@ struct Pending {
     const float* y = nullptr;
     int split = 0;
     const Sub* sub = nullptr;
+    ExpertMix mix{};
 };
 
 StreamsArgs streams_args(const DecoderState& d, int rows) {
@@ -365,6 +481,54 @@ void fold(StreamsArgs& a, const Pending& p, int rows) {
 template <typename T>
 T* at(void* state, int64_t off) { return reinterpret_cast<T*>(reinterpret_cast<uint8_t*>(state) + off); }
 
+ResidualArgs residual_args(const DecoderState& d, int rows, const Pending& p, const uint16_t* norm) {
+    ResidualArgs a{};
+    a.X = d.X; a.rows = rows; a.D = d.c.width; a.E = d.embed; a.escale = d.c.embed_scale; a.vocab = d.c.vocab;
+    a.y = p.y; a.ysplit = p.split; a.ystride = (long)rows * a.D; a.mix = p.mix; a.mult = d.c.residual_mult;
+    a.w = norm; a.w_scalar = d.c.norm_scalar; a.eps = d.c.norm_eps; a.h = d.h; a.ldh = d.ldh;
+    return a;
+}
+
+// ids: the embedding makes X
+void residual_embed(ResidualArgs& a, const DecoderState& d, const int64_t* ids, void* state, const StateMap& st, int max_tokens) {
+    a.ids = ids;
+    if (!d.c.bigram_buckets) return;
+    a.pairs = d.pairs; a.mul_prev = d.c.bigram_mul_prev; a.mul_cur = d.c.bigram_mul_cur; a.buckets = d.c.bigram_buckets;
+    a.history = reinterpret_cast<int*>(reinterpret_cast<uint8_t*>(state) + st.history);
+    a.max_tokens = max_tokens;
+}
+
+WAttnHeads attn_heads(const DecoderState& d, const pgmi_layer_spec& l, const LayerW& w) {
+    return {l.heads, l.kv_heads, l.dim, l.vdim, r8(l.dim), r8(l.vdim), l.kv_from < 0, l.qk_norm != 0, l.v_norm != 0,
+            d.c.norm_eps, w.turns, l.rot_dims};
+}
+WAttnScore attn_score(const pgmi_layer_spec& l, const LayerW& w) {
+    return {l.window, l.keep_first, l.scale, l.softcap, w.r1, w.r2};
+}
+
+RouteArgs route_args(const DecoderState& d, const pgmi_layer_spec& l, const LayerW& w, int rows, int split) {
+    RouteArgs a{};
+    a.z = d.slabs; a.split = split; a.ldz = w.router.n; a.zstride = (long)rows * a.ldz; a.rows = rows;
+    a.n = l.experts + l.identity; a.experts = l.experts; a.top = l.top; a.groups = l.groups; a.keep = l.groups_keep;
+    a.correction = w.correction; a.sel = d.esel; a.w = d.ew; a.gate = l.shared_ff ? d.egate : nullptr;
+    a.cnt = d.ecnt; a.list = d.elist; a.cap = rows;
+    return a;
+}
+ExpertArgs expert_args(const DecoderState& d, const pgmi_layer_spec& l, const LayerW& w, int rows, ExpertMode mode) {
+    ExpertArgs a{};
+    const bool up = mode == EX_SWIGLU;
+    const Lin& lin = up ? w.egu : w.ed;
+    a.A = up ? d.h : d.ea; a.lda = up ? d.ldh : r8(l.expert_ff); a.gather = up ? l.top : 1;
+    a.W = lin.w; a.ldw = lin.ldw; a.K = lin.k; a.N = up ? l.expert_ff : d.c.width;
+    a.wstride = (long)(up ? 2 : 1) * a.N * lin.ldw;
+    a.out = up ? d.ea : d.ey; a.ldo = up ? r8(l.expert_ff) : d.ldh;
+    a.cnt = d.ecnt; a.list = d.elist; a.cap = rows; a.experts = l.experts; a.entries = rows * l.top;
+    return a;
+}
+ExpertMix expert_mix(const DecoderState& d, const pgmi_layer_spec& l) {
+    return {d.ey, d.ldh, d.esel, d.ew, l.top, l.experts, d.h, d.ldh, l.shared_ff ? d.egate : nullptr};
+}
+
 // device addresses of a step's metadata
 struct Meta {
     const SeqInfo* seqs;
@@ -383,11 +547,33 @@ int forward_body(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int rows, const
                  int max_tokens, int n_want, float* logits, float* taps) {
     DecoderState& d = *x->dec;
     const int D = d.c.width;
-    std::vector<StateAt> st;
-    state_layout(d, n_slots, max_tokens, &st);
+    const StateMap sm = state_layout(d, n_slots, max_tokens);
+    const std::vector<StateAt>& st = sm.at;
     Pending pend;
     bool first = true;
-    auto read = [&](const Sub& sub, float* tap) {
+    // the finished sublayer folded into the residual, and the input of sublayer q of layer i in d.h
+    auto read = [&](int i, int q, float* tap) {
+        const LayerW& w = d.W[i];
+        const Sub& sub = w.sub[q];
+        if (d.c.plain_residual) {
+            ResidualArgs a = residual_args(d, rows, pend, sub.norm);
+            const bool conv = q == 0 && d.c.canon_taps > 0;
+            if (first) residual_embed(a, d, ids, state, sm, max_tokens);
+            a.seqs = m.seqs; a.row_seq = m.row_seq; a.tap = tap;
+            if (conv) { a.h = nullptr; a.inv = d.inv; }
+            if (q == 1 && d.L[i].experts) { a.zero = d.ecnt; a.nzero = d.L[i].experts; }
+            residual_norm(s, d.act, a);
+            if (conv) {
+                CanonArgs c{};
+                c.X = d.X; c.inv = d.inv; c.w = sub.norm; c.w_scalar = d.c.norm_scalar; c.rows = rows; c.D = D;
+                c.taps = d.c.canon_taps; c.cw = w.canon; c.ring = at<float>(state, st[i].ring); c.h = d.h; c.ldh = d.ldh;
+                c.seqs = m.seqs; c.nseq = m.nseq; c.chunks = m.scan.p; c.nchunk = m.scan.n;
+                canon(s, d.act, c);
+            }
+            pend = {};
+            first = false;
+            return;
+        }
         StreamsArgs a = streams_args(d, rows);
         if (first) a.ids = ids;
         fold(a, pend, rows);
@@ -404,7 +590,7 @@ int forward_body(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int rows, const
     for (int i = 0; i < d.c.n_layers; ++i) {
         const pgmi_layer_spec& l = d.L[i];
         const LayerW& w = d.W[i];
-        read(w.sub[0], taps && i ? taps + (long)(i - 1) * rows * D : nullptr);
+        read(i, 0, taps && i ? taps + (long)(i - 1) * rows * D : nullptr);
         if (l.mixer == PGMI_MIXER_MAMBA1) {
             const int C = l.inner, N = l.state, R = l.dt_rank, ldc = r8(C), ldxz = r8(2 * C), ldd = r8(R);
             matmul_rt(s, d.act, d.h, d.ldh, w.in.w, w.in.ldw, rows, 2 * C, w.in.k, RT_ACT, nullptr, d.p0, ldxz, 0, nullptr);
@@ -423,12 +609,11 @@ int forward_body(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int rows, const
             out_proj(w.o, d.p2, ldc, w.sub[0]);
         } else if (l.mixer == PGMI_MIXER_ATTENTION) {
             WAttnArgs a{};
-            a.H = l.heads; a.G = l.kv_heads; a.d = l.dim; a.e = l.vdim; a.dp = r8(l.dim); a.ep = r8(l.vdim);
-            a.ldqkv = r8(w.in.n); a.ldo = r8(a.H * a.e);
+            a.hd = attn_heads(d, l, w); a.sc = attn_score(l, w);
+            a.ldqkv = r8(w.in.n); a.ldo = r8(l.heads * l.vdim);
             matmul_rt(s, d.act, d.h, d.ldh, w.in.w, w.in.ldw, rows, w.in.n, w.in.k, RT_ACT, w.bias, d.p0, a.ldqkv, 0, nullptr);
             a.qkv = d.p0; a.q = d.p1; a.kc = at<void>(state, st[i].a); a.vc = at<void>(state, st[i].b);
-            a.max_tokens = max_tokens; a.o = d.p2; a.rows = rows; a.window = l.window; a.scale = l.scale;
-            a.eps = d.c.norm_eps; a.r1 = w.r1; a.r2 = w.r2; a.seqs = m.seqs; a.nseq = m.nseq; a.row_seq = m.row_seq;
+            a.max_tokens = max_tokens; a.o = d.p2; a.rows = rows; a.seqs = m.seqs; a.nseq = m.nseq; a.row_seq = m.row_seq;
             const auto& t = m.tiles.at(l.heads / l.kv_heads);
             a.tiles = t.first; a.ntile = t.second;
             wattn_append(s, d.act, a);
@@ -443,14 +628,28 @@ int forward_body(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int rows, const
             mingru_scan(s, d.act, a);
             out_proj(w.o, d.p2, ldc, w.sub[0]);
         }
-        if (l.ff) {
-            read(w.sub[1], nullptr);
-            matmul_rt(s, d.act, d.h, d.ldh, w.gu.w, w.gu.ldw, rows, l.ff, w.gu.k, RT_SWIGLU, nullptr, d.p2, r8(l.ff), 0,
-                      reinterpret_cast<float*>(d.p0));
-            out_proj(w.down, d.p2, r8(l.ff), w.sub[1]);
+        if (has_ff(l)) read(i, 1, nullptr);
+        if (l.experts) {
+            const int sp = matmul_rt(s, d.act, d.h, d.ldh, w.router.w, w.router.ldw, rows, w.router.n, w.router.k, RT_SLABS,
+                                     nullptr, d.slabs, 0, d.slab_bytes, nullptr);
+            route(s, route_args(d, l, w, rows, sp));
+            experts_rt(s, d.act, EX_SWIGLU, expert_args(d, l, w, rows, EX_SWIGLU));
+            experts_rt(s, d.act, EX_STORE, expert_args(d, l, w, rows, EX_STORE));
         }
+        if (const int ff = l.experts ? l.shared_ff : l.ff) {
+            matmul_rt(s, d.act, d.h, d.ldh, w.gu.w, w.gu.ldw, rows, ff, w.gu.k, RT_SWIGLU, nullptr, d.p2, r8(ff), 0,
+                      reinterpret_cast<float*>(d.p0));
+            out_proj(w.down, d.p2, r8(ff), w.sub[1]);
+        }
+        if (l.experts) pend.mix = expert_mix(d, l);
     }
-    if (taps) {
+    if (taps && d.c.plain_residual) {
+        ResidualArgs a = residual_args(d, rows, pend, nullptr);
+        a.h = nullptr;
+        a.tap = taps + (long)(d.c.n_layers - 1) * rows * D;
+        residual_norm(s, d.act, a);
+        pend = {};
+    } else if (taps) {
         StreamsArgs a = streams_args(d, rows);
         fold(a, pend, rows);
         a.h = nullptr;
@@ -459,18 +658,26 @@ int forward_body(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int rows, const
         pend = {};
     }
     if (n_want > 0) {
-        StreamsArgs a = streams_args(d, n_want);
-        fold(a, pend, rows);
-        a.in = nullptr; a.w = d.fnorm; a.rows_idx = m.want;
-        streams_norm(s, d.act, a);
+        const void* h = d.h;
+        if (d.c.plain_residual) {
+            ResidualArgs a = residual_args(d, rows, pend, d.fnorm);
+            a.rows = n_want; a.rows_idx = m.want;
+            h = a.h = d.p0;  // other rows' d.h is still read (identity experts)
+            residual_norm(s, d.act, a);
+        } else {
+            StreamsArgs a = streams_args(d, n_want);
+            fold(a, pend, rows);
+            a.in = nullptr; a.w = d.fnorm; a.rows_idx = m.want;
+            streams_norm(s, d.act, a);
+        }
         const GemvRtForm form = gemv_rt_form(n_want, d.act, 1, 1);
         if (gemv_rt_fits(form, d.head.k, d.act)) {
             GemvRtArgs g{};
-            g.form = form; g.B = n_want; g.N = d.c.vocab; g.K = d.head.k; g.W = d.head.w; g.ldw = d.head.ldw; g.x = d.h; g.ldx = d.ldh;
+            g.form = form; g.B = n_want; g.N = d.c.vocab; g.K = d.head.k; g.W = d.head.w; g.ldw = d.head.ldw; g.x = h; g.ldx = d.ldh;
             g.out = logits; g.ldo = d.c.vocab;
             gemv_rt(s, d.act, GR_F32, g);
         } else {
-            matmul_rt(s, d.act, d.h, d.ldh, d.head.w, d.head.ldw, n_want, d.c.vocab, d.head.k, RT_F32, nullptr, logits,
+            matmul_rt(s, d.act, h, d.ldh, d.head.w, d.head.ldw, n_want, d.c.vocab, d.head.k, RT_F32, nullptr, logits,
                       d.c.vocab, 0, nullptr);
         }
     }
@@ -482,16 +689,34 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
                    float* logits, int64_t* next, int64_t* hist) {
     DecoderState& d = *x->dec;
     const int D = d.c.width, V = d.c.vocab;
-    std::vector<StateAt> st;
-    state_layout(d, n_slots, max_tokens, &st);
-    {   // the embedding rows into every stream, and the first sublayer's input
+    const StateMap sm = state_layout(d, n_slots, max_tokens);
+    const std::vector<StateAt>& st = sm.at;
+    const bool plain = d.c.plain_residual;
+    if (!plain) {  // the embedding rows into every stream, and the first sublayer's input
         StreamsArgs a = streams_args(d, B);
         a.ids = ids; a.in = d.W[0].sub[0].in; a.w = d.W[0].sub[0].norm;
         streams_norm(s, d.act, a);
     }
     const GemvRtForm form = gemv_rt_form(B, d.act, d.c.streams, D);
-    bool have_h = true;  // d.h holds the coming sublayer's input
+    bool have_h = !plain;  // d.h holds the coming sublayer's input
+    bool first = true;     // plain residual: X is not made yet
     Pending pend;
+    // plain residual: the finished sublayer folded in and the input of sublayer q of layer i (the end: i = n_layers) in d.h
+    auto read = [&](int i, int q) {
+        if (!plain) return;
+        const bool end = i == d.c.n_layers;
+        ResidualArgs a = residual_args(d, B, pend, end ? d.fnorm : d.W[i].sub[q].norm);
+        if (first) residual_embed(a, d, ids, state, sm, max_tokens);
+        a.slot = d.slot; a.pos = d.pos;
+        if (!end && q == 0 && d.c.canon_taps > 0) {
+            a.taps = d.c.canon_taps; a.cw = d.W[i].canon; a.ring = at<float>(state, st[i].ring);
+        }
+        if (!end && q == 1 && d.L[i].experts) { a.zero = d.ecnt; a.nzero = d.L[i].experts; }
+        residual_norm(s, d.act, a);
+        pend = {};
+        first = false;
+        have_h = true;
+    };
     // the input side of a projection: d.h, or (fused) the streams' read and norm inside the GEMV
     auto base = [&](const Sub& sub, const Lin& w, bool fused) {
         if (!have_h && (!fused || pend.y || form != GF_STREAM)) {
@@ -520,10 +745,10 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
             GemvRtArgs g = row_in(o, in, ldin);
             g.out = d.slabs; g.ldo = D; g.split = gemv_rt_split(form, D, o.k);
             gemv_rt(s, d.act, GR_F32, g);
-            pend = {d.slabs, g.split, &sub};
+            pend = {d.slabs, g.split, &sub, {}};
         } else if (fits) {
             GemvRtArgs g = row_in(o, in, ldin);
-            g.X = d.X; g.S = d.c.streams; g.D = D; g.mix = sub.mix; g.wout = sub.out;
+            g.X = d.X; g.S = d.c.streams; g.D = D; g.mix = sub.mix; g.wout = sub.out; g.mult = d.c.residual_mult;
             gemv_rt(s, d.act, GR_STREAMS, g);
         } else {
             pend.split = matmul_rt(s, d.act, in, ldin, o.w, o.ldw, B, D, o.k, RT_SLABS, nullptr, d.slabs, D, d.slab_bytes, nullptr);
@@ -535,6 +760,7 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
         const pgmi_layer_spec& l = d.L[i];
         const LayerW& w = d.W[i];
         const bool fin = gemv_rt_fits(form, w.in.k, d.act);
+        read(i, 0);
         if (l.mixer == PGMI_MIXER_MAMBA1) {
             const int C = l.inner, N = l.state, R = l.dt_rank, ldc = r8(C);
             float* taps = at<float>(state, st[i].a);
@@ -568,8 +794,8 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
             out_proj(w.o, d.p2, ldc, w.sub[0]);
         } else if (l.mixer == PGMI_MIXER_ATTENTION) {
             WAttnDecodeArgs a{};
-            a.H = l.heads; a.G = l.kv_heads; a.d = l.dim; a.e = l.vdim; a.dp = r8(l.dim); a.ep = r8(l.vdim);
-            a.ldqkv = r8(w.in.n); a.ldo = r8(a.H * a.e);
+            a.hd = attn_heads(d, l, w); a.sc = attn_score(l, w);
+            a.ldqkv = r8(w.in.n); a.ldo = r8(l.heads * l.vdim);
             GemvRtArgs g = base(w.sub[0], w.in, fin);
             if (fin) {
                 g.out = d.p0; g.ldo = a.ldqkv; g.bias = w.bias;
@@ -578,8 +804,8 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
                 matmul_rt(s, d.act, d.h, d.ldh, w.in.w, w.in.ldw, B, w.in.n, w.in.k, RT_ACT, w.bias, d.p0, a.ldqkv, 0, nullptr);
             }
             a.qkv = d.p0; a.kc = at<void>(state, st[i].a); a.vc = at<void>(state, st[i].b); a.max_tokens = max_tokens;
-            a.o = d.p2; a.B = B; a.window = l.window; a.scale = l.scale; a.eps = d.c.norm_eps; a.r1 = w.r1; a.r2 = w.r2;
-            a.slot = d.slot; a.pos = d.pos; a.part = d.part; a.nsplit = wattn_decode_splits(B, a.G, a.window, max_tokens);
+            a.o = d.p2; a.B = B; a.slot = d.slot; a.pos = d.pos; a.part = d.part;
+            a.nsplit = wattn_decode_splits(B, l.kv_heads, a.sc, max_tokens);
             wattn_decode(s, d.act, a);
             out_proj(w.o, d.p2, a.ldo, w.sub[0]);
         } else {
@@ -594,19 +820,64 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
             }
             out_proj(w.o, d.p2, ldc, w.sub[0]);
         }
-        if (l.ff) {
+        if (has_ff(l)) read(i, 1);
+        bool shared_done = false;
+        if (l.experts) {
+            const bool fr = gemv_rt_fits(form, w.router.k, d.act);
+            GemvRtArgs g = base(w.sub[1], w.router, fr);
+            int sp;
+            if (fr) {
+                g.out = d.slabs; g.ldo = w.router.n; sp = g.split = gemv_rt_split(form, w.router.n, w.router.k);
+                gemv_rt(s, d.act, GR_F32, g);
+            } else {
+                sp = matmul_rt(s, d.act, d.h, d.ldh, w.router.w, w.router.ldw, B, w.router.n, w.router.k, RT_SLABS, nullptr,
+                               d.slabs, 0, d.slab_bytes, nullptr);
+            }
+            RouteArgs r = route_args(d, l, w, B, sp);
+            ExpertArgs up = expert_args(d, l, w, B, EX_SWIGLU), down = expert_args(d, l, w, B, EX_STORE);
+            if (d.act == ACT_BF16 && B <= kRouteRows) {  // the shared expert rides along
+                r.active = d.eactive;
+                up.active = down.active = d.eactive;
+                route(s, r);
+                up.B = down.B = B;
+                if (l.shared_ff) {
+                    up.Wsh = w.gu.w; up.ldwsh = w.gu.ldw; up.Nsh = l.shared_ff; up.Ksh = w.gu.k; up.Ash = d.h; up.ldash = d.ldh;
+                    up.outsh = d.p2; up.ldosh = r8(l.shared_ff);
+                    down.Wsh = w.down.w; down.ldwsh = w.down.ldw; down.Nsh = D; down.Ksh = w.down.k; down.Ash = d.p2;
+                    down.ldash = r8(l.shared_ff); down.outsh = d.slabs; down.ldosh = D;
+                }
+                experts_skinny(s, EX_SWIGLU, up);
+                experts_skinny(s, EX_STORE, down);
+                if (l.shared_ff) pend = {d.slabs, 1, &w.sub[1], {}};
+                shared_done = true;
+            } else {
+                route(s, r);
+                experts_rt(s, d.act, EX_SWIGLU, up);
+                experts_rt(s, d.act, EX_STORE, down);
+            }
+        }
+        if (const int ff = l.experts ? l.shared_ff : l.ff; ff && !shared_done) {
             const bool fgu = gemv_rt_fits(form, w.gu.k, d.act);
+            if (l.experts) have_h = true;  // the mixture's input, once more
             GemvRtArgs g = base(w.sub[1], w.gu, fgu);
             if (fgu) {
-                g.N = l.ff; g.out = d.p2; g.ldo = r8(l.ff);
+                g.N = ff; g.out = d.p2; g.ldo = r8(ff);
                 gemv_rt(s, d.act, GR_SWIGLU, g);
             } else {
-                matmul_rt(s, d.act, d.h, d.ldh, w.gu.w, w.gu.ldw, B, l.ff, w.gu.k, RT_SWIGLU, nullptr, d.p2, r8(l.ff), 0,
+                matmul_rt(s, d.act, d.h, d.ldh, w.gu.w, w.gu.ldw, B, ff, w.gu.k, RT_SWIGLU, nullptr, d.p2, r8(ff), 0,
                           reinterpret_cast<float*>(d.p0));
             }
-            out_proj(w.down, d.p2, r8(l.ff), w.sub[1]);
+            if (l.experts) {  // the next residual pass scales it by its gate
+                pend.split = matmul_rt(s, d.act, d.p2, r8(ff), w.down.w, w.down.ldw, B, D, w.down.k, RT_SLABS, nullptr, d.slabs, D,
+                                       d.slab_bytes, nullptr);
+                pend.y = d.slabs;
+            } else {
+                out_proj(w.down, d.p2, r8(ff), w.sub[1]);
+            }
         }
+        if (l.experts) pend.mix = expert_mix(d, l);
     }
+    read(d.c.n_layers, 0);
     const Sub fin{nullptr, nullptr, nullptr, d.fnorm};
     const bool fl = gemv_rt_fits(form, d.head.k, d.act);
     GemvRtArgs g = base(fin, d.head, fl);
@@ -652,6 +923,14 @@ int pgmi_decoder_create(int device, const pgmi_decoder_config* cfg, const pgmi_l
     if (c.vocab < 1 || c.width < 1 || c.n_layers < 1) return fail(PGMI_E_ARG, "vocab, width and layers must be positive");
     if (c.streams < 1 || c.streams > 8) return fail(PGMI_E_ARG, "streams must be in [1, 8]");
     if (c.norm_groups < 1 || c.width % c.norm_groups != 0) return fail(PGMI_E_ARG, "norm groups must divide the width");
+    if (c.plain_residual && (c.streams != 1 || c.norm_groups != 1))
+        return fail(PGMI_E_ARG, "a plain residual has one stream and one norm group");
+    if (!c.plain_residual && (c.norm_scalar || c.canon_taps || c.bigram_buckets))
+        return fail(PGMI_E_ARG, "scalar norms, the input convolution and token pairs go with a plain residual");
+    if (c.canon_taps < 0 || c.bigram_buckets < 0) return fail(PGMI_E_ARG, "negative taps or buckets");
+    if (c.bigram_buckets && (c.bigram_mul_prev < 0 || c.bigram_mul_cur < 0 || c.bigram_mul_prev >= c.bigram_buckets ||
+                             c.bigram_mul_cur >= c.bigram_buckets))
+        return fail(PGMI_E_ARG, "token pair factors must be reduced modulo the buckets");
     if (c.width > 16384) return fail(PGMI_E_ARG, "width must be at most 16384");
     if (c.max_batch < 1) return fail(PGMI_E_ARG, "max_batch must be positive");
     if (c.act_dtype != PGMI_DTYPE_BF16 && c.act_dtype != PGMI_DTYPE_F32)
@@ -668,10 +947,35 @@ int pgmi_decoder_create(int device, const pgmi_decoder_config* cfg, const pgmi_l
                 return fail(PGMI_E_ARG, at + "attention sizes must be positive");
             if (l.heads % l.kv_heads != 0) return fail(PGMI_E_ARG, at + "kv_heads must divide heads");
             if (l.dim > 512 || l.vdim > 2048) return fail(PGMI_E_ARG, at + "head sizes are at most 512 (query / key) and 2048 (value)");
+            if (l.keep_first < 0) return fail(PGMI_E_ARG, at + "negative number of kept tokens");
+            if (l.softcap < 0 || (l.softcap > 0 && l.distance_bias))
+                return fail(PGMI_E_ARG, at + "the score cap must be positive, and goes without a distance bias");
+            if (l.rot_dims < 0 || l.rot_dims % 2 != 0 || l.rot_dims > l.dim || (l.rot_dims > 0 && !(l.rot_base > 0)))
+                return fail(PGMI_E_ARG, at + "rotated dims must be even and inside the head, with a positive base");
+            if (l.rot_original > 0 && !(l.rot_factor > 0 && l.rot_low > 0 && l.rot_high > l.rot_low))
+                return fail(PGMI_E_ARG, at + "rotary scaling needs a factor and 0 < low < high");
+            if (l.kv_from >= i) return fail(PGMI_E_ARG, at + "keys and values come from an earlier layer");
+            if (l.kv_from >= 0) {
+                const pgmi_layer_spec& k = layers[l.kv_from];
+                if (k.mixer != PGMI_MIXER_ATTENTION || k.kv_from >= 0 || k.kv_heads != l.kv_heads || k.dim != l.dim || k.vdim != l.vdim)
+                    return fail(PGMI_E_ARG, at + "keys and values come from an attention layer with its own, of equal sizes");
+            }
         } else if (l.mixer == PGMI_MIXER_MINGRU) {
             if (l.width < 1) return fail(PGMI_E_ARG, at + "mingru width must be positive");
         } else {
             return fail(PGMI_E_ARG, at + "unknown mixer");
+        }
+        if (l.experts < 0 || l.identity < 0 || l.shared_ff < 0) return fail(PGMI_E_ARG, at + "negative expert sizes");
+        if (l.experts) {
+            const int n = l.experts + l.identity;
+            if (!c.plain_residual) return fail(PGMI_E_ARG, at + "a mixture of experts goes with a plain residual");
+            if (l.ff) return fail(PGMI_E_ARG, at + "a feed-forward is gated or a mixture of experts");
+            if (n > kMaxExperts) return fail(PGMI_E_ARG, at + "at most " + std::to_string(kMaxExperts) + " experts");
+            if (l.expert_ff < 1) return fail(PGMI_E_ARG, at + "expert size must be positive");
+            if (l.groups < 1 || n % l.groups != 0 || l.groups_keep < 1 || l.groups_keep > l.groups)
+                return fail(PGMI_E_ARG, at + "groups must divide the experts, and some of them be kept");
+            if (l.top < 1 || l.top > n / l.groups * l.groups_keep)
+                return fail(PGMI_E_ARG, at + "more experts per token than the kept groups hold");
         }
     }
     auto* x = new pgmi_ctx();
@@ -788,7 +1092,7 @@ int pgmi_decoder_decode(pgmi_ctx* x, const int64_t* ids, int B, const int32_t* s
     size_t need = 0;
     for (const pgmi_layer_spec& l : d.L)
         if (l.mixer == PGMI_MIXER_ATTENTION)
-            need = std::max(need, wattn_decode_floats(B, l.heads, r8(l.vdim), wattn_decode_splits(B, l.kv_heads, l.window, max_tokens)));
+            need = std::max(need, wattn_decode_floats(B, l.heads, r8(l.vdim), wattn_decode_splits(B, l.kv_heads, attn_score(l, {}), max_tokens)));
     if (need > d.part_floats) {
         HIPCHK(hipDeviceSynchronize());
         clear_dgraphs(x);

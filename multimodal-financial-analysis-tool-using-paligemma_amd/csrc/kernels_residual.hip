@@ -1,0 +1,306 @@
+// kernels_residual.hip -- one residual stream: the embedding (with a table of token pairs), the scaled update from a
+// finished sublayer (split-K slabs, a mixture's outputs), the RMS norm in front of the next one, and the causal input
+// convolution added to what a mixer reads.  Stream, sums, norms and the convolution are fp32.
+#include <algorithm>
+
+#include "act.h"
+#include "decoder.h"
+
+namespace pgmi {
+
+namespace {
+
+__device__ __forceinline__ void ldv(const float* p, float (&v)[4]) { ld4(p, v); }
+__device__ __forceinline__ void ldv(const uint16_t* p, float (&v)[4]) { ld4(p, v); }
+template <typename S>
+__device__ __forceinline__ void ldv(const S* p, float (&v)[1]) { v[0] = ldf(p); }
+template <typename S>
+__device__ __forceinline__ void stv(S* p, const float (&v)[4]) { st4(p, v); }
+template <typename S>
+__device__ __forceinline__ void stv(S* p, const float (&v)[1]) { stf(p, v[0]); }
+
+// One workgroup per row; PC pieces of V elements per thread, every load of a source issued before its first use.
+template <typename T, int V, int PC>
+__global__ void __launch_bounds__(1024) k_residual(ResidualArgs a) {
+    __shared__ float red[16];
+    const int tid = threadIdx.x, NT = blockDim.x, D = a.D;
+    const int row = a.rows_idx ? a.rows_idx[blockIdx.x] : blockIdx.x;
+    if (a.zero && blockIdx.x == 0)
+        for (int i = tid; i < a.nzero; i += NT) a.zero[i] = 0;
+    float* Xr = a.X + (long)row * D;
+    float x[PC][V];
+    int dd[PC];
+    bool ok[PC];
+#pragma unroll
+    for (int i = 0; i < PC; ++i) {
+        const int d = (i * NT + tid) * V;
+        ok[i] = d < D;
+        dd[i] = ok[i] ? d : 0;
+    }
+    int slot = 0, pos = 0;
+    if (a.ids) {
+        long id = a.ids[row];
+        id = id < 0 ? 0 : (id >= a.vocab ? a.vocab - 1 : id);
+        const uint16_t* er = a.E + id * D;
+#pragma unroll
+        for (int i = 0; i < PC; ++i) {
+            ldv(er + dd[i], x[i]);
+#pragma unroll
+            for (int v = 0; v < V; ++v) x[i][v] *= a.escale;
+        }
+        if (a.pairs) {
+            bool here = false;  // the previous token is the row before this one
+            if (a.seqs) {
+                const SeqInfo q = a.seqs[a.row_seq[row]];
+                slot = q.slot;
+                pos = q.start + row - q.off;
+                here = row > q.off;
+            } else {
+                slot = a.slot[row];
+                pos = a.pos[row];
+            }
+            int* hist = a.history + (long)slot * a.max_tokens + pos;
+            long p = a.buckets;
+            if (pos > 0) {
+                long prev = here ? a.ids[row - 1] : hist[-1];
+                prev = prev < 0 ? 0 : (prev >= a.vocab ? a.vocab - 1 : prev);
+                p = (prev * a.mul_prev + id * a.mul_cur) % a.buckets;
+            }
+            if (tid == 0) *hist = (int)id;
+            const uint16_t* pr = a.pairs + p * D;
+#pragma unroll
+            for (int i = 0; i < PC; ++i) {
+                float q[V];
+                ldv(pr + dd[i], q);
+#pragma unroll
+                for (int v = 0; v < V; ++v) x[i][v] += q[v];
+            }
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < PC; ++i) ldv(Xr + dd[i], x[i]);
+    }
+    if (a.y || a.mix.y) {
+        float y[PC][V];
+#pragma unroll
+        for (int i = 0; i < PC; ++i)
+#pragma unroll
+            for (int v = 0; v < V; ++v) y[i][v] = 0.0f;
+        if (a.y) {
+#pragma unroll 4
+            for (int z = 0; z < a.ysplit; ++z) {
+                const float* yr = a.y + (long)z * a.ystride + (long)row * D;
+#pragma unroll
+                for (int i = 0; i < PC; ++i) {
+                    float q[V];
+                    ldv(yr + dd[i], q);
+#pragma unroll
+                    for (int v = 0; v < V; ++v) y[i][v] += q[v];
+                }
+            }
+        }
+        if (a.mix.y) {
+            const ExpertMix& m = a.mix;
+            if (m.gate) {
+                const float g = m.gate[row];
+#pragma unroll
+                for (int i = 0; i < PC; ++i)
+#pragma unroll
+                    for (int v = 0; v < V; ++v) y[i][v] *= g;
+            }
+            const T* hr = reinterpret_cast<const T*>(m.h) + (long)row * m.ldh;
+#pragma unroll 4
+            for (int k = 0; k < m.top; ++k) {
+                const long e = (long)row * m.top + k;
+                const T* yr = m.sel[e] < m.experts ? reinterpret_cast<const T*>(m.y) + e * m.ldy : hr;
+                const float w = m.w[e];
+#pragma unroll
+                for (int i = 0; i < PC; ++i) {
+                    float q[V];
+                    ldv(yr + dd[i], q);
+#pragma unroll
+                    for (int v = 0; v < V; ++v) y[i][v] = fmaf(w, q[v], y[i][v]);
+                }
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < PC; ++i)
+#pragma unroll
+            for (int v = 0; v < V; ++v) x[i][v] = fmaf(a.mult, y[i][v], x[i][v]);
+    }
+    float ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < PC; ++i) {
+        if (!ok[i]) continue;
+#pragma unroll
+        for (int v = 0; v < V; ++v) ss = fmaf(x[i][v], x[i][v], ss);
+        if (!a.rows_idx && (a.ids || a.y || a.mix.y)) stv(Xr + dd[i], x[i]);
+        if (a.tap) stv(a.tap + (long)row * D + dd[i], x[i]);
+    }
+    if (!a.h && !a.inv) return;
+    ss = wave_sum(ss);
+    if ((tid & 63) == 0) red[tid >> 6] = ss;
+    __syncthreads();
+    ss = 0.0f;
+    for (int w = 0; w < NT / 64; ++w) ss += red[w];
+    const float inv = 1.0f / sqrtf(ss / (float)D + a.eps);
+    if (a.inv && tid == 0) a.inv[row] = inv;
+    if (!a.h) return;
+    T* h = reinterpret_cast<T*>(a.h) + (long)blockIdx.x * a.ldh;
+    const float g = a.w_scalar ? bf2f(a.w[0]) : 0.0f;
+    float* ring = nullptr;
+    if (a.taps > 0) {
+        slot = a.slot[row];
+        pos = a.pos[row];
+        ring = a.ring + (long)slot * a.taps * D;
+    }
+#pragma unroll
+    for (int i = 0; i < PC; ++i) {
+        if (!ok[i]) continue;
+        float n[V], o[V];
+#pragma unroll
+        for (int v = 0; v < V; ++v) o[v] = n[v] = x[i][v] * inv * (a.w_scalar ? g : bf2f(a.w[dd[i] + v]));
+        if (a.taps > 0) {
+            const uint16_t* cw = a.cw + (long)dd[i] * a.taps;
+            for (int j = 0; j < a.taps && j <= pos; ++j) {
+                float q[V];
+                if (j > 0) {
+                    ldv(ring + (long)((pos - j) % a.taps) * D + dd[i], q);
+                } else {
+#pragma unroll
+                    for (int v = 0; v < V; ++v) q[v] = n[v];
+                }
+#pragma unroll
+                for (int v = 0; v < V; ++v) o[v] = fmaf(bf2f(cw[v * a.taps + a.taps - 1 - j]), q[v], o[v]);
+            }
+            stv(ring + (long)(pos % a.taps) * D + dd[i], n);
+        }
+        stv(h + dd[i], o);
+    }
+    for (int d = D + tid; d < a.ldh; d += NT) stf(h + d, 0.0f);
+}
+
+template <typename T>
+void residual_t(hipStream_t s, const ResidualArgs& a) {
+    auto go = [&](auto kern, int v) {
+        const int threads = std::min(1024, (a.D / v + 63) / 64 * 64);
+        hipLaunchKernelGGL(kern, dim3(a.rows), dim3(std::max(64, threads)), 0, s, a);
+    };
+    if (a.D % 4 == 0 && a.D <= 4096) go(k_residual<T, 4, 1>, 4);
+    else if (a.D % 4 == 0) go(k_residual<T, 4, 4>, 4);
+    else if (a.D <= 1024) go(k_residual<T, 1, 1>, 1);
+    else go(k_residual<T, 1, 16>, 1);
+}
+
+// ---------------------------------------------------------------- input convolution
+// the norm's output at the sequence's relative row p (p < 0: an earlier step's, from the ring)
+__device__ __forceinline__ float canon_at(const CanonArgs& a, const SeqInfo& q, int p, int c) {
+    if (p >= 0) return a.X[(long)(q.off + p) * a.D + c] * a.inv[q.off + p] * bf2f(a.w[a.w_scalar ? 0 : c]);
+    p += q.start;
+    return p >= 0 ? a.ring[((long)q.slot * a.taps + p % a.taps) * a.D + c] : 0.0f;
+}
+
+// four channels per lane, KT taps in registers, each wave a run of consecutive rows
+template <typename T, int KT>
+__global__ void __launch_bounds__(256) k_canon(CanonArgs a) {
+    const ChunkInfo ck = a.chunks[blockIdx.y];
+    const SeqInfo q = a.seqs[ck.seq];
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int run = (ck.len + 3) / 4, r0 = wave * run, r1 = min(ck.len, r0 + run);
+    const int c = (blockIdx.x * 64 + lane) * 4;
+    if (c >= a.D || r0 >= r1) return;
+    float wk[KT][4], g[4], win[KT][4];
+#pragma unroll
+    for (int v = 0; v < 4; ++v) {
+        g[v] = bf2f(a.w[a.w_scalar ? 0 : c + v]);
+#pragma unroll
+        for (int t = 0; t < KT; ++t) wk[t][v] = bf2f(a.cw[(long)(c + v) * KT + t]);
+    }
+    auto take = [&](int row, float (&n)[4]) {
+        const float inv = a.inv[row];
+        ld4(a.X + (long)row * a.D + c, n);
+#pragma unroll
+        for (int v = 0; v < 4; ++v) n[v] = n[v] * inv * g[v];
+    };
+#pragma unroll
+    for (int t = 0; t < KT - 1; ++t) {
+        const int p = ck.rel + r0 - (KT - 1) + t;
+        if (p >= 0) {
+            take(q.off + p, win[t]);
+        } else {
+#pragma unroll
+            for (int v = 0; v < 4; ++v) win[t][v] = canon_at(a, q, p, c + v);
+        }
+    }
+    T* h = reinterpret_cast<T*>(a.h);
+#pragma unroll 4
+    for (int r = r0; r < r1; ++r) {
+        take(ck.row + r, win[KT - 1]);
+        float y[4];
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            y[v] = win[KT - 1][v];
+#pragma unroll
+            for (int t = KT - 1; t >= 0; --t) y[v] = fmaf(wk[t][v], win[t][v], y[v]);
+#pragma unroll
+            for (int t = 0; t + 1 < KT; ++t) win[t][v] = win[t + 1][v];
+        }
+        st4(h + (long)(ck.row + r) * a.ldh + c, y);
+        if (c + 4 == a.D)
+            for (int d = a.D; d < a.ldh; ++d) stf(h + (long)(ck.row + r) * a.ldh + d, 0.0f);
+    }
+}
+
+// any number of taps and channels
+template <typename T>
+__global__ void __launch_bounds__(256) k_canon_any(CanonArgs a) {
+    const ChunkInfo ck = a.chunks[blockIdx.y];
+    const SeqInfo q = a.seqs[ck.seq];
+    const int c = blockIdx.x * 64 + (threadIdx.x & 63);
+    if (c >= a.ldh) return;
+    T* h = reinterpret_cast<T*>(a.h);
+    for (int r = threadIdx.x >> 6; r < ck.len; r += 4) {
+        float y = 0.0f;
+        if (c < a.D) {
+            y = canon_at(a, q, ck.rel + r, c);
+            for (int t = a.taps - 1; t >= 0; --t)
+                y = fmaf(bf2f(a.cw[(long)c * a.taps + t]), canon_at(a, q, ck.rel + r - (a.taps - 1) + t, c), y);
+        }
+        stf(h + (long)(ck.row + r) * a.ldh + c, y);
+    }
+}
+
+// the sequences' last taps - 1 rows of this step into the ring
+__global__ void __launch_bounds__(256) k_canon_keep(CanonArgs a) {
+    const int n = a.taps - 1;
+    const SeqInfo q = a.seqs[blockIdx.y / n];
+    const int c = blockIdx.x * 256 + threadIdx.x, p = q.len - 1 - (int)(blockIdx.y % n);
+    if (c >= a.D || p < 0) return;
+    a.ring[((long)q.slot * a.taps + (q.start + p) % a.taps) * a.D + c] = canon_at(a, q, p, c);
+}
+
+template <typename T>
+void canon_t(hipStream_t s, const CanonArgs& a) {
+    const dim3 grid((a.D + 255) / 256, a.nchunk);
+    if (a.D % 4 == 0 && a.taps == 4) hipLaunchKernelGGL((k_canon<T, 4>), grid, dim3(256), 0, s, a);
+    else if (a.D % 4 == 0 && a.taps == 3) hipLaunchKernelGGL((k_canon<T, 3>), grid, dim3(256), 0, s, a);
+    else if (a.D % 4 == 0 && a.taps == 2) hipLaunchKernelGGL((k_canon<T, 2>), grid, dim3(256), 0, s, a);
+    else hipLaunchKernelGGL((k_canon_any<T>), dim3((a.ldh + 63) / 64, a.nchunk), dim3(256), 0, s, a);
+    if (a.taps > 1)
+        hipLaunchKernelGGL(k_canon_keep, dim3((a.D + 255) / 256, a.nseq * (a.taps - 1)), dim3(256), 0, s, a);
+}
+
+}  // namespace
+
+void residual_norm(hipStream_t s, Act act, const ResidualArgs& a) {
+    if (a.rows <= 0) return;
+    if (act == ACT_F32) residual_t<float>(s, a);
+    else residual_t<uint16_t>(s, a);
+}
+
+void canon(hipStream_t s, Act act, const CanonArgs& a) {
+    if (act == ACT_F32) canon_t<float>(s, a);
+    else canon_t<uint16_t>(s, a);
+}
+
+}  // namespace pgmi

@@ -74,6 +74,10 @@ __device__ __forceinline__ void step_epilogue(const GemvRtArgs& a, int n, int b,
         stf(reinterpret_cast<T*>(a.out) + (long)b * a.ldo + n, siluf_(v) * v1);
     } else {  // GR_STREAMS: the whole column of streams at once
         float* Xr = a.X + (long)b * a.S * a.D + n;
+        if (!a.mix) {
+            *Xr = fmaf(a.mult, v, *Xr);
+            return;
+        }
         float x[8];
 #pragma unroll
         for (int s = 0; s < 8; ++s) x[s] = s < a.S ? Xr[(long)s * a.D] : 0.0f;

@@ -39,14 +39,22 @@ class PgmiConfig(ctypes.Structure):
 
 
 class LayerSpec(ctypes.Structure):
-    _fields_ = [(n, ctypes.c_int) for n in ("mixer", "conv", "dt_rank", "inner", "state", "width", "heads", "kv_heads",
-                                            "dim", "vdim", "window")] + [("scale", ctypes.c_float), ("ff", ctypes.c_int)]
+    _fields_ = ([(n, ctypes.c_int) for n in ("mixer", "conv", "dt_rank", "inner", "state", "width", "heads", "kv_heads",
+                                             "dim", "vdim", "window")] + [("scale", ctypes.c_float), ("ff", ctypes.c_int)] +
+                [(n, ctypes.c_int) for n in ("qk_norm", "v_norm", "proj_bias", "distance_bias", "keep_first", "kv_from")] +
+                [("softcap", ctypes.c_float), ("rot_dims", ctypes.c_int)] +
+                [(n, ctypes.c_double) for n in ("rot_base", "rot_factor", "rot_low", "rot_high", "rot_original")] +
+                [(n, ctypes.c_int) for n in ("experts", "identity", "top", "groups", "groups_keep", "expert_ff",
+                                             "shared_ff")])
 
 
 class DecoderConfigC(ctypes.Structure):
     _fields_ = [("vocab", ctypes.c_int), ("width", ctypes.c_int), ("streams", ctypes.c_int), ("norm_groups", ctypes.c_int),
                 ("n_layers", ctypes.c_int), ("norm_eps", ctypes.c_float), ("embed_scale", ctypes.c_float),
-                ("max_batch", ctypes.c_int), ("act_dtype", ctypes.c_int)]
+                ("max_batch", ctypes.c_int), ("act_dtype", ctypes.c_int), ("plain_residual", ctypes.c_int),
+                ("residual_mult", ctypes.c_float), ("norm_scalar", ctypes.c_int), ("canon_taps", ctypes.c_int),
+                ("bigram_buckets", ctypes.c_int), ("bigram_mul_prev", ctypes.c_int64), ("bigram_mul_cur", ctypes.c_int64),
+                ("untied_head", ctypes.c_int)]
 
 
 vp, i32, i64, f32, u64 = ctypes.c_void_p, ctypes.c_int, ctypes.c_int64, ctypes.c_float, ctypes.c_uint64

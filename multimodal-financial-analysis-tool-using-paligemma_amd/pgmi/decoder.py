@@ -1,9 +1,9 @@
-"""Layered decoders: text models described by a list of layers (a mixer each, optionally a gated feed-forward)
-around residual streams, run by libpgmi's decoder engine (pgmi_decoder_* in include/pgmi.h).
+"""Layered decoders: text models described by a list of layers (a mixer each, optionally a gated feed-forward or a
+mixture of experts) around residual streams or one plain residual, run by libpgmi's decoder engine (pgmi_decoder_* in include/pgmi.h).
 
 DecoderConfig is the family's configuration; a design's config.json is turned into one by its reader in
 pgmi/registry.py.  DecoderEngine owns the context and weights, StateCache the per-sequence state of up to
-`slots` sequences (key / value rows, scan and recurrent states, convolution taps), step() runs the next tokens
+`slots` sequences (key / value rows, scan and recurrent states, convolution taps, token ids), step() runs the next tokens
 of any set of sequences -- whole prompts, portions, single tokens, of unequal lengths, in one batch -- and
 generate() decodes a batch of prompts with the token picking every engine shares.
 """
@@ -37,6 +37,28 @@ class DecoderLayer:
     window: int = 0
     scale: float = 0.0
     ff: int = 0           # gated feed-forward size, 0: none
+    # attention, continued
+    qk_norm: int = 0        # queries and keys over their root mean square per head
+    v_norm: int = 0         # values too
+    proj_bias: int = 0
+    distance_bias: int = 0  # r1 ln(1 + r2 distance) off the scores
+    keep_first: int = 0     # the first tokens that stay visible past the window
+    kv_from: int = -1       # the earlier attention layer whose keys and values this one reads, -1: its own
+    softcap: float = 0.0    # score = softcap tanh(score / softcap), 0: as it is
+    rot_dims: int = 0       # interleaved rotary positions on this many leading dims of q and k
+    rot_base: float = 0.0
+    rot_factor: float = 1.0    # frequency scaling by wavelength, rot_original 0: none
+    rot_low: float = 0.0
+    rot_high: float = 0.0
+    rot_original: float = 0.0
+    # mixture of experts (instead of ff), experts 0: none
+    experts: int = 0
+    identity: int = 0       # experts past them that return their input
+    top: int = 0
+    groups: int = 0         # groups of neighbours, of which the groups_keep best can be chosen from
+    groups_keep: int = 0
+    expert_ff: int = 0
+    shared_ff: int = 0      # gated shared expert, 0: none
 
 
 @dataclass
@@ -48,6 +70,26 @@ class DecoderConfig:
     norm_eps: float
     embed_scale: float
     layers: List[DecoderLayer] = field(default_factory=list)
+    plain_residual: bool = False  # one stream, x + residual_mult * sublayer, instead of hyper-connections
+    residual_mult: float = 1.0
+    norm_scalar: bool = False     # norms weigh with one number
+    canon_taps: int = 0           # causal input convolution in front of every mixer
+    bigram_buckets: int = 0       # rows of the bigram embedding (less the first token's)
+    bigram_mul_prev: int = 0
+    bigram_mul_cur: int = 0
+    untied_head: bool = False
+
+    def native(self, max_batch: int, act_dtype: int):
+        """The C ABI's view: (pgmi_decoder_config, array of pgmi_layer_spec)."""
+        c = N.DecoderConfigC(self.vocab, self.width, self.streams, self.norm_groups, len(self.layers), self.norm_eps,
+                             self.embed_scale, max_batch, act_dtype, self.plain_residual, self.residual_mult,
+                             self.norm_scalar, self.canon_taps, self.bigram_buckets, self.bigram_mul_prev,
+                             self.bigram_mul_cur, self.untied_head)
+        layers = (N.LayerSpec * len(self.layers))()
+        for spec, layer in zip(layers, self.layers):
+            for name, _ in N.LayerSpec._fields_:
+                setattr(spec, name, getattr(layer, name))
+        return c, layers
 
 
 class StateCache:
@@ -95,12 +137,7 @@ class DecoderEngine(EngineBase):
         self.cfg = cfg
         self.device = torch.device("cuda", torch.cuda.current_device() if device is None else
                                    torch.device(device).index or 0)
-        c = N.DecoderConfigC(cfg.vocab, cfg.width, cfg.streams, cfg.norm_groups, len(cfg.layers), cfg.norm_eps,
-                             cfg.embed_scale, max_batch, ACT_DTYPES[dtype])
-        layers = (N.LayerSpec * len(cfg.layers))()
-        for spec, layer in zip(layers, cfg.layers):
-            for name, _ in N.LayerSpec._fields_:
-                setattr(spec, name, getattr(layer, name))
+        c, layers = cfg.native(max_batch, ACT_DTYPES[dtype])
         h = ctypes.c_void_p()
         N.check(self.lib.pgmi_decoder_create(self.device.index, ctypes.byref(c), layers, ctypes.byref(h)),
                 "pgmi_decoder_create")

@@ -15,13 +15,7 @@ def engine_ctx(cfg, dtype=0, max_batch=4):
     """A bare context (no device memory is touched until weights are bound)."""
     from pgmi import _native as N
     from pgmi import registry
-    d = registry.decoder_config(cfg)
-    c = N.DecoderConfigC(d.vocab, d.width, d.streams, d.norm_groups, len(d.layers), d.norm_eps, d.embed_scale, max_batch,
-                         dtype)
-    layers = (N.LayerSpec * len(d.layers))()
-    for spec, layer in zip(layers, d.layers):
-        for name, _ in N.LayerSpec._fields_:
-            setattr(spec, name, getattr(layer, name))
+    c, layers = registry.decoder_config(cfg).native(max_batch, dtype)
     h = ctypes.c_void_p()
     N.check(N.lib().pgmi_decoder_create(0, ctypes.byref(c), layers, ctypes.byref(h)))
     return h
