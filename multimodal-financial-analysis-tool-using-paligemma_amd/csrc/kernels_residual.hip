@@ -173,7 +173,7 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a) {
 #pragma unroll
                 for (int v = 0; v < V; ++v) o[v] = fmaf(bf2f(cw[v * a.taps + a.taps - 1 - j]), q[v], o[v]);
             }
-            stv(ring + (long)(pos % a.taps) * D + dd[i], n);
+            if (a.taps > 1) stv(ring + (long)(pos % a.taps) * D + dd[i], n);
         }
         stv(h + dd[i], o);
     }

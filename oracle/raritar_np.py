@@ -67,7 +67,7 @@ def visible(i, mask):
 
 
 def capped(s, cap):
-    return cap * np.tanh(s / cap)
+    return cap * np.tanh(s / cap) if cap else s
 
 
 def attend(q, k, v, scale, cap):
@@ -202,27 +202,60 @@ def bf16(w):
     return u.view(np.float32).reshape(np.shape(w))
 
 
+def route_margin(z, correction, r):
+    """How far the nearest other choice of experts is: the smallest gap between a choice score that is taken (of the
+    groups, then of the experts in them) and one that is left."""
+    s = np.exp(z - z.max())
+    choice = (s / s.sum() + correction).reshape(r["groups"]["count"], -1)
+    best = np.sort(choice.max(1))[::-1]
+    keep, top = r["groups"]["keep"], r["top"]
+    gap = best[keep - 1] - best[keep] if keep < len(best) else np.inf
+    kept = choice[np.argsort(-choice.max(1), kind="stable")[:keep]].reshape(-1)
+    kept = np.sort(kept)[::-1]
+    return min(gap, kept[top - 1] - kept[top] if top < len(kept) else np.inf)
+
+
+KINDS = 5
+
+
 def random_weights(cfg, seed):
-    """float32 arrays holding bf16 values; scales chosen so that every mechanism moves the logits."""
+    """float32 arrays holding bf16 values; scales chosen so that every mechanism moves the logits.  The last coordinates
+    of the stream hold one of KINDS patterns by token, which no layer changes and which alone the routers read: a choice
+    of experts is never a close call that rounding could turn."""
     rng = np.random.default_rng(seed)
-    W = {}
+    D, W = cfg["width"], {}
+    T = max(KINDS, D // 6)
+    patterns = np.sign(rng.standard_normal((KINDS, T))) * 2.0
     for n, shp in tensor_shapes(cfg).items():
         r = rng.standard_normal(shp)
         leaf = n.split(".", 1)[1] if n[0] == "l" else n
         if leaf in ("embed", "bigram"):
             w = r
+            w[:, D - T:] = patterns[np.arange(shp[0]) % KINDS] if leaf == "embed" else 0.0
         elif "norm" in leaf:
-            w = 1.0 + 0.3 * r
+            w = rng.uniform(0.85, 1.15, shp) if leaf == "norm2" else 1.0 + 0.2 * r
         elif leaf == "canon1":
             w = r * 0.4
         elif leaf == "mlp.correction":
-            w = 0.3 * r
+            continue  # with the router
         elif leaf == "mlp.router":
-            w = r * (2.0 / np.sqrt(shp[-1]))
-        elif leaf.endswith("down"):
-            w = r * (2.5 / np.sqrt(shp[-1]))
-        elif leaf == "mix.o":
-            w = r * (2.0 / np.sqrt(shp[-1]))
+            m = cfg["layers"][int(n[1:n.index(".")])]["mlp"]["router"]
+            for _ in range(20000):
+                w = np.zeros(shp)
+                w[:, D - T:] = bf16(rng.standard_normal((shp[0], T)) * (1.2 / np.sqrt(T)))
+                c = bf16(rng.standard_normal(shp[0]) * 0.2 - 0.2)
+                # the norm divides the patterns by anything from 1.2 to 4.2, say: the choice is the same for all of it
+                zs = [[w[:, D - T:] @ p / d for d in np.geomspace(1.2, 4.2, 9)] for p in patterns]
+                sets = [{frozenset(e for e, _ in route(z, c, m)) for z in per} for per in zs]
+                if all(len(x) == 1 for x in sets) and (len(set.union(*sets)) > 2 or m["top"] == shp[0]) and \
+                        all(route_margin(z, c, m) > 0.003 for per in zs for z in per):
+                    break
+            else:
+                raise ValueError("no router with a margin found")
+            W[n.replace("router", "correction")] = c
+        elif leaf.endswith("down") or leaf == "mix.o":
+            w = r * ((2.5 if leaf.endswith("down") else 1.5) / np.sqrt(shp[-1]))
+            w[D - T:] = 0.0
         else:
             w = r * (1.3 / np.sqrt(shp[-1]))
         W[n] = bf16(w)
