@@ -66,7 +66,7 @@ def parse():
                     help="skip the drop-in module API leg (inference.py's loop through PaliGemmaForConditionalGeneration)")
     ap.add_argument("--api-tokens", type=int, default=32)
     ap.add_argument("--decoder", default=None, metavar="SIZES",
-                    help="measure the layered decoders instead (1b, 2b, 7b, with commas between; bench_decoder.py): one "
+                    help="measure the layered decoders instead (1b, 2b, 7b, raritar-1b, ..., with commas between; bench_decoder.py): one "
                          "JSON line per size, one GPU")
     ap.add_argument("--dry-run", action="store_true",
                     help="rank logic only (world / batch / image shards / max-over-ranks timing / token gather) "

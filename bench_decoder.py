@@ -1,6 +1,6 @@
-"""The layered-decoder legs of bench.py (`python bench.py --decoder 1b,2b,7b`): prefill and decode throughput of Tuvodra
-at the layer sizes of real models (random weights), one JSON line per size, and for "2b" PaliGemma's text decoder at
-the same width, feed-forward and vocabulary beside it.  One GPU."""
+"""The layered-decoder legs of bench.py (`python bench.py --decoder 1b,2b,7b,raritar-2b`): prefill and decode throughput of
+Tuvodra and Raritar at the layer sizes of real models (random weights), one JSON line per size, and for Tuvodra "2b"
+PaliGemma's text decoder at the same width, feed-forward and vocabulary beside it.  One GPU."""
 from __future__ import annotations
 
 import gc
@@ -32,6 +32,21 @@ def decode_entry(ms, B, weight_bytes):
             "weights_GBs": round(weight_bytes / ms / 1e6, 1), "frac_hbm": round(weight_bytes / ms / 1e6 / HBM_PEAK_GBS, 4)}
 
 
+def step_bytes(eng, cfg, B):
+    """Weight bytes a decode step of B sequences reads: every weight once (a table's rows not counted, the embedding where
+    it is the output matrix), of a mixture the experts that B rows choose on average."""
+    total = 0.0
+    for name, v in eng.views.items():
+        n = v.numel() * 2
+        if name == "bigram" or (name == "embed" and cfg.untied_head):
+            n = 0
+        elif ".mlp.e" in name:
+            layer = cfg.layers[int(name[1:name.index(".")])]
+            n *= 1.0 - (1.0 - layer.top / (layer.experts + layer.identity)) ** B
+        total += n
+    return total
+
+
 def decoder_leg(size, steps, warmup, seed, dev):
     from pgmi import DecoderEngine, registry
     from pgmi.synthetic import decoder_bench_config, decoder_policy
@@ -41,7 +56,6 @@ def decoder_leg(size, steps, warmup, seed, dev):
     eng.fill_synthetic(seed, decoder_policy)
     eng.prepare()
     V = cfg.vocab
-    # every weight is read once per step (the embedding as the output matrix)
     weight_bytes = sum(v.numel() * 2 for v in eng.views.values())
     out = {"params_bytes": weight_bytes, "prefill": {}, "decode": {}}
     for B, T in PREFILLS:
@@ -64,7 +78,7 @@ def decoder_leg(size, steps, warmup, seed, dev):
         ids = torch.randint(0, V, (B,), device=dev)
         lg = torch.empty((B, V), device=dev)
         ms = timed(lambda: eng.decode(cache, slots, ids, logits=lg, next_ids=ids, graph=True), steps, max(3, warmup))
-        out["decode"][f"{B}x{CONTEXT}"] = decode_entry(ms, B, weight_bytes)
+        out["decode"][f"{B}x{CONTEXT}"] = decode_entry(ms, B, step_bytes(eng, cfg, B))
         del cache
     return raw, out
 
@@ -117,12 +131,13 @@ def run(a) -> None:
     for size in a.decoder.split(","):
         raw, leg = decoder_leg(size, steps, warmup, a.seed, dev)
         one = leg["decode"][f"1x{CONTEXT}"]
-        line = {"metric": f"layered decoder (Tuvodra {size}) greedy decode tokens/s, batch 1", "value": one["tok_s"],
+        ffs = [x["mlp"] for x in raw["layers"] if x["mlp"]]
+        line = {"metric": f"layered decoder ({raw['architecture']} {size}) greedy decode tokens/s, batch 1", "value": one["tok_s"],
                 "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": warmup, "ms_per_step": one["ms_per_step"],
                 "higher_is_better": True, "dtype": "bf16", "data": "synthetic (random weights, random token ids)",
                 "config": {"width": raw["width"], "layers": [x["type"] for x in raw["layers"]], "vocab": raw["vocab"],
-                           "mixers": {x["type"]: x["mixer"] for x in raw["layers"]}, "streams": raw["streams"],
-                           "ff": next(x["mlp"]["ff"] for x in raw["layers"] if x["mlp"])}, **leg}
+                           "mixers": {x["type"]: x["mixer"] for x in raw["layers"]}, "streams": raw.get("streams", 1),
+                           "ff": ffs[0]["ff"] if ffs[0]["kind"] == "dense" else ffs[0]}, **leg}
         gc.collect()
         if size == "2b":
             line["paligemma_text"] = gemma_leg(steps, warmup, a.seed, dev)

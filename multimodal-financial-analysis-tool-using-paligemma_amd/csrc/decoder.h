@@ -104,7 +104,12 @@ struct ResidualArgs {
     int taps;
     float* ring;
 };
+struct RouteArgs;
 void residual_norm(hipStream_t s, Act act, const ResidualArgs& a);
+// residual_norm of one row per sequence and bf16 activations with the mixture's router behind it, in one launch:
+// logits h . W^T (rows n, then the shared expert's gate), the choice, and the lists (RouteArgs.active given).
+bool residual_route_fits(Act act, int rows, int D);
+void residual_route(hipStream_t s, const ResidualArgs& a, const uint16_t* W, int ldw, const RouteArgs& r);
 
 // Input convolution over packed rows: n = X * inv * w is what the norm gives, h = n + conv(n),
 // conv(n)_t = sum_j cw[:, j] n_(t - taps + 1 + j), zeros before the sequence.  ring [slot][taps][D] fp32 keeps the norm of
@@ -130,7 +135,7 @@ void canon(hipStream_t s, Act act, const CanonArgs& a);
 // z: fp32 slabs [split][rows][ldz], summed: columns 0 .. n-1 the router's logits, column n the shared expert's gate (gate
 // != null).  Scores are their softmax; choice = score + correction picks the groups (largest choice of a group, `keep` of
 // `groups` equal ones) and the top experts inside them; weights are the scores.  Lists: list[e * cap ..] the entries
-// (row * top + k) of expert e < experts, cnt[e] how many.
+// (row * top + k) of expert e < experts in any order, cnt[e] how many (zero before the launch).
 struct RouteArgs {
     const float* z;
     int split;
@@ -140,12 +145,12 @@ struct RouteArgs {
     int* sel;
     float* w;
     float* gate;
-    int* cnt;  // zeroed before the launch, unless active is given
+    int* cnt;
     int* list;
     int cap;
-    int* active;  // up to kRouteRows rows: cnt is set, active[0] experts are used, active[1 ..] which
+    int* active;  // residual_route: active[0] (zero before the launch) experts are used, active[1 ..] which
 };
-constexpr int kRouteRows = 16;
+constexpr int kRouteRows = 16;  // most rows of residual_route and experts_skinny
 constexpr int kMaxExperts = 512;  // identity experts included: a workgroup's choice scores fit LDS
 void route(hipStream_t s, const RouteArgs& a);
 
@@ -167,7 +172,7 @@ struct ExpertArgs {
     const int* cnt;
     const int* list;
     int cap, experts, entries;  // entries: rows * top
-    // few rows (RouteArgs.active given): the shared expert rides along, its rows 0 .. B-1 (Wsh null: none)
+    // experts_skinny: the used experts (RouteArgs.active); the shared expert rides along, its rows 0 .. B-1 (Wsh null: none)
     const int* active;
     const uint16_t* Wsh;
     int ldwsh, Nsh, Ksh;

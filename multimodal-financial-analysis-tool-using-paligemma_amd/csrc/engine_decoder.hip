@@ -66,6 +66,7 @@ struct DecoderState {
     uint8_t *ea = nullptr, *ey = nullptr;
     float *inv = nullptr, *ew = nullptr, *egate = nullptr;
     int *esel = nullptr, *elist = nullptr, *ecnt = nullptr, *eactive = nullptr;
+    int zero_words = 0;  // the counters and the number of used experts
     size_t slab_bytes = 0;
     int ldh = 0, ld0 = 0, ld1 = 0, ld2 = 0, ldd = 0;
     // step metadata
@@ -450,6 +451,7 @@ int ensure_workspace(pgmi_ctx* x, int rows, int chunks, int gchunks) {
     d.elist = reinterpret_cast<int*>(p + off[17]);
     d.ecnt = reinterpret_cast<int*>(p + off[18]);
     d.eactive = d.ecnt + ne;
+    d.zero_words = ne + 1;
     d.rows = rows;
     d.chunks = chunks;
     d.gchunks = gchunks;
@@ -701,8 +703,9 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
     bool have_h = !plain;  // d.h holds the coming sublayer's input
     bool first = true;     // plain residual: X is not made yet
     Pending pend;
-    // plain residual: the finished sublayer folded in and the input of sublayer q of layer i (the end: i = n_layers) in d.h
-    auto read = [&](int i, int q) {
+    // plain residual: the finished sublayer folded in and the input of sublayer q of layer i (the end: i = n_layers) in d.h;
+    // router: a mixture's choice in the same launch
+    auto read = [&](int i, int q, const RouteArgs* router = nullptr) {
         if (!plain) return;
         const bool end = i == d.c.n_layers;
         ResidualArgs a = residual_args(d, B, pend, end ? d.fnorm : d.W[i].sub[q].norm);
@@ -711,8 +714,9 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
         if (!end && q == 0 && d.c.canon_taps > 0) {
             a.taps = d.c.canon_taps; a.cw = d.W[i].canon; a.ring = at<float>(state, st[i].ring);
         }
-        if (!end && q == 1 && d.L[i].experts) { a.zero = d.ecnt; a.nzero = d.L[i].experts; }
-        residual_norm(s, d.act, a);
+        if (!end && q == 0 && d.L[i].experts) { a.zero = d.ecnt; a.nzero = d.zero_words; }
+        if (router) residual_route(s, a, d.W[i].router.w, d.W[i].router.ldw, *router);
+        else residual_norm(s, d.act, a);
         pend = {};
         first = false;
         have_h = true;
@@ -820,9 +824,25 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
             }
             out_proj(w.o, d.p2, ldc, w.sub[0]);
         }
-        if (has_ff(l)) read(i, 1);
-        bool shared_done = false;
-        if (l.experts) {
+        const bool few = l.experts && residual_route_fits(d.act, B, D);
+        if (has_ff(l) && !few) read(i, 1);
+        if (few) {  // router and choice behind the norm; the shared expert rides along with the others
+            RouteArgs r = route_args(d, l, w, B, 1);
+            r.active = d.eactive;
+            read(i, 1, &r);
+            ExpertArgs up = expert_args(d, l, w, B, EX_SWIGLU), down = expert_args(d, l, w, B, EX_STORE);
+            up.active = down.active = d.eactive;
+            up.B = down.B = B;
+            if (l.shared_ff) {
+                up.Wsh = w.gu.w; up.ldwsh = w.gu.ldw; up.Nsh = l.shared_ff; up.Ksh = w.gu.k; up.Ash = d.h; up.ldash = d.ldh;
+                up.outsh = d.p2; up.ldosh = r8(l.shared_ff);
+                down.Wsh = w.down.w; down.ldwsh = w.down.ldw; down.Nsh = D; down.Ksh = w.down.k; down.Ash = d.p2;
+                down.ldash = r8(l.shared_ff); down.outsh = d.slabs; down.ldosh = D;
+            }
+            experts_skinny(s, EX_SWIGLU, up);
+            experts_skinny(s, EX_STORE, down);
+            if (l.shared_ff) pend = {d.slabs, 1, &w.sub[1], {}};
+        } else if (l.experts) {
             const bool fr = gemv_rt_fits(form, w.router.k, d.act);
             GemvRtArgs g = base(w.sub[1], w.router, fr);
             int sp;
@@ -833,30 +853,11 @@ int decode_body_rt(pgmi_ctx* x, hipStream_t s, const int64_t* ids, int B, void* 
                 sp = matmul_rt(s, d.act, d.h, d.ldh, w.router.w, w.router.ldw, B, w.router.n, w.router.k, RT_SLABS, nullptr,
                                d.slabs, 0, d.slab_bytes, nullptr);
             }
-            RouteArgs r = route_args(d, l, w, B, sp);
-            ExpertArgs up = expert_args(d, l, w, B, EX_SWIGLU), down = expert_args(d, l, w, B, EX_STORE);
-            if (d.act == ACT_BF16 && B <= kRouteRows) {  // the shared expert rides along
-                r.active = d.eactive;
-                up.active = down.active = d.eactive;
-                route(s, r);
-                up.B = down.B = B;
-                if (l.shared_ff) {
-                    up.Wsh = w.gu.w; up.ldwsh = w.gu.ldw; up.Nsh = l.shared_ff; up.Ksh = w.gu.k; up.Ash = d.h; up.ldash = d.ldh;
-                    up.outsh = d.p2; up.ldosh = r8(l.shared_ff);
-                    down.Wsh = w.down.w; down.ldwsh = w.down.ldw; down.Nsh = D; down.Ksh = w.down.k; down.Ash = d.p2;
-                    down.ldash = r8(l.shared_ff); down.outsh = d.slabs; down.ldosh = D;
-                }
-                experts_skinny(s, EX_SWIGLU, up);
-                experts_skinny(s, EX_STORE, down);
-                if (l.shared_ff) pend = {d.slabs, 1, &w.sub[1], {}};
-                shared_done = true;
-            } else {
-                route(s, r);
-                experts_rt(s, d.act, EX_SWIGLU, up);
-                experts_rt(s, d.act, EX_STORE, down);
-            }
+            route(s, route_args(d, l, w, B, sp));
+            experts_rt(s, d.act, EX_SWIGLU, expert_args(d, l, w, B, EX_SWIGLU));
+            experts_rt(s, d.act, EX_STORE, expert_args(d, l, w, B, EX_STORE));
         }
-        if (const int ff = l.experts ? l.shared_ff : l.ff; ff && !shared_done) {
+        if (const int ff = few ? 0 : l.experts ? l.shared_ff : l.ff) {
             const bool fgu = gemv_rt_fits(form, w.gu.k, d.act);
             if (l.experts) have_h = true;  // the mixture's input, once more
             GemvRtArgs g = base(w.sub[1], w.gu, fgu);

@@ -13,123 +13,49 @@
 
 #include "act.h"
 #include "decoder.h"
+#include "route.h"
 
 namespace pgmi {
 
 namespace {
 
 // ---------------------------------------------------------------- routing
-__device__ __forceinline__ void wave_best(float& v, int& i) {  // largest value, smallest index among equals
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-        const float u = __shfl_xor(v, o, 64);
-        const int j = __shfl_xor(i, o, 64);
-        if (u > v || (u == v && j < i)) { v = u; i = j; }
-    }
-}
-// LDS written by one lane of a wave and read by another (a wave's LDS operations complete in order)
-__device__ __forceinline__ void wave_sync() {
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-}
-
-constexpr int kNobody = 0x7fffffff;
-
-// dynamic LDS: per wave n choice scores and `groups` group scores; then the experts' counters, the places of their local
-// lists, and per wave the places of its row's entries
+// dynamic LDS: per wave route_words() of its row; then the experts' counters, the places of their local lists, and per
+// wave the expert and the place of its row's entries
 __global__ void __launch_bounds__(1024) k_route(RouteArgs a) {
-    extern __shared__ float sm[];
-    __shared__ int used;
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, NW = blockDim.x / 64, n = a.n;
-    float* ch = sm + (long)wave * (n + a.groups);
-    float* gr = ch + n;
-    int* lcnt = reinterpret_cast<int*>(sm + (long)NW * (n + a.groups));
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, NW = blockDim.x / 64, n = a.n, words = route_words(n, a.groups);
+    float* sc = sm + (long)wave * words;
+    int* lcnt = reinterpret_cast<int*>(sm + (long)NW * words);
     int* base = lcnt + a.experts;
-    int* rank = base + a.experts + wave * a.top;
+    int* who = base + a.experts + wave * 2 * a.top;
+    int* rank = who + a.top;
     for (int e = threadIdx.x; e < a.experts; e += blockDim.x) lcnt[e] = 0;
-    if (threadIdx.x == 0) used = 0;
     __syncthreads();
-    const int row = blockIdx.x * NW + wave, gs = n / a.groups;
+    const int row = blockIdx.x * NW + wave;
     if (row < a.rows) {
         auto logit = [&](int c) {
             float z = 0.0f;
             for (int q = 0; q < a.split; ++q) z += a.z[(long)q * a.zstride + (long)row * a.ldz + c];
             return z;
         };
-        float mx = -INFINITY;
-        for (int c = lane; c < n; c += 64) {
-            ch[c] = logit(c);
-            mx = fmaxf(mx, ch[c]);
-        }
-        mx = wave_max(mx);
-        float sum = 0.0f;
-        for (int c = lane; c < n; c += 64) {
-            ch[c] = expf(ch[c] - mx);
-            sum += ch[c];
-        }
-        const float inv = 1.0f / wave_sum(sum);
-        for (int c = lane; c < n; c += 64) ch[c] = fmaf(ch[c], inv, bf2f(a.correction[c]));
+        for (int c = lane; c < n; c += 64) sc[c] = logit(c);
         if (a.gate && lane == 0) a.gate[row] = 1.0f / (1.0f + expf(-logit(n)));
         wave_sync();
-        const bool limited = a.keep < a.groups;
-        if (limited) {
-            for (int g = lane; g < a.groups; g += 64) {
-                float b = -INFINITY;
-                for (int c = 0; c < gs; ++c) b = fmaxf(b, ch[g * gs + c]);
-                gr[g] = b;
-            }
-            wave_sync();
-            for (int k = 0; k < a.keep; ++k) {  // the best groups become +inf
-                float b = -INFINITY;
-                int bi = kNobody;
-                for (int g = lane; g < a.groups; g += 64)
-                    if (gr[g] != INFINITY && (gr[g] > b || bi == kNobody)) { b = gr[g]; bi = g; }
-                wave_best(b, bi);
-                if (lane == 0 && bi != kNobody) gr[bi] = INFINITY;
-                wave_sync();
-            }
-        }
-        for (int k = 0; k < a.top; ++k) {
-            float b = -INFINITY;
-            int bi = kNobody;
-            for (int c = lane; c < n; c += 64)
-                if (ch[c] > b && (!limited || gr[c / gs] == INFINITY)) { b = ch[c]; bi = c; }
-            wave_best(b, bi);
-            if (lane == 0) {
-                const long at = (long)row * a.top + k;
-                rank[k] = -1;
-                if (bi != kNobody) {
-                    a.sel[at] = bi;
-                    a.w[at] = expf(logit(bi) - mx) * inv;
-                    ch[bi] = -INFINITY;  // not again
-                    if (bi < a.experts) rank[k] = atomicAdd(&lcnt[bi], 1);
-                } else {  // no score left to compare (not a number): nobody's entry, and its weight says so
-                    a.sel[at] = n;
-                    a.w[at] = NAN;
-                }
-            }
-            wave_sync();
-        }
+        route_row(sc, a.correction, n, a.groups, a.keep, a.top, lane, [&](int k, int e, float w) {
+            const long at = (long)row * a.top + k;
+            a.sel[at] = e;
+            a.w[at] = w;
+            who[k] = e;
+            if (e < a.experts) rank[k] = atomicAdd(&lcnt[e], 1);
+        });
     }
     __syncthreads();
-    if (a.active) {  // one workgroup: its counts are the counts
-        for (int e = threadIdx.x; e < a.experts; e += blockDim.x) {
-            base[e] = 0;
-            a.cnt[e] = lcnt[e];
-            if (lcnt[e] > 0) a.active[1 + atomicAdd(&used, 1)] = e;
-        }
-        __syncthreads();
-        if (threadIdx.x == 0) a.active[0] = used;
-    } else {
-        for (int e = threadIdx.x; e < a.experts; e += blockDim.x) base[e] = lcnt[e] > 0 ? atomicAdd(&a.cnt[e], lcnt[e]) : 0;
-        __syncthreads();
-    }
+    for (int e = threadIdx.x; e < a.experts; e += blockDim.x) base[e] = lcnt[e] > 0 ? atomicAdd(&a.cnt[e], lcnt[e]) : 0;
+    __syncthreads();
     if (row < a.rows)
         for (int k = lane; k < a.top; k += 64)
-            if (rank[k] >= 0) {
-                const int at = row * a.top + k, e = a.sel[at];
-                a.list[(long)e * a.cap + base[e] + rank[k]] = at;
-            }
+            if (who[k] < a.experts) a.list[(long)who[k] * a.cap + base[who[k]] + rank[k]] = row * a.top + k;
 }
 
 // ---------------------------------------------------------------- which expert a tile belongs to
@@ -378,7 +304,7 @@ __global__ void __launch_bounds__(256) k_experts_f32(ExpertArgs a) {
 // its list.  4 waves split K; a lane reads 32 contiguous bytes of its weight row per 64-deep step, as k_skinny.
 template <int MODE>
 __global__ void __launch_bounds__(256) k_experts_skinny(ExpertArgs a) {
-    constexpr int NM = MODE == EX_SWIGLU ? 2 : 1, U = 4;
+    constexpr int NM = MODE == EX_SWIGLU ? 2 : 1, U = 8 / NM;
     __shared__ float sums[4][NM][16][17];
     const bool shared = blockIdx.y == 0;
     if (shared ? !a.Wsh : (int)blockIdx.y > a.active[0]) return;
@@ -388,11 +314,8 @@ __global__ void __launch_bounds__(256) k_experts_skinny(ExpertArgs a) {
     if (n0 >= ldo) return;
     const uint16_t* W = shared ? a.Wsh : a.W + e * a.wstride;
     const int* list = a.list + (long)e * a.cap;
-    const int cnt = shared ? a.B : a.cnt[e];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int li = lane & 15, lg = lane >> 4;
-    const int m = min(li, cnt - 1), row = shared ? m : list[m] / a.gather;
-    const uint16_t* xp = reinterpret_cast<const uint16_t*>(shared ? a.Ash : a.A) + (long)row * (shared ? a.ldash : a.lda);
     const uint16_t* wp[NM];
 #pragma unroll
     for (int q = 0; q < NM; ++q) wp[q] = W + ((long)q * N + min(n0 + li, N - 1)) * ldw;
@@ -400,18 +323,28 @@ __global__ void __launch_bounds__(256) k_experts_skinny(ExpertArgs a) {
 #pragma unroll
     for (int q = 0; q < NM; ++q) acc[q] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int nstep = (K + 63) / 64;
-    for (int s0 = wave; s0 < nstep; s0 += 4 * U) {
-        uint4 w[U][NM][2], x[U][2];
+    uint4 w[U][NM][2];
+    auto wload = [&](int s0) {
 #pragma unroll
         for (int i = 0; i < U; ++i) {
             const int k = (s0 + 4 * i) * 64 + lg * 16;
 #pragma unroll
-            for (int h = 0; h < 2; ++h) {
-                const bool ok = k + 8 * h < K;
+            for (int h = 0; h < 2; ++h)
 #pragma unroll
-                for (int q = 0; q < NM; ++q) w[i][q][h] = ldg16_sel(wp[q] + k + 8 * h, ok, wp[q]);
-                x[i][h] = ldg16_sel(xp + k + 8 * h, ok, xp);
-            }
+                for (int q = 0; q < NM; ++q) w[i][q][h] = ldg16_sel(wp[q] + k + 8 * h, k + 8 * h < K, wp[q]);
+        }
+    };
+    wload(wave);  // in flight while the rows are looked up
+    const int cnt = shared ? a.B : a.cnt[e];
+    const int m = min(li, cnt - 1), row = shared ? m : list[m] / a.gather;
+    const uint16_t* xp = reinterpret_cast<const uint16_t*>(shared ? a.Ash : a.A) + (long)row * (shared ? a.ldash : a.lda);
+    for (int s0 = wave; s0 < nstep; s0 += 4 * U) {
+        uint4 x[U][2];
+#pragma unroll
+        for (int i = 0; i < U; ++i) {
+            const int k = (s0 + 4 * i) * 64 + lg * 16;
+#pragma unroll
+            for (int h = 0; h < 2; ++h) x[i][h] = ldg16_sel(xp + k + 8 * h, k + 8 * h < K, xp);
         }
 #pragma unroll
         for (int i = 0; i < U; ++i)
@@ -420,6 +353,7 @@ __global__ void __launch_bounds__(256) k_experts_skinny(ExpertArgs a) {
 #pragma unroll
                 for (int q = 0; q < NM; ++q)
                     acc[q] = mfma16(__builtin_bit_cast(short8, w[i][q][h]), __builtin_bit_cast(short8, x[i][h]), acc[q]);
+        if (s0 + 4 * U < nstep) wload(s0 + 4 * U);
     }
 #pragma unroll
     for (int q = 0; q < NM; ++q)
@@ -443,8 +377,8 @@ __global__ void __launch_bounds__(256) k_experts_skinny(ExpertArgs a) {
 }  // namespace
 
 void route(hipStream_t s, const RouteArgs& a) {
-    const int nw = a.active ? std::max(1, a.rows) : a.rows >= 2048 ? 16 : 4;
-    const size_t lds = ((size_t)nw * (a.n + a.groups + a.top) + 2 * a.experts) * sizeof(float);
+    const int nw = a.rows >= 2048 ? 16 : 4;
+    const size_t lds = ((size_t)nw * (route_words(a.n, a.groups) + 2 * a.top) + 2 * a.experts) * sizeof(float);
     if (lds > 60 * 1024)
         (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&k_route), hipFuncAttributeMaxDynamicSharedMemorySize,
                                   (int)lds);

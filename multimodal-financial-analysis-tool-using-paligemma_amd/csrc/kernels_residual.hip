@@ -1,10 +1,12 @@
 // kernels_residual.hip -- one residual stream: the embedding (with a table of token pairs), the scaled update from a
-// finished sublayer (split-K slabs, a mixture's outputs), the RMS norm in front of the next one, and the causal input
-// convolution added to what a mixer reads.  Stream, sums, norms and the convolution are fp32.
+// finished sublayer (split-K slabs, a mixture's outputs), the RMS norm in front of the next one, a mixture's router behind
+// that norm, and the causal input convolution added to what a mixer reads.  Stream, sums, norms, router and convolution
+// are fp32.
 #include <algorithm>
 
 #include "act.h"
 #include "decoder.h"
+#include "route.h"
 
 namespace pgmi {
 
@@ -19,10 +21,35 @@ __device__ __forceinline__ void stv(S* p, const float (&v)[4]) { st4(p, v); }
 template <typename S>
 __device__ __forceinline__ void stv(S* p, const float (&v)[1]) { stf(p, v[0]); }
 
+struct RouterArgs {
+    const uint16_t* W;  // [n, and the gate's row][ldw]
+    int ldw;
+    RouteArgs r;
+};
+
 // One workgroup per row; PC pieces of V elements per thread, every load of a source issued before its first use.
-template <typename T, int V, int PC>
-__global__ void __launch_bounds__(1024) k_residual(ResidualArgs a) {
+// RT: the router of the row and its choice behind the norm, 16 waves; dynamic LDS: route_words(), then h [ldh].
+template <typename T, int V, int PC, bool RT>
+__global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt) {
     __shared__ float red[16];
+    extern __shared__ __attribute__((aligned(16))) float rsm[];
+    constexpr int RR = 4, RK = 4;  // router rows and 512-wide steps a wave has in flight
+    const int rows_r = RT ? rt.r.n + (rt.r.gate != nullptr) : 0;
+    uint4 rw[RT ? RR : 1][RT ? RK : 1];
+    auto rload = [&](int n0, int k0) {
+        if constexpr (RT) {
+#pragma unroll
+            for (int q = 0; q < RR; ++q) {
+                const uint16_t* p = rt.W + (long)min(n0 + 16 * q, rows_r - 1) * rt.ldw;
+#pragma unroll
+                for (int i = 0; i < RK; ++i) {
+                    const int k = k0 + i * 512 + (threadIdx.x & 63) * 8;
+                    rw[q][i] = ldg16_sel(p + k, k < a.ldh, p);
+                }
+            }
+        }
+    };
+    rload(threadIdx.x >> 6, 0);  // in flight during the update and the norm
     const int tid = threadIdx.x, NT = blockDim.x, D = a.D;
     const int row = a.rows_idx ? a.rows_idx[blockIdx.x] : blockIdx.x;
     if (a.zero && blockIdx.x == 0)
@@ -147,6 +174,7 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a) {
     if (a.inv && tid == 0) a.inv[row] = inv;
     if (!a.h) return;
     T* h = reinterpret_cast<T*>(a.h) + (long)blockIdx.x * a.ldh;
+    T* hs = reinterpret_cast<T*>(rsm + (RT ? route_words(rt.r.n, rt.r.groups) : 0));
     const float g = a.w_scalar ? bf2f(a.w[0]) : 0.0f;
     float* ring = nullptr;
     if (a.taps > 0) {
@@ -176,20 +204,65 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a) {
             if (a.taps > 1) stv(ring + (long)(pos % a.taps) * D + dd[i], n);
         }
         stv(h + dd[i], o);
+        if constexpr (RT) stv(hs + dd[i], o);
     }
-    for (int d = D + tid; d < a.ldh; d += NT) stf(h + d, 0.0f);
+    for (int d = D + tid; d < a.ldh; d += NT) {
+        stf(h + d, 0.0f);
+        if constexpr (RT) stf(hs + d, 0.0f);
+    }
+    if constexpr (RT) {
+        const RouteArgs& r = rt.r;
+        const int lane = tid & 63, wave = tid >> 6;
+        float* z = rsm;
+        __shared__ float gate;
+        __syncthreads();
+        for (int n0 = wave; n0 < rows_r; n0 += 16 * RR) {
+            float acc[RR] = {};
+            for (int k0 = 0; k0 < a.ldh; k0 += 512 * RK) {
+                if (n0 > wave || k0 > 0) rload(n0, k0);
+#pragma unroll
+                for (int i = 0; i < RK; ++i) {
+                    const int k = k0 + i * 512 + lane * 8;
+                    const uint4 x = k < a.ldh ? *reinterpret_cast<const uint4*>(hs + k) : make_uint4(0, 0, 0, 0);
+#pragma unroll
+                    for (int q = 0; q < RR; ++q) acc[q] = dot8(rw[q][i], x, acc[q]);
+                }
+            }
+#pragma unroll
+            for (int q = 0; q < RR; ++q) acc[q] = wave_sum(acc[q]);
+#pragma unroll
+            for (int q = 0; q < RR; ++q)
+                if (lane == 0 && n0 + 16 * q < rows_r) {
+                    if (n0 + 16 * q < r.n) z[n0 + 16 * q] = acc[q];
+                    else gate = acc[q];
+                }
+        }
+        __syncthreads();
+        if (wave > 0) return;
+        if (lane == 0 && r.gate) r.gate[row] = 1.0f / (1.0f + expf(-gate));
+        route_row(z, r.correction, r.n, r.groups, r.keep, r.top, lane, [&](int k, int e, float w) {
+            const int at = row * r.top + k;
+            r.sel[at] = e;
+            r.w[at] = w;
+            if (e < r.experts) {
+                const int m = atomicAdd(&r.cnt[e], 1);
+                r.list[(long)e * r.cap + m] = at;
+                if (m == 0) r.active[1 + atomicAdd(&r.active[0], 1)] = e;
+            }
+        });
+    }
 }
 
 template <typename T>
 void residual_t(hipStream_t s, const ResidualArgs& a) {
     auto go = [&](auto kern, int v) {
         const int threads = std::min(1024, (a.D / v + 63) / 64 * 64);
-        hipLaunchKernelGGL(kern, dim3(a.rows), dim3(std::max(64, threads)), 0, s, a);
+        hipLaunchKernelGGL(kern, dim3(a.rows), dim3(std::max(64, threads)), 0, s, a, RouterArgs{});
     };
-    if (a.D % 4 == 0 && a.D <= 4096) go(k_residual<T, 4, 1>, 4);
-    else if (a.D % 4 == 0) go(k_residual<T, 4, 4>, 4);
-    else if (a.D <= 1024) go(k_residual<T, 1, 1>, 1);
-    else go(k_residual<T, 1, 16>, 1);
+    if (a.D % 4 == 0 && a.D <= 4096) go(k_residual<T, 4, 1, false>, 4);
+    else if (a.D % 4 == 0) go(k_residual<T, 4, 4, false>, 4);
+    else if (a.D <= 1024) go(k_residual<T, 1, 1, false>, 1);
+    else go(k_residual<T, 1, 16, false>, 1);
 }
 
 // ---------------------------------------------------------------- input convolution
@@ -296,6 +369,15 @@ void residual_norm(hipStream_t s, Act act, const ResidualArgs& a) {
     if (a.rows <= 0) return;
     if (act == ACT_F32) residual_t<float>(s, a);
     else residual_t<uint16_t>(s, a);
+}
+
+bool residual_route_fits(Act act, int rows, int D) {
+    return act == ACT_BF16 && rows <= kRouteRows && D % 4 == 0 && D <= 4096;
+}
+
+void residual_route(hipStream_t s, const ResidualArgs& a, const uint16_t* W, int ldw, const RouteArgs& r) {
+    const size_t lds = (size_t)route_words(r.n, r.groups) * sizeof(float) + (size_t)a.ldh * sizeof(uint16_t);
+    hipLaunchKernelGGL((k_residual<uint16_t, 4, 1, true>), dim3(a.rows), dim3(1024), lds, s, a, RouterArgs{W, ldw, r});
 }
 
 void canon(hipStream_t s, Act act, const CanonArgs& a) {

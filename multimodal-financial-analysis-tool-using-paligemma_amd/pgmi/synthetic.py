@@ -72,8 +72,10 @@ def decoder_policy(name: str, shape: tuple) -> "tuple[float, float]":
     """init_policy's counterpart for layered decoders (pgmi/decoder.py tensor names): values that keep the streams,
     decays and gates in an ordinary range, for benchmarks."""
     leaf = name.split(".", 1)[1] if name.startswith("l") else name
-    if leaf == "embed":
+    if leaf in ("embed", "bigram", "mlp.correction"):
         return 0.02, 0.0
+    if leaf == "canon1":
+        return 0.3, 0.0
     if "norm" in leaf:
         return 0.1, 1.0
     if leaf.startswith("hc"):
@@ -94,11 +96,31 @@ def decoder_policy(name: str, shape: tuple) -> "tuple[float, float]":
 
 
 def decoder_bench_config(size: str) -> dict:
-    """Tuvodra configurations with the layer sizes of real models, random weights ("2b": PaliGemma's text width,
-    feed-forward, attention width and vocabulary)."""
+    """Configurations with the layer sizes of real models, random weights: Tuvodra "1b", "2b" (PaliGemma's text width,
+    feed-forward, attention width and vocabulary), "7b"; "raritar-1b", ... : Raritar at the same widths, head counts,
+    windows and vocabularies."""
+    design, _, size = size.rpartition("-")
+    if design not in ("", "raritar"):
+        raise ValueError(f"unknown benchmark design '{design}'")
     w = {"1b": 1024, "2b": 2048, "7b": 4096}[size]
     heads, kv, ff, vocab, blocks = {"1b": (8, 2, 4096, 32768, 4), "2b": (16, 2, 16384, 257216, 4),
                                     "7b": (32, 8, 14336, 65536, 2)}[size]
+    if design == "raritar":
+        experts, expert_ff, shared_ff, n = {"1b": (28, 512, 1024, 8), "2b": (60, 1024, 4096, 8), "7b": (60, 2048, 8192, 4)}[size]
+        moe = {"kind": "moe", "expert": {"ff": expert_ff}, "shared": {"ff": shared_ff},
+               "router": {"experts": experts, "identity": 4, "top": 6, "groups": {"count": 4, "keep": 2}}}
+
+        def layer(i):
+            m = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 50.0,
+                 "mask": {"size": 1024, "keep_first": 16},
+                 "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+            if i > n // 2:
+                m["kv_from"] = n // 2
+            return {"type": "attention", "mixer": m, "mlp": moe}
+
+        return {"architecture": "Raritar", "vocab": vocab, "width": w, "canon": {"taps": 4}, "norm": {"eps": 1e-5},
+                "embedding": {"bigram": {"buckets": 65521, "mul_prev": 4099, "mul_cur": 257}}, "residual_mult": 0.5,
+                "layers": [layer(i) for i in range(n)]}
     mamba = {"type": "mamba1", "mixer": {"inner": 2 * w, "state": 16, "dt_rank": w // 16, "conv": 4}, "mlp": None}
     gru = {"type": "mingru", "mixer": {"width": w}, "mlp": None}
     attn = {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
