@@ -148,7 +148,7 @@ struct RouteArgs {
     int* cnt;
     int* list;
     int cap;
-    int* active;  // residual_route: active[0] (zero before the launch) experts are used, active[1 ..] which
+    int* active;  // residual_route: active[1 .. active[0]] are the experts used, -1: none (active[0] is zero before)
 };
 constexpr int kRouteRows = 16;  // most rows of residual_route and experts_skinny
 constexpr int kMaxExperts = 512;  // identity experts included: a workgroup's choice scores fit LDS

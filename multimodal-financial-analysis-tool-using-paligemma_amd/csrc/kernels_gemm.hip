@@ -991,11 +991,19 @@ __global__ void __launch_bounds__(64 * (NW + LW), 1) k_gemm_w(const uint16_t* __
 // cdna_hip_programming.md's 256^2 8-phase template, restated for this LDS image, with B0's
 // fragments kept in registers across the tile (one fewer fragment read per K-tile).
 // LDS rows are 128 B with the 16-B chunk XOR-swizzled by (row & 7) on the DMA's source address.
-template <int TM, int EPI, bool SPLIT>
-__global__ void __launch_bounds__(512, 1) k_gemm_8p(const uint16_t* __restrict__ A, int lda,
-                                                    const uint16_t* __restrict__ W, int ldw, int M, int N, int K,
-                                                    int kt_per_split, EpiArgs ea, float* __restrict__ ws, long up_off,
-                                                    int n_mt, int code) {
+//
+// G: which rows a tile is made of.  AllRows: consecutive rows of A, the XCD-aware tile order.  A grouped form
+// (G::kGrouped, no split) cuts the tiles out of row lists: tile(BM, BN) finds the workgroup's (false: none left) and
+// sets rows (of its list), m0, nt; weights() its matrix; source(m) the row of A behind list place m, target(m) the row
+// of the output.
+struct AllRows {
+    static constexpr bool kGrouped = false;
+};
+
+template <int TM, int EPI, bool SPLIT, class G>
+__device__ __forceinline__ void gemm_8p(const uint16_t* __restrict__ A, int lda, const uint16_t* __restrict__ W, int ldw, int M,
+                                        int N, int K, int kt_per_split, const EpiArgs& ea, float* __restrict__ ws, long up_off,
+                                        int n_mt, int code, G g) {
     static_assert(TM % 2 == 0, "row halves of whole 16-row tiles");
     constexpr bool DUAL = epi_dual(EPI);
     constexpr int H = TM / 2;                 // row tiles per quadrant
@@ -1010,9 +1018,19 @@ __global__ void __launch_bounds__(512, 1) k_gemm_8p(const uint16_t* __restrict__
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int wm = wave >> 2, wn = wave & 3;
-    int mt, nt, z;
-    xcd_tile(n_mt, code, mt, nt, z);
-    const int m0 = mt * BM, n0 = nt * (DUAL ? 128 : 256);
+    int m0, nt, z = 0;
+    if constexpr (G::kGrouped) {
+        if (!g.tile(BM, DUAL ? 128 : 256)) return;
+        M = g.rows;
+        m0 = g.m0;
+        nt = g.nt;
+        W = g.weights();
+    } else {
+        int mt;
+        xcd_tile(n_mt, code, mt, nt, z);
+        m0 = mt * BM;
+    }
+    const int n0 = nt * (DUAL ? 128 : 256);
     const int nkt_total = K / 64;
     const int kt0 = z * kt_per_split;
     const int kt1 = kt0 + kt_per_split < nkt_total ? kt0 + kt_per_split : nkt_total;
@@ -1037,6 +1055,7 @@ __global__ void __launch_bounds__(512, 1) k_gemm_8p(const uint16_t* __restrict__
         for (int qa = 0; qa < 2; ++qa) {
             int row = m0 + wr * 16 * TM + qa * 8 * TM + r;
             row = row < M ? row : M - 1;
+            if constexpr (G::kGrouped) row = g.source(row);
             sa[qa][i] = A + (long)row * lda + ((pch ^ (ir & 7)) << 3);
         }
     }
@@ -1188,7 +1207,29 @@ __global__ void __launch_bounds__(512, 1) k_gemm_8p(const uint16_t* __restrict__
             a0[i][jj] = acc[i][jj];
             a1[i][jj] = acc[i][2 + jj];
         }
-    if constexpr (SPLIT) {
+    if constexpr (G::kGrouped) {
+#pragma unroll
+        for (int i = 0; i < TM; ++i) {
+            int to[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int m = mb + i * 16 + (lane >> 4) * 4 + r;
+                to[r] = g.target(m < M ? m : M - 1);
+            }
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                if (mb + i * 16 + (lane >> 4) * 4 + r >= M) continue;
+                uint16_t* out = ea.out + (long)to[r] * ea.ldo;
+#pragma unroll
+                for (int j = 0; j < (DUAL ? 2 : 4); ++j) {  // columns N .. ldo-1: zeros
+                    const int n = n0 + wn * (DUAL ? 32 : 64) + j * 16 + (lane & 15);
+                    float v = acc[i][j][r];
+                    if constexpr (EPI == EPI_SWIGLU) v = v / (1.0f + __expf(-v)) * acc[i][2 + j][r];
+                    if (n < ea.ldo) out[n] = n < N ? f2bf(v) : 0;
+                }
+            }
+        }
+    } else if constexpr (SPLIT) {
 #pragma unroll
         for (int i = 0; i < TM; ++i)
 #pragma unroll
@@ -1206,6 +1247,14 @@ __global__ void __launch_bounds__(512, 1) k_gemm_8p(const uint16_t* __restrict__
         epi_tile<EPI, TM, 2>(ea, M, N, mb, n0 + wn * 64, lane, a0, a0);
         epi_tile<EPI, TM, 2>(ea, M, N, mb, n0 + wn * 64 + 32, lane, a1, a1);
     }
+}
+
+template <int TM, int EPI, bool SPLIT>
+__global__ void __launch_bounds__(512, 1) k_gemm_8p(const uint16_t* __restrict__ A, int lda,
+                                                    const uint16_t* __restrict__ W, int ldw, int M, int N, int K,
+                                                    int kt_per_split, EpiArgs ea, float* __restrict__ ws, long up_off,
+                                                    int n_mt, int code) {
+    gemm_8p<TM, EPI, SPLIT>(A, lda, W, ldw, M, N, K, kt_per_split, ea, ws, up_off, n_mt, code, AllRows{});
 }
 
 // (PGMI_GEMM_KERNELS_ONLY: the kernel templates alone -- kernels_matmul.hip instantiates its own few)

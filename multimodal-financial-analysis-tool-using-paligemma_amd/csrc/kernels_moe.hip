@@ -4,6 +4,7 @@
 //   k_route           a wave per row; entries are counted and listed per expert
 //   k_experts         bf16 MFMA, LDS-DMA ring with loader waves: row tiles of one expert's list, gathered by each
 //                     loader lane's own source address, results scattered to the entries' rows
+//   k_experts_8p      the same rows on the 8-phase 256 x 256 tiles of kernels_gemm.hip, for long lists
 //   k_experts_f32     the same product on fp32 FMA tiles
 //   k_experts_skinny  few rows: one workgroup per (16 outputs, used expert), MFMA straight from HBM
 #define PGMI_GEMM_KERNELS_ONLY
@@ -104,9 +105,11 @@ long max_tiles(const ExpertArgs& a, int BM) { return a.entries / BM + std::min(a
 // ---------------------------------------------------------------- bf16
 // BM = 32 TM rows x BN = 64 (gate and up: 64 + 64) or 128 columns x 64 deep; 8 compute waves in a 2 x 4 grid, 4 loader
 // waves, ST ring slots.  The ring, its LDS image and the fragment schedule are k_gemm_w's.
+constexpr int ring_slots(int TM) { return TM <= 2 ? 3 : 4; }  // small tiles: two workgroups per CU
+
 template <int TM, int MODE>
 __global__ void __launch_bounds__(64 * 12, 1) k_experts(ExpertArgs a) {
-    constexpr int NW = 8, LW = 4, WM = 2, WN = 4, NB = MODE == EX_SWIGLU ? 2 : 1, TN = MODE == EX_SWIGLU ? 1 : 2, ST = 4;
+    constexpr int NW = 8, LW = 4, WM = 2, WN = 4, NB = MODE == EX_SWIGLU ? 2 : 1, TN = MODE == EX_SWIGLU ? 1 : 2, ST = ring_slots(TM);
     constexpr int BM = WM * TM * 16, BN = WN * TN * 16;
     constexpr int APC = BM / 8, PCS = APC + NB * BN / 8, GPW = (PCS + LW - 1) / LW;
     constexpr int ABYTES = BM * 128, SBYTES = (BM + NB * BN) * 128;
@@ -240,7 +243,7 @@ __global__ void __launch_bounds__(64 * 12, 1) k_experts(ExpertArgs a) {
 template <int TM, int MODE>
 void run_experts(hipStream_t s, const ExpertArgs& a) {
     constexpr int BM = 32 * TM, BN = MODE == EX_SWIGLU ? 64 : 128;
-    constexpr size_t lds = (size_t)4 * (BM + 128) * 128;
+    constexpr size_t lds = (size_t)ring_slots(TM) * (BM + 128) * 128;
     static bool done = false;
     if (!done && lds > 64 * 1024) {
         (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&k_experts<TM, MODE>),
@@ -250,6 +253,51 @@ void run_experts(hipStream_t s, const ExpertArgs& a) {
     const int n_nt = (a.N + BN - 1) / BN;
     // a run of one XCD is up to one tile longer than total / 8
     hipLaunchKernelGGL((k_experts<TM, MODE>), dim3((unsigned)((max_tiles(a, BM) * n_nt + 7) / 8 * 8)), dim3(64 * 12), lds, s, a);
+}
+
+// the row lists of gemm_8p's tiles
+struct ExpertRows {
+    static constexpr bool kGrouped = true;
+    const ExpertArgs& a;
+    const int* list = nullptr;
+    int e = 0, rows = 0, m0 = 0, nt = 0;
+    __device__ __forceinline__ explicit ExpertRows(const ExpertArgs& x) : a(x) {}
+    __device__ __forceinline__ bool tile(int BM, int BN) {
+        const TileAt t = find_tile(a.cnt, a.experts, BM, (a.N + BN - 1) / BN);
+        e = t.e;
+        rows = t.cnt;
+        m0 = t.m0;
+        nt = t.nt;
+        list = a.list + (long)e * a.cap;
+        return e >= 0;
+    }
+    __device__ __forceinline__ const uint16_t* weights() const { return a.W + e * a.wstride; }
+    __device__ __forceinline__ int source(int m) const { return list[m] / a.gather; }
+    __device__ __forceinline__ int target(int m) const { return list[m]; }
+};
+
+template <int TM, int MODE>
+__global__ void __launch_bounds__(512, 1) k_experts_8p(ExpertArgs a) {
+    EpiArgs ea;
+    ea.out = reinterpret_cast<uint16_t*>(a.out);
+    ea.ldo = a.ldo;
+    gemm_8p<TM, MODE == EX_SWIGLU ? EPI_SWIGLU : EPI_STORE, false>(reinterpret_cast<const uint16_t*>(a.A), a.lda, a.W, a.ldw, 0,
+                                                                  a.N, a.K, a.K / 64, ea, nullptr, (long)a.N * a.ldw, 0, 0,
+                                                                  ExpertRows(a));
+}
+
+template <int TM, int MODE>
+void run_experts_8p(hipStream_t s, const ExpertArgs& a) {
+    constexpr int BM = 32 * TM, BN = MODE == EX_SWIGLU ? 128 : 256;
+    constexpr size_t lds = (size_t)2 * (2 * 16 * TM * 128 + 2 * 128 * 128);
+    static bool done = false;
+    if (!done) {
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&k_experts_8p<TM, MODE>),
+                                  hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        done = true;
+    }
+    const int n_nt = (a.N + BN - 1) / BN;
+    hipLaunchKernelGGL((k_experts_8p<TM, MODE>), dim3((unsigned)((max_tiles(a, BM) * n_nt + 7) / 8 * 8)), dim3(512), lds, s, a);
 }
 
 // ---------------------------------------------------------------- fp32
@@ -302,13 +350,15 @@ __global__ void __launch_bounds__(256) k_experts_f32(ExpertArgs a) {
 // ---------------------------------------------------------------- few rows
 // grid (output tiles of 16, 1 + used experts): y == 0 is the shared expert, y > 0 the (y - 1)-th used one, whose rows are
 // its list.  4 waves split K; a lane reads 32 contiguous bytes of its weight row per 64-deep step, as k_skinny.
-template <int MODE>
+// U: 64-deep steps a wave has in flight.
+template <int MODE, int U>
 __global__ void __launch_bounds__(256) k_experts_skinny(ExpertArgs a) {
-    constexpr int NM = MODE == EX_SWIGLU ? 2 : 1, U = 8 / NM;
+    constexpr int NM = MODE == EX_SWIGLU ? 2 : 1;
     __shared__ float sums[4][NM][16][17];
     const bool shared = blockIdx.y == 0;
     if (shared ? !a.Wsh : (int)blockIdx.y > a.active[0]) return;
     const int e = shared ? 0 : a.active[blockIdx.y];
+    if (e < 0) return;
     const int N = shared ? a.Nsh : a.N, K = shared ? a.Ksh : a.K, ldw = shared ? a.ldwsh : a.ldw, n0 = blockIdx.x * 16;
     const int ldo = shared ? a.ldosh : a.ldo;
     if (n0 >= ldo) return;
@@ -393,22 +443,28 @@ void experts_rt(hipStream_t s, Act act, ExpertMode mode, const ExpertArgs& a) {
         return;
     }
     const int per = a.entries / std::max(1, a.experts);  // rows of an average expert
-    if (mode == EX_SWIGLU) {
-        if (per > 96) run_experts<4, EX_SWIGLU>(s, a);
-        else if (per > 32) run_experts<2, EX_SWIGLU>(s, a);
-        else run_experts<1, EX_SWIGLU>(s, a);
-    } else {
-        if (per > 96) run_experts<4, EX_STORE>(s, a);
-        else if (per > 32) run_experts<2, EX_STORE>(s, a);
-        else run_experts<1, EX_STORE>(s, a);
-    }
+    auto go = [&](auto mode_c) {
+        constexpr int MODE = decltype(mode_c)::value;
+        const bool p8 = a.K % 64 == 0 && a.K >= 512;
+        if (p8 && per > 384) run_experts_8p<8, MODE>(s, a);
+        else if (p8 && per > 128) run_experts_8p<6, MODE>(s, a);
+        else if (per > 96) run_experts<4, MODE>(s, a);
+        else if (per > 32) run_experts<2, MODE>(s, a);
+        else run_experts<1, MODE>(s, a);
+    };
+    if (mode == EX_SWIGLU) go(std::integral_constant<int, EX_SWIGLU>{});
+    else go(std::integral_constant<int, EX_STORE>{});
 }
 
 void experts_skinny(hipStream_t s, ExpertMode mode, const ExpertArgs& a) {
     const int n = std::max(a.ldo, a.Wsh ? a.ldosh : 0);
-    const dim3 grid((n + 15) / 16, 1 + std::min(a.experts, a.entries));
-    if (mode == EX_SWIGLU) hipLaunchKernelGGL((k_experts_skinny<EX_SWIGLU>), grid, dim3(256), 0, s, a);
-    else hipLaunchKernelGGL((k_experts_skinny<EX_STORE>), grid, dim3(256), 0, s, a);
+    // one row lists its choices by place, identities included
+    const dim3 grid((n + 15) / 16, 1 + (a.B == 1 ? a.entries : std::min(a.experts, a.entries)));
+    // one row has too few workgroups to cover the memory's latency with four steps: 25.0 -> 20.5 us (width 2048, 6 + 1
+    // experts); with more rows, or the shorter rows of the down product, eight are slower
+    if (mode == EX_SWIGLU && a.B == 1) hipLaunchKernelGGL((k_experts_skinny<EX_SWIGLU, 8>), grid, dim3(256), 0, s, a);
+    else if (mode == EX_SWIGLU) hipLaunchKernelGGL((k_experts_skinny<EX_SWIGLU, 4>), grid, dim3(256), 0, s, a);
+    else hipLaunchKernelGGL((k_experts_skinny<EX_STORE, 4>), grid, dim3(256), 0, s, a);
 }
 
 }  // namespace pgmi

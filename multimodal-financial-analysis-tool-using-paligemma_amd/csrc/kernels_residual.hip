@@ -29,12 +29,13 @@ struct RouterArgs {
 
 // One workgroup per row; PC pieces of V elements per thread, every load of a source issued before its first use.
 // RT: the router of the row and its choice behind the norm, 16 waves; dynamic LDS: route_words(), then h [ldh].
-template <typename T, int V, int PC, bool RT>
+// KT > 0: the input convolution's step with KT taps, its operands loaded ahead of the norm (0: any number, or none).
+template <typename T, int V, int PC, bool RT, int KT>
 __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt) {
     __shared__ float red[16];
     extern __shared__ __attribute__((aligned(16))) float rsm[];
     constexpr int RR = 4, RK = 4;  // router rows and 512-wide steps a wave has in flight
-    const int rows_r = RT ? rt.r.n + (rt.r.gate != nullptr) : 0;
+    const int rows_r = RT ? rt.r.n : 0;
     uint4 rw[RT ? RR : 1][RT ? RK : 1];
     auto rload = [&](int n0, int k0) {
         if constexpr (RT) {
@@ -65,6 +66,31 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
         dd[i] = ok[i] ? d : 0;
     }
     int slot = 0, pos = 0;
+    if (!a.seqs && a.slot) {
+        slot = a.slot[row];
+        pos = a.pos[row];
+    }
+    float* ring = a.taps > 0 ? a.ring + (long)slot * a.taps * D : nullptr;
+    float wk[KT > 0 ? KT : 1][PC][V], back[KT > 1 ? KT - 1 : 1][PC][V];  // back[j]: the norm j + 1 positions ago
+    if constexpr (KT > 0) {
+#pragma unroll
+        for (int i = 0; i < PC; ++i) {
+#pragma unroll
+            for (int v = 0; v < V; ++v)
+#pragma unroll
+                for (int j = 0; j < KT; ++j) wk[j][i][v] = bf2f(a.cw[(long)(dd[i] + v) * KT + j]);
+#pragma unroll
+            for (int j = 0; j < KT - 1; ++j) {
+                const int p = pos - 1 - j;
+                ldv(ring + (long)((p < 0 ? 0 : p) % KT) * D + dd[i], back[j][i]);
+#pragma unroll
+                for (int v = 0; v < V; ++v) back[j][i][v] = p < 0 ? 0.0f : back[j][i][v];
+            }
+        }
+    }
+    float gw[V];  // the gate's row of the router
+#pragma unroll
+    for (int v = 0; v < V; ++v) gw[v] = RT && rt.r.gate && ok[0] ? bf2f(rt.W[(long)rt.r.n * rt.ldw + dd[0] + v]) : 0.0f;
     if (a.ids) {
         long id = a.ids[row];
         id = id < 0 ? 0 : (id >= a.vocab ? a.vocab - 1 : id);
@@ -82,9 +108,6 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
                 slot = q.slot;
                 pos = q.start + row - q.off;
                 here = row > q.off;
-            } else {
-                slot = a.slot[row];
-                pos = a.pos[row];
             }
             int* hist = a.history + (long)slot * a.max_tokens + pos;
             long p = a.buckets;
@@ -114,7 +137,7 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
 #pragma unroll
             for (int v = 0; v < V; ++v) y[i][v] = 0.0f;
         if (a.y) {
-#pragma unroll 4
+#pragma unroll(PC == 1 ? 4 : 1)
             for (int z = 0; z < a.ysplit; ++z) {
                 const float* yr = a.y + (long)z * a.ystride + (long)row * D;
 #pragma unroll
@@ -136,18 +159,29 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
                     for (int v = 0; v < V; ++v) y[i][v] *= g;
             }
             const T* hr = reinterpret_cast<const T*>(m.h) + (long)row * m.ldh;
-#pragma unroll 4
+            const long e0 = (long)row * m.top;
+            // every entry's row is read and dropped where an identity was chosen (it holds nothing then): no load waits
+            // for the choice
+            float self = 0.0f;
+#pragma unroll(PC == 1 ? 8 : 1)
             for (int k = 0; k < m.top; ++k) {
-                const long e = (long)row * m.top + k;
-                const T* yr = m.sel[e] < m.experts ? reinterpret_cast<const T*>(m.y) + e * m.ldy : hr;
-                const float w = m.w[e];
+                const bool real = m.sel[e0 + k] < m.experts;
+                const float w = m.w[e0 + k];
+                self += real ? 0.0f : w;
 #pragma unroll
                 for (int i = 0; i < PC; ++i) {
                     float q[V];
-                    ldv(yr + dd[i], q);
+                    ldv(reinterpret_cast<const T*>(m.y) + (e0 + k) * m.ldy + dd[i], q);
 #pragma unroll
-                    for (int v = 0; v < V; ++v) y[i][v] = fmaf(w, q[v], y[i][v]);
+                    for (int v = 0; v < V; ++v) y[i][v] = real ? fmaf(w, q[v], y[i][v]) : y[i][v];
                 }
+            }
+#pragma unroll
+            for (int i = 0; i < PC; ++i) {
+                float q[V];
+                ldv(hr + dd[i], q);
+#pragma unroll
+                for (int v = 0; v < V; ++v) y[i][v] = fmaf(self, q[v], y[i][v]);
             }
         }
 #pragma unroll
@@ -176,19 +210,22 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
     T* h = reinterpret_cast<T*>(a.h) + (long)blockIdx.x * a.ldh;
     T* hs = reinterpret_cast<T*>(rsm + (RT ? route_words(rt.r.n, rt.r.groups) : 0));
     const float g = a.w_scalar ? bf2f(a.w[0]) : 0.0f;
-    float* ring = nullptr;
-    if (a.taps > 0) {
-        slot = a.slot[row];
-        pos = a.pos[row];
-        ring = a.ring + (long)slot * a.taps * D;
-    }
+    float part = 0.0f;  // of the gate
 #pragma unroll
     for (int i = 0; i < PC; ++i) {
         if (!ok[i]) continue;
         float n[V], o[V];
 #pragma unroll
         for (int v = 0; v < V; ++v) o[v] = n[v] = x[i][v] * inv * (a.w_scalar ? g : bf2f(a.w[dd[i] + v]));
-        if (a.taps > 0) {
+        if constexpr (KT > 0) {
+#pragma unroll
+            for (int v = 0; v < V; ++v) {
+                o[v] = fmaf(wk[KT - 1][i][v], n[v], o[v]);
+#pragma unroll
+                for (int j = 0; j < KT - 1; ++j) o[v] = fmaf(wk[KT - 2 - j][i][v], back[j][i][v], o[v]);
+            }
+            if (KT > 1) stv(ring + (long)(pos % KT) * D + dd[i], n);
+        } else if (a.taps > 0) {
             const uint16_t* cw = a.cw + (long)dd[i] * a.taps;
             for (int j = 0; j < a.taps && j <= pos; ++j) {
                 float q[V];
@@ -204,7 +241,11 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
             if (a.taps > 1) stv(ring + (long)(pos % a.taps) * D + dd[i], n);
         }
         stv(h + dd[i], o);
-        if constexpr (RT) stv(hs + dd[i], o);
+        if constexpr (RT) {
+            stv(hs + dd[i], o);
+#pragma unroll
+            for (int v = 0; v < V; ++v) part = fmaf(gw[v], rbf(o[v]), part);
+        }
     }
     for (int d = D + tid; d < a.ldh; d += NT) {
         stf(h + d, 0.0f);
@@ -214,7 +255,9 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
         const RouteArgs& r = rt.r;
         const int lane = tid & 63, wave = tid >> 6;
         float* z = rsm;
-        __shared__ float gate;
+        __shared__ float gate[16];
+        part = wave_sum(part);
+        if (lane == 0) gate[wave] = part;
         __syncthreads();
         for (int n0 = wave; n0 < rows_r; n0 += 16 * RR) {
             float acc[RR] = {};
@@ -232,19 +275,29 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
             for (int q = 0; q < RR; ++q) acc[q] = wave_sum(acc[q]);
 #pragma unroll
             for (int q = 0; q < RR; ++q)
-                if (lane == 0 && n0 + 16 * q < rows_r) {
-                    if (n0 + 16 * q < r.n) z[n0 + 16 * q] = acc[q];
-                    else gate = acc[q];
-                }
+                if (lane == 0 && n0 + 16 * q < rows_r) z[n0 + 16 * q] = acc[q];
         }
         __syncthreads();
         if (wave > 0) return;
-        if (lane == 0 && r.gate) r.gate[row] = 1.0f / (1.0f + expf(-gate));
+        if (r.gate) {
+            part = 0.0f;
+#pragma unroll
+            for (int w = 0; w < 16; ++w) part += gate[w];
+            if (lane == 0) r.gate[row] = 1.0f / (1.0f + expf(-part));
+        }
+        const bool alone = a.rows == 1;  // nobody else counts: the used experts by place, -1 for an identity
+        if (alone && lane == 0) r.active[0] = r.top;
         route_row(z, r.correction, r.n, r.groups, r.keep, r.top, lane, [&](int k, int e, float w) {
             const int at = row * r.top + k;
             r.sel[at] = e;
             r.w[at] = w;
-            if (e < r.experts) {
+            if (alone) {
+                r.active[1 + k] = e < r.experts ? e : -1;
+                if (e < r.experts) {
+                    r.cnt[e] = 1;
+                    r.list[(long)e * r.cap] = at;
+                }
+            } else if (e < r.experts) {
                 const int m = atomicAdd(&r.cnt[e], 1);
                 r.list[(long)e * r.cap + m] = at;
                 if (m == 0) r.active[1 + atomicAdd(&r.active[0], 1)] = e;
@@ -259,10 +312,18 @@ void residual_t(hipStream_t s, const ResidualArgs& a) {
         const int threads = std::min(1024, (a.D / v + 63) / 64 * 64);
         hipLaunchKernelGGL(kern, dim3(a.rows), dim3(std::max(64, threads)), 0, s, a, RouterArgs{});
     };
-    if (a.D % 4 == 0 && a.D <= 4096) go(k_residual<T, 4, 1, false>, 4);
-    else if (a.D % 4 == 0) go(k_residual<T, 4, 4, false>, 4);
-    else if (a.D <= 1024) go(k_residual<T, 1, 1, false>, 1);
-    else go(k_residual<T, 1, 16, false>, 1);
+    if (a.D % 4 == 0 && a.D <= 4096) {
+        if (a.taps == 4) go(k_residual<T, 4, 1, false, 4>, 4);
+        else if (a.taps == 3) go(k_residual<T, 4, 1, false, 3>, 4);
+        else if (a.taps == 2) go(k_residual<T, 4, 1, false, 2>, 4);
+        else go(k_residual<T, 4, 1, false, 0>, 4);
+    } else if (a.D % 4 == 0) {
+        go(k_residual<T, 4, 4, false, 0>, 4);
+    } else if (a.D <= 1024) {
+        go(k_residual<T, 1, 1, false, 0>, 1);
+    } else {
+        go(k_residual<T, 1, 16, false, 0>, 1);
+    }
 }
 
 // ---------------------------------------------------------------- input convolution
@@ -377,7 +438,7 @@ bool residual_route_fits(Act act, int rows, int D) {
 
 void residual_route(hipStream_t s, const ResidualArgs& a, const uint16_t* W, int ldw, const RouteArgs& r) {
     const size_t lds = (size_t)route_words(r.n, r.groups) * sizeof(float) + (size_t)a.ldh * sizeof(uint16_t);
-    hipLaunchKernelGGL((k_residual<uint16_t, 4, 1, true>), dim3(a.rows), dim3(1024), lds, s, a, RouterArgs{W, ldw, r});
+    hipLaunchKernelGGL((k_residual<uint16_t, 4, 1, true, 0>), dim3(a.rows), dim3(1024), lds, s, a, RouterArgs{W, ldw, r});
 }
 
 void canon(hipStream_t s, Act act, const CanonArgs& a) {

@@ -259,11 +259,12 @@ def test_rotation_far_from_the_start(dtype):
 
 # ---------------------------------------------------------------- mixture of experts
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("mlp", [C.moe(4, 24, 2, 40), C.moe(12, 72, 3, 16, identity=4, groups=(4, 2)), C.moe(3, 136, 3, 8),
-                                 C.moe(90, 16, 4, 8, identity=6, groups=(3, 2))])
-def test_long_expert_lists(mlp, dtype):
+@pytest.mark.parametrize("width,mlp", [
+    (104, C.moe(4, 24, 2, 40)), (104, C.moe(12, 72, 3, 16, identity=4, groups=(4, 2))), (104, C.moe(3, 136, 3, 8)),
+    (104, C.moe(70, 16, 4, 8, identity=5, groups=(3, 2))), (576, C.moe(3, 512, 2, 24)), (512, C.moe(4, 520, 2, 16, identity=1))])
+def test_long_expert_lists(width, mlp, dtype):
     """Hundreds of rows per expert and few: every row tile, in one step and in portions."""
-    cfg = C.model([C.layer(2, 1, 16, 24, 30, keep=1, mlp=mlp)], width=104)
+    cfg = C.model([C.layer(2, 1, 16, 24, 30, keep=1, mlp=mlp)], width=width)
     eng, W = build(cfg, dtype)
     toks = tokens(cfg, 700, 61)
     want = R.run(cfg, W, toks)
