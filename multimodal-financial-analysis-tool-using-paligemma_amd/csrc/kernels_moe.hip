@@ -43,7 +43,7 @@ __global__ void __launch_bounds__(1024) k_route(RouteArgs a) {
         for (int c = lane; c < n; c += 64) sc[c] = logit(c);
         if (a.gate && lane == 0) a.gate[row] = 1.0f / (1.0f + expf(-logit(n)));
         wave_sync();
-        route_row(sc, a.correction, n, a.groups, a.keep, a.top, lane, [&](int k, int e, float w) {
+        route_row(sc, [&](int c) { return bf2f(a.correction[c]); }, n, a.groups, a.keep, a.top, lane, [&](int k, int e, float w) {
             const long at = (long)row * a.top + k;
             a.sel[at] = e;
             a.w[at] = w;

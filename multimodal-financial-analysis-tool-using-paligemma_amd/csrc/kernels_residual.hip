@@ -50,7 +50,6 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
             }
         }
     };
-    rload(threadIdx.x >> 6, 0);  // in flight during the update and the norm
     const int tid = threadIdx.x, NT = blockDim.x, D = a.D;
     const int row = a.rows_idx ? a.rows_idx[blockIdx.x] : blockIdx.x;
     if (a.zero && blockIdx.x == 0)
@@ -189,6 +188,8 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
 #pragma unroll
             for (int v = 0; v < V; ++v) x[i][v] = fmaf(a.mult, y[i][v], x[i][v]);
     }
+    rload(tid >> 6, 0);  // in flight during the norm (loads return in order: not ahead of the update's)
+    const float corr = RT ? bf2f(rt.r.correction[min(tid & 63, rt.r.n - 1)]) : 0.0f;
     float ss = 0.0f;
 #pragma unroll
     for (int i = 0; i < PC; ++i) {
@@ -287,7 +288,7 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
         }
         const bool alone = a.rows == 1;  // nobody else counts: the used experts by place, -1 for an identity
         if (alone && lane == 0) r.active[0] = r.top;
-        route_row(z, r.correction, r.n, r.groups, r.keep, r.top, lane, [&](int k, int e, float w) {
+        route_row(z, [&](int c) { return c < 64 ? corr : bf2f(r.correction[c]); }, r.n, r.groups, r.keep, r.top, lane, [&](int k, int e, float w) {
             const int at = row * r.top + k;
             r.sel[at] = e;
             r.w[at] = w;

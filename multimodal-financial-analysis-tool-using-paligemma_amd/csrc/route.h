@@ -20,13 +20,12 @@ __device__ __forceinline__ uint32_t order_key(float f) {
 // LDS words of one row: scores, choice keys (padded to 4), group keys
 __host__ __device__ inline int route_words(int n, int groups) { return 2 * ((n + 3) & ~3) + ((groups + 3) & ~3); }
 
-// sc[0 .. n) holds the row's logits and receives their softmax; choice = score + correction.  A group's key is its largest
+// sc[0 .. n) holds the row's logits and receives their softmax; choice = score + correction(expert).  A group's key is its largest
 // choice; experts outside the `keep` best groups cannot be chosen.  The place of an expert is the number of those before
 // it (larger choice, or equal and a smaller index), so exactly `top` places 0 .. top-1 are taken, each by one lane:
 // take(place, expert, score).
-template <typename F>
-__device__ __forceinline__ void route_row(float* sc, const uint16_t* correction, int n, int groups, int keep, int top, int lane,
-                                          F take) {
+template <typename C, typename F>
+__device__ __forceinline__ void route_row(float* sc, C correction, int n, int groups, int keep, int top, int lane, F take) {
     const int np = (n + 3) & ~3, gs = n / groups;
     uint32_t* key = reinterpret_cast<uint32_t*>(sc + np);
     uint32_t* gr = key + np;
@@ -48,7 +47,7 @@ __device__ __forceinline__ void route_row(float* sc, const uint16_t* correction,
         if (c < n) {
             const float s = sc[c] * inv;
             sc[c] = s;
-            k = order_key(s + bf2f(correction[c]));
+            k = order_key(s + correction(c));
             if (limited) atomicMax(&gr[c / gs], k);
         }
         key[c] = k;
