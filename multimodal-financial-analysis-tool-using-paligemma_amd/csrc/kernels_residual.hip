@@ -160,19 +160,26 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
             const T* hr = reinterpret_cast<const T*>(m.h) + (long)row * m.ldh;
             const long e0 = (long)row * m.top;
             // every entry's row is read and dropped where an identity was chosen (it holds nothing then): no load waits
-            // for the choice
+            // for the choice; KB rows in flight together
+            constexpr int KB = PC == 1 ? 8 : 1;
             float self = 0.0f;
-#pragma unroll(PC == 1 ? 8 : 1)
-            for (int k = 0; k < m.top; ++k) {
-                const bool real = m.sel[e0 + k] < m.experts;
-                const float w = m.w[e0 + k];
-                self += real ? 0.0f : w;
+            for (int k0 = 0; k0 < m.top; k0 += KB) {
+                float q[KB][PC][V];
 #pragma unroll
-                for (int i = 0; i < PC; ++i) {
-                    float q[V];
-                    ldv(reinterpret_cast<const T*>(m.y) + (e0 + k) * m.ldy + dd[i], q);
+                for (int j = 0; j < KB; ++j)
 #pragma unroll
-                    for (int v = 0; v < V; ++v) y[i][v] = real ? fmaf(w, q[v], y[i][v]) : y[i][v];
+                    for (int i = 0; i < PC; ++i)
+                        ldv(reinterpret_cast<const T*>(m.y) + (e0 + min(k0 + j, m.top - 1)) * m.ldy + dd[i], q[j][i]);
+#pragma unroll
+                for (int j = 0; j < KB; ++j) {
+                    const long e = e0 + min(k0 + j, m.top - 1);
+                    const float w = k0 + j < m.top ? m.w[e] : 0.0f;
+                    const bool real = m.sel[e] < m.experts && k0 + j < m.top;
+                    self += real ? 0.0f : w;
+#pragma unroll
+                    for (int i = 0; i < PC; ++i)
+#pragma unroll
+                        for (int v = 0; v < V; ++v) y[i][v] = real ? fmaf(w, q[j][i][v], y[i][v]) : y[i][v];
                 }
             }
 #pragma unroll
