@@ -1,7 +1,7 @@
 // engine_decoder.hip -- the layered-decoder family of libpgmi: a text model described as a list of layers, each a
-// mixer and an optional feed-forward, around residual streams or one plain residual.  Weight layout, derived tensors, the per-sequence
-// state slab, the ragged forward (prompts and portions of prompts) and the decode step (hipGraph-replayed), over
-// the mechanisms of decoder.h.  A design is its layer list and constants; nothing here names one.
+// mixer and an optional feed-forward, around residual streams or one plain residual.  Weight layout, derived
+// tensors, the per-sequence state slab, the ragged forward (prompts and portions of prompts) and the decode step
+// (hipGraph-replayed), over the mechanisms of decoder.h.  A design is its layer list and constants; nothing here names one.
 #include <set>
 
 #include "decoder.h"

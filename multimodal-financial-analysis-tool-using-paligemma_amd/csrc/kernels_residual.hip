@@ -295,7 +295,8 @@ __global__ void __launch_bounds__(1024) k_residual(ResidualArgs a, RouterArgs rt
         }
         const bool alone = a.rows == 1;  // nobody else counts: the used experts by place, -1 for an identity
         if (alone && lane == 0) r.active[0] = r.top;
-        route_row(z, [&](int c) { return c < 64 ? corr : bf2f(r.correction[c]); }, r.n, r.groups, r.keep, r.top, lane, [&](int k, int e, float w) {
+        const auto correction = [&](int c) { return c < 64 ? corr : bf2f(r.correction[c]); };
+        route_row(z, correction, r.n, r.groups, r.keep, r.top, lane, [&](int k, int e, float w) {
             const int at = row * r.top + k;
             r.sel[at] = e;
             r.w[at] = w;

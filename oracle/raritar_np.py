@@ -1,4 +1,4 @@
-"""oracle/raritar_np.py -- TEST INFRASTRUCTURE ONLY (checker side, never the product).
+"""oracle/raritar_np.py -- TEST INFRASTRUCTURE ONLY (never the product).
 
 Plain, slow restatement (numpy, float64) of Raritar, one function per mechanism, token by token, sharing no code with
 the product: one residual stream with a scaled update, one-number RMS norms, a short causal convolution added to what
